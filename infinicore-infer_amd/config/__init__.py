@@ -7,10 +7,11 @@ from .fopezen import FopezenConfig
 from .mezinex import MezinexConfig
 from .daborax import DaboraxConfig
 from .fizelix import FizelixConfig
+from .pekarax import PekaraxConfig
 
 __all__ = [
     "ConfigError", "config_from_dict", "config_from_dir", "read_config_json",
     "register_architecture", "registered_architectures", "resolve_architecture",
     "ExecEntry", "LayerSpec", "ModelSpec", "PartSpec", "default_schedule",
-    "MiniCPMConfig", "RopeScaling", "FopezenConfig", "MezinexConfig", "DaboraxConfig", "FizelixConfig",
+    "MiniCPMConfig", "RopeScaling", "FopezenConfig", "MezinexConfig", "DaboraxConfig", "FizelixConfig", "PekaraxConfig",
 ]

@@ -167,15 +167,26 @@ int ic_attn_pooled_prefill_supported(int dtype, int dk, int dv);
 int ic_attn_pooled_prefill(const void* q, int q_stride, void* out, int out_stride, int dtype, const void* kcache, const void* vcache, const void* kpool, const void* vpool, const int* block_tables, int bt_stride, const int* pool_tables, int pt_stride, const int* tiles, int n_tiles, const float* bias, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int P, hipStream_t stream);
 
 // ---- moe.hip: routed experts --------------------------------------------------------------------------------------
-int ic_moe_route(const float* z, int z_stride, int T, int E, int top, int mode, int renorm, int* ids, float* weights, hipStream_t stream);
+int ic_moe_route(const float* z, int z_stride, int T, int E, int top, int mode, int renorm, const float* correction, int groups, int group_keep, float scale, int* ids, float* weights, hipStream_t stream);
 int ic_moe_sort(const int* ids, int n, int E, int* offsets, int* order, int* place, hipStream_t stream);
 int ic_moe_gather(const void* h, int h_stride, int dtype, const int* order, const float* weights, int n, int top, int d, void* out, hipStream_t stream);
-int ic_moe_expert_product(const void* a, int a_stride, const void* w, long long w_expert_stride, int dtype, const int* offsets, void* out, int out_stride, int E, int N, int K, int glu, int compute_units, hipStream_t stream);
-int ic_moe_combine(const void* y, int y_stride, int dtype, const int* place, const float* weights, const void* shared, int shared_stride, int T, int top, int d, void* out, int out_stride, hipStream_t stream);
+int ic_moe_expert_product(const void* a, int a_stride, const void* w, long long w_expert_stride, int dtype, const int* offsets, void* out, int out_stride, int E, int N, int K, int glu, float limit, float slope, int compute_units, hipStream_t stream);
+int ic_moe_combine(const void* y, int y_stride, int dtype, const int* place, const float* weights, const void* shared, int shared_stride, const void* own, int own_stride, const int* n_routed, int T, int top, int d, void* out, int out_stride, hipStream_t stream);
 
 // ---- stream_rows.hip: a gate on a sublayer's result, a gate on a slice of a token table -----------------------------------
 int ic_gated_norm_into_stream(const void* y, const void* g, int g_stride, int y_dtype, const float* gb, const float* w, float* x, void* copy, int copy_dtype, int T, int d, float eps, hipStream_t stream);
 int ic_token_gate(const void* z, int z_stride, const void* table, int table_stride, int dtype, const int* tokens, int col0, int n, void* out, int T, hipStream_t stream);
+
+// Queries, keys and values through a short convolution, a rotation of halves and a norm per head, into the cache.
+int ic_conv_rope_norm_store(const void* rows, int row_stride, int dtype, const float* cw, int taps, const int* positions, const float* freq, int rot_dims, const float* qw, const float* kw, int norm, float eps, void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh, int nkvh, int dk, int dv, int page_size, float* state, long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int R, int single, hipStream_t stream);
+// x = rmsnorm(alpha x + sa ya + sb yb) * w, the norm on the sum; copy: the new x in the results' dtype.
+int ic_sum_norm(const void* ya, float sa, const void* yb, float sb, int dtype, float alpha, const float* w, float* x, void* copy, int T, int d, float eps, hipStream_t stream);
+
+// ---- matrix_memory.hip: recurrences with a matrix state per head, decays per key channel or per head, the delta rule --------
+int ic_delta_prep(const void* rows, int row_stride, int dtype, const float* w, int taps, const void* b, int b_stride, float* out, float* beta, int G, int H, int dk, int dv, float unit_eps, float* state, long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int T, int R, int single, hipStream_t stream);
+int ic_memory_gates(const float* z, int z_stride, const float* bi, const float* bf, float cap, int H, float* keep, float* add, float* floor_, float* state, long long state_stride, const int* req_start, const int* state_slots, int R, hipStream_t stream);
+int ic_matrix_memory(const void* q, int q_stride, const void* k, int k_stride, const void* v, int v_stride, int dtype, const float* decay, int per_channel, const float* scale, int delta, int H, int per, int dk, int dv, float q_scale, float* out, float* extra_out, float* state, long long state_stride, const int* req_start, const int* state_slots, int R, int single, int columns_a_thread, hipStream_t stream);
+int ic_gated_head_norm(const float* y, const float* num, const float* floor_, const void* z, int z_stride, int dtype, const float* w, int w_shared, int T, int H, int dv, float eps, void* out, int gate, hipStream_t stream);
 
 // ---- sampling.hip -----------------------------------------------------------------------------------
 // Greedy choice per row; scratch_val / scratch_idx: 64 * n_rows elements.

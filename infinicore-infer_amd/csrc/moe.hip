@@ -1,7 +1,9 @@
 // A feed-forward of routed experts.  A token's router logits z[E] (float32) give scores s = sigmoid(z) (or, for
 // another design, a softmax over the experts); the `top` experts with the largest scores are chosen (the lower
 // index wins a tie), their weights are the scores, optionally renormalised over the chosen ones.  A (token,
-// choice) pair is numbered token * top + choice.
+// choice) pair is numbered token * top + choice.  Options of the choice: a correction per expert that is added to the scores
+// for the choice alone; groups of neighbouring experts, of which only the best few (by their best corrected score) may be
+// chosen from; identity experts behind the others, whose result is the token's own input.
 //
 //   * ic_moe_route: scores, choice and weights of every token,
 //   * ic_moe_sort: the pairs in expert order (stable): offsets[E + 1], order[n] (sorted place -> pair),
@@ -9,9 +11,10 @@
 //   * ic_moe_gather: the sorted pairs' input rows, each multiplied by its weight (a design whose weight is on the
 //     expert's INPUT) or as they are,
 //   * ic_moe_expert_product: for few rows, the product of every sorted row with its own expert's matrix, the
-//     weights streamed once per expert and chunk of rows; with the gated unit silu(gate) * up in its epilogue,
+//     weights streamed once per expert and chunk of rows; with the gated unit silu(gate) * up (or, with a limit, the
+//     unit with bounded branches) in its epilogue,
 //   * ic_moe_combine: a token's result is the sum of its pairs' rows (times the weight when it is on the
-//     OUTPUT), plus an optional row of a shared expert.
+//     OUTPUT), plus an optional row of a shared expert; a pair of an identity expert counts the token's own row.
 // For many rows the products between gather and combine are library products over each expert's run of rows.
 #include "common.h"
 
@@ -19,47 +22,110 @@ constexpr int kMoeMaxExperts = 1024;
 constexpr int kMoeMaxTop = 16;
 
 // ---------------------------------------------------------------------------------------------
-// One thread a token.  mode 0: s = sigmoid(z); mode 1: s = softmax(z) over all experts.
+// A wave a token, four tokens a block; lane l holds experts l, l + 64, ...  mode 0: s = sigmoid(z); mode 1: s = softmax(z)
+// over all experts.  The choice goes by s + correction (without a correction by z, with which both scores grow), the weights
+// are s.  groups > 1: a group of E / groups neighbours is as good as its best member, the `group_keep` best groups (lower
+// index first among equals) stay, the members of the others cannot be chosen.  renorm: the weights are divided by their sum
+// + 1e-20; then all are multiplied by `scale`.
 // ---------------------------------------------------------------------------------------------
+template <int PER>                                        // experts a lane holds at most
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const float* __restrict__ z, int z_stride, int T, int E, int top, int mode, int renorm,
-                 int* __restrict__ ids, float* __restrict__ weights) {
-    const int t = blockIdx.x * blockDim.x + threadIdx.x;
-    if (t >= T) return;
+                 const float* __restrict__ correction, int groups, int group_keep, float scale, int* __restrict__ ids,
+                 float* __restrict__ weights) {
+    __shared__ float c_s[4][64 * PER], best_s[4][64 * PER];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const bool live = blockIdx.x * 4 + wave < T;
+    const int t = live ? blockIdx.x * 4 + wave : T - 1;
     const float* zr = z + (size_t)t * z_stride;
-    float zmax = -INFINITY, den = 1.f;
+    float s[PER], c[PER];
+    float zmax = -INFINITY, den = 0.f;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+        const int e = lane + 64 * j;
+        s[j] = e < E ? zr[e] : -INFINITY;
+        zmax = fmaxf(zmax, s[j]);
+    }
     if (mode == 1) {
-        for (int e = 0; e < E; ++e) zmax = fmaxf(zmax, zr[e]);
-        den = 0.f;
-        for (int e = 0; e < E; ++e) den += expf(zr[e] - zmax);
-    }
-    int chosen[kMoeMaxTop];
-    float total = 0.f;
-    for (int k = 0; k < top; ++k) {
-        int best = -1;
-        float bz = -INFINITY;
-        for (int e = 0; e < E; ++e) {
-            bool taken = false;
-            for (int j = 0; j < k; ++j) taken |= chosen[j] == e;
-            if (!taken && (best < 0 || zr[e] > bz)) { best = e; bz = zr[e]; }     // both score functions grow with z
+        zmax = wave_max(zmax);
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            if (lane + 64 * j < E) den += expf(s[j] - zmax);
         }
-        chosen[k] = best;
-        const float s = mode == 1 ? expf(bz - zmax) / den : 1.0f / (1.0f + expf(-bz));
-        ids[(size_t)t * top + k] = best;
-        weights[(size_t)t * top + k] = s;
-        total += s;
+        den = wave_sum(den);
     }
-    if (renorm)
-        for (int k = 0; k < top; ++k) weights[(size_t)t * top + k] /= total;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+        const int e = lane + 64 * j;
+        const float zv = s[j];
+        s[j] = mode == 1 ? expf(zv - zmax) / den : 1.0f / (1.0f + expf(-zv));
+        c[j] = e >= E ? -INFINITY : correction ? s[j] + correction[e] : zv;
+    }
+    if (groups > 1) {                                      // (the same branch in the whole block)
+        const int size = E / groups;
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            if (lane + 64 * j < E) c_s[wave][lane + 64 * j] = c[j];
+        }
+        __syncthreads();
+        for (int g = lane; g < groups; g += 64) {
+            float best = -INFINITY;
+            for (int i = 0; i < size; ++i) best = fmaxf(best, c_s[wave][g * size + i]);
+            best_s[wave][g] = best;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            const int e = lane + 64 * j;
+            if (e >= E) continue;
+            const int g = e / size;
+            const float mine = best_s[wave][g];
+            int better = 0;
+            for (int o = 0; o < groups; ++o) better += best_s[wave][o] > mine || (best_s[wave][o] == mine && o < g);
+            if (better >= group_keep) c[j] = -INFINITY;
+        }
+    }
+    unsigned taken = 0;                                    // bit j: this lane's expert lane + 64 j is chosen already (or is none)
+    float total = 0.f, w_mine = 0.f;
+    int id_mine = 0;
+    for (int k = 0; k < top; ++k) {
+        float bc = -INFINITY, bs = 0.f;
+        int be = kMoeMaxExperts;
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            const int e = lane + 64 * j;
+            if (e < E && !((taken >> j) & 1u) && (be == kMoeMaxExperts || c[j] > bc)) { bc = c[j]; be = e; bs = s[j]; }
+        }
+        for (int o = 32; o > 0; o >>= 1) {
+            const float oc = __shfl_xor(bc, o, kWave), os = __shfl_xor(bs, o, kWave);
+            const int oe = __shfl_xor(be, o, kWave);
+            if (oe < kMoeMaxExperts && (be == kMoeMaxExperts || oc > bc || (oc == bc && oe < be))) { bc = oc; be = oe; bs = os; }
+        }
+        if ((be & 63) == lane) taken |= 1u << (be >> 6);
+        total += bs;
+        if (lane == k) { id_mine = be; w_mine = bs; }
+    }
+    if (live && lane < top) {
+        ids[(size_t)t * top + lane] = id_mine;
+        weights[(size_t)t * top + lane] = (renorm ? w_mine / (total + 1e-20f) : w_mine) * scale;
+    }
 }
 
-IC_EXPORT int ic_moe_route(const float* z, int z_stride, int T, int E, int top, int mode, int renorm, int* ids,
-                           float* weights, hipStream_t stream) {
+IC_EXPORT int ic_moe_route(const float* z, int z_stride, int T, int E, int top, int mode, int renorm, const float* correction,
+                           int groups, int group_keep, float scale, int* ids, float* weights, hipStream_t stream) {
     if (T <= 0) return IC_OK;
     if (E <= 0 || E > kMoeMaxExperts || top <= 0 || top > kMoeMaxTop || top > E || z_stride < E || (mode != 0 && mode != 1))
         return IC_ERR_ARG;
-    hipLaunchKernelGGL(moe_route_kernel, dim3((T + 255) / 256), dim3(256), 0, stream, z, z_stride, T, E, top, mode, renorm,
-                       ids, weights);
+    if (groups < 1 || E % groups || group_keep < 1 || group_keep > groups || (groups > 1 && group_keep * (E / groups) < top))
+        return IC_ERR_ARG;
+#define IC_ROUTE(PER)                                                                                                     \
+    hipLaunchKernelGGL(moe_route_kernel<PER>, dim3((T + 3) / 4), dim3(256), 0, stream, z, z_stride, T, E, top, mode, renorm, \
+                       correction, groups, group_keep, scale, ids, weights)
+    if (E <= 64) IC_ROUTE(1);
+    else if (E <= 128) IC_ROUTE(2);
+    else if (E <= 256) IC_ROUTE(4);
+    else IC_ROUTE(kMoeMaxExperts / 64);
+#undef IC_ROUTE
     return ic_launch_status();
 }
 
@@ -168,7 +234,7 @@ template <typename T, bool GLU, bool VEC, int kMoeRC>
 __global__ void __launch_bounds__(256)
 moe_expert_product_kernel(const T* __restrict__ a, int a_stride, const T* __restrict__ w, long long w_expert_stride,
                           const int* __restrict__ offsets, T* __restrict__ out, int out_stride, int N, int K,
-                          int cols_per_block) {
+                          int cols_per_block, float limit, float slope) {
     extern __shared__ float rows_lds[];            // [kMoeRC][K]
     const int e = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
     const int r0 = offsets[e], r1 = offsets[e + 1];
@@ -230,7 +296,7 @@ moe_expert_product_kernel(const T* __restrict__ a, int a_stride, const T* __rest
                             // the gate and up products are rounded to the rows' dtype first, as a product kernel followed
                             // by the gated unit's kernel would leave them
                             const float g = to_f32(from_f32<T>(acc[r])), u = to_f32(from_f32<T>(acc2[r]));
-                            v = u * (g / (1.0f + expf(-g)));
+                            v = limit > 0.f ? glu_clamped_f(g, u, limit, slope) : u * (g / (1.0f + expf(-g)));
                         }
                         out[(size_t)(rb + r) * out_stride + c] = from_f32<T>(v);
                     }
@@ -258,7 +324,7 @@ template <bool GLU>
 __global__ void __launch_bounds__(256)
 moe_expert_product_mfma_kernel(const uint16_t* __restrict__ a, int a_stride, const uint16_t* __restrict__ w,
                                long long w_expert_stride, const int* __restrict__ offsets, uint16_t* __restrict__ out,
-                               int out_stride, int N, int K) {
+                               int out_stride, int N, int K, float limit, float slope) {
     constexpr int NW = GLU ? 2 : 1;                       // weight rows per column: gate and up, or one
     constexpr int MT = 2;                                 // tiles of 16 token rows per pass over the weights
     __shared__ float sums[4][MT][NW][16][17];
@@ -319,7 +385,7 @@ moe_expert_product_mfma_kernel(const uint16_t* __restrict__ a, int a_stride, con
                     const float u2 = sums[0][m][NW - 1][col][j] + sums[1][m][NW - 1][col][j] + sums[2][m][NW - 1][col][j] + sums[3][m][NW - 1][col][j];
                     // gate and up are rounded to bfloat16 first, as a product kernel followed by the gated unit's kernel leaves them
                     const float g = bf16_bits_to_f32(f32_to_bf16_bits(v)), u = bf16_bits_to_f32(f32_to_bf16_bits(u2));
-                    v = u * (g / (1.0f + expf(-g)));
+                    v = limit > 0.f ? glu_clamped_f(g, u, limit, slope) : u * (g / (1.0f + expf(-g)));
                 }
                 out[(size_t)row * out_stride + c0 + col] = f32_to_bf16_bits(v);
             }
@@ -329,17 +395,17 @@ moe_expert_product_mfma_kernel(const uint16_t* __restrict__ a, int a_stride, con
 
 IC_EXPORT int ic_moe_expert_product(const void* a, int a_stride, const void* w, long long w_expert_stride, int dtype,
                                     const int* offsets, void* out, int out_stride, int E, int N, int K, int glu,
-                                    int compute_units, hipStream_t stream) {
+                                    float limit, float slope, int compute_units, hipStream_t stream) {
     if (E <= 0 || E > 65535 || N <= 0 || K <= 0) return IC_ERR_ARG;
     if (dtype == IC_BF16 && N % 16 == 0 && K % 32 == 0 && (w_expert_stride % 8) == 0 && (a_stride % 8) == 0 &&
         ((uintptr_t)w % 16) == 0 && ((uintptr_t)a % 16) == 0 && N / 16 <= 0x7fffffff / 2) {
         dim3 grid((unsigned)(N / 16), (unsigned)E), block(256);
         if (glu)
             hipLaunchKernelGGL(moe_expert_product_mfma_kernel<true>, grid, block, 0, stream, (const uint16_t*)a, a_stride,
-                               (const uint16_t*)w, w_expert_stride, offsets, (uint16_t*)out, out_stride, N, K);
+                               (const uint16_t*)w, w_expert_stride, offsets, (uint16_t*)out, out_stride, N, K, limit, slope);
         else
             hipLaunchKernelGGL(moe_expert_product_mfma_kernel<false>, grid, block, 0, stream, (const uint16_t*)a, a_stride,
-                               (const uint16_t*)w, w_expert_stride, offsets, (uint16_t*)out, out_stride, N, K);
+                               (const uint16_t*)w, w_expert_stride, offsets, (uint16_t*)out, out_stride, N, K, limit, slope);
         return ic_launch_status();
     }
     int rc = 8;
@@ -356,7 +422,7 @@ IC_EXPORT int ic_moe_expert_product(const void* a, int a_stride, const void* w, 
     dim3 grid((unsigned)bx, (unsigned)E), block(256);
 #define IC_MOE_LAUNCH(TT, G, V, R)                                                                                       \
     hipLaunchKernelGGL((moe_expert_product_kernel<TT, G, V, R>), grid, block, lds, stream, (const TT*)a, a_stride,        \
-                       (const TT*)w, w_expert_stride, offsets, (TT*)out, out_stride, N, K, cols)
+                       (const TT*)w, w_expert_stride, offsets, (TT*)out, out_stride, N, K, cols, limit, slope)
 #define IC_MOE_RC(TT, G, V)                                                                                              \
     do {                                                                                                                 \
         if (rc == 8) IC_MOE_LAUNCH(TT, G, V, 8);                                                                         \
@@ -379,7 +445,8 @@ IC_EXPORT int ic_moe_expert_product(const void* a, int a_stride, const void* w, 
 }
 
 // ---------------------------------------------------------------------------------------------
-// out[t] = sum_k y[place[t * top + k]] * (weights[t * top + k] or 1) + shared[t].  grid (T, blocks over the columns), a
+// out[t] = sum_k y[place[t * top + k]] * (weights[t * top + k] or 1) + shared[t]; pairs of identity experts (sorted behind
+// the *n_routed others) take the token's own row own[t] for y.  grid (T, blocks over the columns), a
 // thread 16 bytes of columns (one column where rows are not made of whole 16-byte pieces): the pairs' places are read
 // once, then the top + 1 loads of a piece are in flight together.
 // ---------------------------------------------------------------------------------------------
@@ -399,7 +466,8 @@ template <> __device__ __forceinline__ void moe_store<bf16>(bf16* p, const float
 template <typename T, bool VEC>
 __global__ void __launch_bounds__(256)
 moe_combine_kernel(const T* __restrict__ y, int y_stride, const int* __restrict__ place, const float* __restrict__ weights,
-                   const T* __restrict__ shared, int shared_stride, int top, int d, T* __restrict__ out, int out_stride) {
+                   const T* __restrict__ shared, int shared_stride, const T* __restrict__ own, int own_stride,
+                   const int* __restrict__ n_routed, int top, int d, T* __restrict__ out, int out_stride) {
     constexpr int V = VEC ? MoeVec<T>::N : 1;
     const int t = blockIdx.x, i = (blockIdx.y * 256 + threadIdx.x) * V;
     if (i >= d) return;
@@ -412,10 +480,11 @@ moe_combine_kernel(const T* __restrict__ y, int y_stride, const int* __restrict_
     } else {
         s[0] = shared ? to_f32(shared[(size_t)t * shared_stride + i]) : 0.f;
     }
+    const int routed = own ? *n_routed : 0;
     for (int k = 0; k < top; ++k) {
-        const int pair = t * top + k;
+        const int pair = t * top + k, at = place[pair];
         const float w = weights ? weights[pair] : 1.f;
-        const T* row = y + (size_t)place[pair] * y_stride + i;
+        const T* row = (own && at >= routed) ? own + (size_t)t * own_stride + i : y + (size_t)at * y_stride + i;
         if (VEC) {
             float v[V];
             MoeVec<T>::load(row, v);
@@ -430,19 +499,21 @@ moe_combine_kernel(const T* __restrict__ y, int y_stride, const int* __restrict_
 }
 
 IC_EXPORT int ic_moe_combine(const void* y, int y_stride, int dtype, const int* place, const float* weights,
-                             const void* shared, int shared_stride, int T, int top, int d, void* out, int out_stride,
-                             hipStream_t stream) {
+                             const void* shared, int shared_stride, const void* own, int own_stride, const int* n_routed, int T,
+                             int top, int d, void* out, int out_stride, hipStream_t stream) {
     if (T <= 0) return IC_OK;
+    if (own && !n_routed) return IC_ERR_ARG;
     if (top <= 0 || top > kMoeMaxTop || d <= 0 || (dtype != IC_F32 && dtype != IC_BF16)) return IC_ERR_ARG;
     const int V = dtype == IC_F32 ? 4 : 8;
     const bool vec = d % V == 0 && y_stride % V == 0 && out_stride % V == 0 && (!shared || shared_stride % V == 0) &&
+                     (!own || own_stride % V == 0) && ((uintptr_t)own % 16) == 0 &&
                      ((uintptr_t)y % 16) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)shared % 16) == 0;
     const int per = 256 * (vec ? V : 1);
     dim3 grid((unsigned)T, (unsigned)((d + per - 1) / per)), block(256);
     if (grid.y > 65535) return IC_ERR_ARG;
 #define IC_MC(TT, VV)                                                                                                   \
     hipLaunchKernelGGL((moe_combine_kernel<TT, VV>), grid, block, 0, stream, (const TT*)y, y_stride, place, weights,      \
-                       (const TT*)shared, shared_stride, top, d, (TT*)out, out_stride)
+                       (const TT*)shared, shared_stride, (const TT*)own, own_stride, n_routed, top, d, (TT*)out, out_stride)
     if (dtype == IC_F32) { if (vec) IC_MC(float, true); else IC_MC(float, false); }
     else { if (vec) IC_MC(bf16, true); else IC_MC(bf16, false); }
 #undef IC_MC

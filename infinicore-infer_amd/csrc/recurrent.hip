@@ -5,9 +5,7 @@
 // A step's tokens are rows 0..T-1; request r owns rows req_start[r] .. req_start[r+1]-1 and the state slot
 // state_slots[r].  State lives in float32, [slots, state_stride] floats, a part of a mixer's state at an offset.
 // Everything that enters a recurrence is float32.
-#include "common.h"
-
-constexpr int kConvMaxTaps = 8;
+#include "short_conv.h"
 
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
@@ -44,26 +42,6 @@ causal_conv_kernel(const T* __restrict__ xin, int xin_stride, const float* __res
     if (act == 1) acc = silu_f(acc);
     out[(size_t)t * C + c] = acc;
     if (out_copy) out_copy[(size_t)t * copy_stride + c] = from_f32<T>(acc);
-}
-
-// The state after the step: the last taps-1 of (old state, the step's inputs).  One thread per (request, channel).
-template <typename T>
-__global__ void __launch_bounds__(256)
-conv_state_kernel(const T* __restrict__ xin, int xin_stride, const float* __restrict__ in_bias, int taps, int C,
-                  float* __restrict__ state, long long state_stride, const int* __restrict__ req_start,
-                  const int* __restrict__ state_slots) {
-    const int c = blockIdx.x * blockDim.x + threadIdx.x, r = blockIdx.y;
-    if (c >= C) return;
-    const int start = req_start[r], n = req_start[r + 1] - start;
-    float* st = state + (long long)state_slots[r] * state_stride;
-    const float ib = in_bias ? in_bias[c] : 0.f;
-    float nv[kConvMaxTaps];
-    for (int k = 0; k < taps - 1; ++k) {
-        const int i = n + k;                      // index into (old state, inputs)
-        nv[k] = i < taps - 1 ? st[(size_t)i * C + c]
-                             : to_f32(xin[(size_t)(start + i - (taps - 1)) * xin_stride + c]) + ib;
-    }
-    for (int k = 0; k < taps - 1; ++k) st[(size_t)k * C + c] = nv[k];
 }
 
 IC_EXPORT int ic_causal_conv(const void* xin, int xin_stride, int dtype, const float* in_bias, const float* w,
@@ -428,12 +406,30 @@ IC_EXPORT int ic_gated_group_norm(const float* y, const void* z, int z_stride, i
 
 // ---- a product with one weight matrix per block of columns --------------------------------------------------------------
 // C[m, b * c_step + n] = sum_k A[m, b * a_step + k] W[b, n, k]  (b < B, n < N, k < K; W contiguous [B, N, K]),
-// optionally times sigmoid(gate[m, b * c_step + n]).  float32 accumulation on the vector units; tiles of BM x 64
-// results per block of 256 threads, 16 k at a time through LDS.
+// with an epilogue: kind 1 multiplies by sigmoid(gate[m, b * c_step + n]); kind 2 turns a low-rank product into the decay
+// factors of a recurrence, exp(-rate[n / per] * softplus(v + bias[n])), and kind 3 into exp(c * logsigmoid(v + bias[n])).
+// float32 accumulation on the vector units; tiles of BM x 64 results per block of 256 threads, 16 k at a time through LDS.
+template <typename T> struct BpEpilogue {
+    int kind;
+    const T* gate;
+    int gate_stride;
+    const float* bias;
+    const float* rate;
+    int per;
+    float c;
+    __device__ __forceinline__ float operator()(float v, int m, int at, int n) const {
+        if (kind == 0) return v;
+        if (kind == 1) return v * sigmoid_f(to_f32(gate[(size_t)m * gate_stride + at]));
+        v += bias[n];
+        if (kind == 2) return expf(-rate[n / per] * softplus_f(v));
+        return expf(-c * softplus_f(-v));
+    }
+};
+
 template <typename T, typename TC, int BM>
 __global__ void __launch_bounds__(256)
 blocked_product_kernel(const T* __restrict__ A, int lda, int a_step, const T* __restrict__ W, TC* __restrict__ C,
-                       int ldc, int c_step, const T* __restrict__ gate, int gate_stride, int M, int N, int K) {
+                       int ldc, int c_step, BpEpilogue<T> ep, int M, int N, int K) {
     constexpr int BN = 64, BK = 16, RM = BM / 16;
     __shared__ float As[BK][BM + 1];
     __shared__ float Ws[BK][BN + 1];
@@ -478,8 +474,7 @@ blocked_product_kernel(const T* __restrict__ A, int lda, int a_step, const T* __
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx + 16 * j;
             if (n >= N) continue;
-            float v = acc[i][j];
-            if (gate) v *= sigmoid_f(to_f32(gate[(size_t)m * gate_stride + (size_t)b * c_step + n]));
+            const float v = ep(acc[i][j], m, b * c_step + n, n);
             C[(size_t)m * ldc + (size_t)b * c_step + n] = from_f32<TC>(v);
         }
     }
@@ -490,7 +485,7 @@ blocked_product_kernel(const T* __restrict__ A, int lda, int a_step, const T* __
 template <typename T, typename TC, int MT>
 __global__ void __launch_bounds__(256)
 blocked_product_rows_kernel(const T* __restrict__ A, int lda, int a_step, const T* __restrict__ W, TC* __restrict__ C,
-                            int ldc, int c_step, const T* __restrict__ gate, int gate_stride, int M, int N, int K) {
+                            int ldc, int c_step, BpEpilogue<T> ep, int M, int N, int K) {
     constexpr int VEC = 16 / sizeof(T);
     extern __shared__ float a_rows[];         // MT * K
     const int b = blockIdx.y, n = blockIdx.x * 32 + threadIdx.x / 8, sub = threadIdx.x % 8;
@@ -521,7 +516,7 @@ blocked_product_rows_kernel(const T* __restrict__ A, int lda, int a_step, const 
         v += __shfl_xor(v, 2, kWave);
         v += __shfl_xor(v, 1, kWave);
         if (sub == 0 && n < N && mm < M) {
-            if (gate) v *= sigmoid_f(to_f32(gate[(size_t)mm * gate_stride + (size_t)b * c_step + n]));
+            v = ep(v, mm, b * c_step + n, n);
             C[(size_t)mm * ldc + (size_t)b * c_step + n] = from_f32<TC>(v);
         }
     }
@@ -537,7 +532,7 @@ typedef float bp_v16f __attribute__((ext_vector_type(16)));
 template <typename TC>
 __global__ void __launch_bounds__(256)
 blocked_product_mfma_kernel(const bf16* __restrict__ A, int lda, int a_step, const bf16* __restrict__ W, TC* __restrict__ C,
-                            int ldc, int c_step, const bf16* __restrict__ gate, int gate_stride, int M, int N, int K) {
+                            int ldc, int c_step, BpEpilogue<bf16> ep, int M, int N, int K) {
     const int b = blockIdx.z, wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lq = lane & 31, half = lane >> 5;
     const int m0 = blockIdx.y * 64 + 32 * (wave >> 1), n0 = blockIdx.x * 64 + 32 * (wave & 1);
     if (m0 >= M || n0 >= N) return;
@@ -568,8 +563,7 @@ blocked_product_mfma_kernel(const bf16* __restrict__ A, int lda, int a_step, con
     for (int r = 0; r < 16; ++r) {
         const int nn = n0 + 8 * (r >> 2) + 4 * half + (r & 3);
         if (nn < N) {
-            float v = acc[r];
-            if (gate) v *= sigmoid_f(to_f32(gate[(size_t)m * gate_stride + (size_t)b * c_step + nn]));
+            const float v = ep(acc[r], m, b * c_step + nn, nn);
             C[(size_t)m * ldc + (size_t)b * c_step + nn] = from_f32<TC>(v);
         }
     }
@@ -580,13 +574,13 @@ template <> struct bp_is_bf16<bf16> { static constexpr bool value = true; };
 
 template <typename T, typename TC>
 static void blocked_product_launch(const void* A, int lda, int a_step, const void* W, void* C, int ldc, int c_step,
-                                   const void* gate, int gate_stride, int M, int N, int K, int B, hipStream_t stream) {
+                                   BpEpilogue<T> ep, int M, int N, int K, int B, hipStream_t stream) {
     constexpr int VEC = 16 / sizeof(T);
     if (M <= 8 && K % VEC == 0 && (size_t)8 * K * sizeof(float) <= 48 * 1024 && ((uintptr_t)W % 16) == 0) {
         dim3 grid((N + 31) / 32, B);
 #define IC_ROWS(MT)                                                                                                   \
     hipLaunchKernelGGL((blocked_product_rows_kernel<T, TC, MT>), grid, dim3(256), (size_t)MT * K * sizeof(float), stream, \
-                       (const T*)A, lda, a_step, (const T*)W, (TC*)C, ldc, c_step, (const T*)gate, gate_stride, M, N, K)
+                       (const T*)A, lda, a_step, (const T*)W, (TC*)C, ldc, c_step, ep, M, N, K)
         if (M == 1) IC_ROWS(1); else if (M == 2) IC_ROWS(2); else if (M <= 4) IC_ROWS(4); else IC_ROWS(8);
 #undef IC_ROWS
         return;
@@ -595,7 +589,7 @@ static void blocked_product_launch(const void* A, int lda, int a_step, const voi
         if (M > 8 && K % 16 == 0 && lda % 8 == 0 && a_step % 8 == 0 && ((uintptr_t)A % 16) == 0 && ((uintptr_t)W % 16) == 0) {
             dim3 grid((N + 63) / 64, (M + 63) / 64, B);
             hipLaunchKernelGGL((blocked_product_mfma_kernel<TC>), grid, dim3(256), 0, stream, (const bf16*)A, lda, a_step,
-                               (const bf16*)W, (TC*)C, ldc, c_step, (const bf16*)gate, gate_stride, M, N, K);
+                               (const bf16*)W, (TC*)C, ldc, c_step, ep, M, N, K);
             return;
         }
     }
@@ -603,26 +597,42 @@ static void blocked_product_launch(const void* A, int lda, int a_step, const voi
     if (M <= 16 || (long long)((N + 63) / 64) * ((M + 63) / 64) * B < 256) {
         dim3 grid((N + 63) / 64, (M + 15) / 16, B);
         hipLaunchKernelGGL((blocked_product_kernel<T, TC, 16>), grid, dim3(256), 0, stream, (const T*)A, lda, a_step,
-                           (const T*)W, (TC*)C, ldc, c_step, (const T*)gate, gate_stride, M, N, K);
+                           (const T*)W, (TC*)C, ldc, c_step, ep, M, N, K);
     } else {
         dim3 grid((N + 63) / 64, (M + 63) / 64, B);
         hipLaunchKernelGGL((blocked_product_kernel<T, TC, 64>), grid, dim3(256), 0, stream, (const T*)A, lda, a_step,
-                           (const T*)W, (TC*)C, ldc, c_step, (const T*)gate, gate_stride, M, N, K);
+                           (const T*)W, (TC*)C, ldc, c_step, ep, M, N, K);
     }
+}
+
+static int blocked_product(const void* A, int lda, int a_step, const void* W, int dtype, void* C, int c_dtype, int ldc, int c_step,
+                           int kind, const void* gate, int gate_stride, const float* bias, const float* rate, int per, float c, int M,
+                           int N, int K, int B, hipStream_t stream) {
+    if (M <= 0) return IC_OK;
+    if (N <= 0 || K <= 0 || B <= 0 || B > 65535 || (M + 15) / 16 > 65535) return IC_ERR_ARG;
+    const BpEpilogue<float> ef{kind, (const float*)gate, gate_stride, bias, rate, per, c};
+    const BpEpilogue<bf16> eb{kind, (const bf16*)gate, gate_stride, bias, rate, per, c};
+    if (dtype == IC_F32 && c_dtype == IC_F32)
+        blocked_product_launch<float, float>(A, lda, a_step, W, C, ldc, c_step, ef, M, N, K, B, stream);
+    else if (dtype == IC_BF16 && c_dtype == IC_BF16)
+        blocked_product_launch<bf16, bf16>(A, lda, a_step, W, C, ldc, c_step, eb, M, N, K, B, stream);
+    else if (dtype == IC_BF16 && c_dtype == IC_F32)
+        blocked_product_launch<bf16, float>(A, lda, a_step, W, C, ldc, c_step, eb, M, N, K, B, stream);
+    else
+        return IC_ERR_UNSUPPORTED;
+    return ic_launch_status();
 }
 
 IC_EXPORT int ic_blocked_product(const void* A, int lda, int a_step, const void* W, int dtype, void* C, int c_dtype,
                                  int ldc, int c_step, const void* gate, int gate_stride, int M, int N, int K, int B,
                                  hipStream_t stream) {
-    if (M <= 0) return IC_OK;
-    if (N <= 0 || K <= 0 || B <= 0 || B > 65535 || (M + 15) / 16 > 65535) return IC_ERR_ARG;
-    if (dtype == IC_F32 && c_dtype == IC_F32)
-        blocked_product_launch<float, float>(A, lda, a_step, W, C, ldc, c_step, gate, gate_stride, M, N, K, B, stream);
-    else if (dtype == IC_BF16 && c_dtype == IC_BF16)
-        blocked_product_launch<bf16, bf16>(A, lda, a_step, W, C, ldc, c_step, gate, gate_stride, M, N, K, B, stream);
-    else if (dtype == IC_BF16 && c_dtype == IC_F32)
-        blocked_product_launch<bf16, float>(A, lda, a_step, W, C, ldc, c_step, gate, gate_stride, M, N, K, B, stream);
-    else
-        return IC_ERR_UNSUPPORTED;
-    return ic_launch_status();
+    return blocked_product(A, lda, a_step, W, dtype, C, c_dtype, ldc, c_step, gate ? 1 : 0, gate, gate_stride, nullptr, nullptr, 1, 0.f, M,
+                           N, K, B, stream);
+}
+
+// C[m, n] = the decay factor of A[m] . W[n] (float32): kind 2 or 3 of the epilogues.
+IC_EXPORT int ic_decay_product(const void* A, int lda, const void* W, int dtype, float* C, int kind, const float* bias, const float* rate,
+                               int per, float c, int M, int N, int K, hipStream_t stream) {
+    if ((kind != 2 && kind != 3) || !bias || (kind == 2 && (!rate || per <= 0))) return IC_ERR_ARG;
+    return blocked_product(A, lda, 0, W, dtype, C, IC_F32, N, 0, kind, nullptr, 0, bias, rate, per, c, M, N, K, 1, stream);
 }

@@ -5,12 +5,15 @@
 //   * bias, query/key norm (per head or over the whole row), value mixing with an earlier layer's
 //     values and the write of keys and values into the paged cache, in one pass over a token's
 //     projected row,
+//   * the same for queries and keys that pass a short convolution, a rotation of halves and then the norm,
+//   * x = rmsnorm(alpha x + the sublayer's results) * w: the norm on the sum,
 //   * element-wise activations of a dense feed-forward.
 // The residual stream is float32; every norm, sum of squares, angle and mix is float32.
 //
 // Cache layout of one layer: K plane [num_pages, n_kv_heads, page_size, key_dim], V plane
 // [num_pages, n_kv_heads, page_size, value_dim].
-#include "common.h"
+#include "rotation.h"
+#include "short_conv.h"
 
 // 16 bytes of a row as float32 values.
 template <typename T> struct RowPack;
@@ -428,6 +431,235 @@ IC_EXPORT int ic_qk_norm_store(const void* rows, int row_stride, int dtype, cons
                            nkvh, dk, dv, page_size);
     else
         return IC_ERR_UNSUPPORTED;
+    return ic_launch_status();
+}
+
+// ---------------------------------------------------------------------------------------------
+// rows[t] = [q (nh * dk) | k (nkvh * dk) | v (nkvh * dv) | ..] of row_stride elements, token by token:
+//   every channel passes a causal convolution (taps 0: none; the inputs before the step come from the request's state);
+//   q and k heads: entry i < rot_dims / 2 turns with entry i + rot_dims / 2 by the angle position * f_i (freq: float32
+//   [2, rot_dims / 2], the frequency and what its rounding left; rot_dims 0: no rotation), then norm 1: unit root mean
+//   square over the head's dk entries, times w[dk] (null: no weight);
+//   q -> q_out[t], k and v -> the cache at slots[t] (null: q only).
+// grid (T, ceil(heads of q, k, v / kRopeHeads)), a wave takes heads in turn: the token's angles are formed once a block.
+// single: every request brings one token, and the wave moves the convolution's state on itself.
+// ---------------------------------------------------------------------------------------------
+constexpr int kRopeHeads = 16;
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+conv_rope_norm_store_kernel(const T* __restrict__ rows, int row_stride, const float* __restrict__ cw, int taps,
+                            const int* __restrict__ positions, const float* __restrict__ freq, int rot_dims,
+                            const float* __restrict__ qw, const float* __restrict__ kw, int norm, float eps, T* __restrict__ q_out,
+                            T* __restrict__ kcache, T* __restrict__ vcache, const int* __restrict__ slots, int nh, int nkvh, int dk,
+                            int dv, int page_size, float* __restrict__ state, long long state_stride, const int* __restrict__ token_req,
+                            const int* __restrict__ req_start, const int* __restrict__ state_slots, int single) {
+    __shared__ float cs_s[256], sn_s[256];
+    const int t = blockIdx.x, lane = threadIdx.x & 63, half = rot_dims / 2;
+    const int C = (nh + nkvh) * dk + nkvh * dv;
+    if (rot_dims) {
+        const float p = (float)positions[t];
+        for (int i = threadIdx.x; i < half; i += 256) {
+            float cs, sn;
+            pair_angle(p, freq[i], freq[half + i], cs, sn);
+            cs_s[i] = cs;
+            sn_s[i] = sn;
+        }
+        __syncthreads();
+    }
+    const int r = taps ? token_req[t] : 0, start = taps ? req_start[r] : 0;
+    float* st = taps > 1 ? state + (long long)state_slots[r] * state_stride : nullptr;
+    const int slot = slots ? slots[t] : -1;
+    const int pg = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot - pg * page_size : 0;
+    const int last = min(nh + 2 * nkvh, (int)(blockIdx.y + 1) * kRopeHeads);
+    for (int head = blockIdx.y * kRopeHeads + (threadIdx.x >> 6); head < last; head += 4) {
+        const bool qk = head < nh + nkvh;
+        const int base = qk ? head * dk : (nh + nkvh) * dk + (head - nh - nkvh) * dv;
+        auto in = [&](int e) {
+            const float v = conv_at<T>(rows, row_stride, cw, taps, C, st, t, start, base + e);
+            if (single && taps > 1) conv_shift(st, taps, C, base + e, to_f32(rows[(size_t)t * row_stride + base + e]));
+            return v;
+        };
+        if (!qk) {
+            T* dst = (slot >= 0 && vcache) ? vcache + (((size_t)pg * nkvh + (head - nh - nkvh)) * page_size + off) * dv : nullptr;
+            for (int e = lane; e < dv; e += 64) {
+                const float v = in(e);
+                if (dst) dst[e] = from_f32<T>(v);
+            }
+            continue;
+        }
+        // a lane holds pairs (i, i + half) and entries that are not rotated
+        float a[4], b[4], rest[8];
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int i = lane + 64 * j;
+            a[j] = b[j] = 0.f;
+            if (i < half) {
+                const float u = in(i), v = in(i + half), cs = cs_s[i], sn = sn_s[i];
+                a[j] = u * cs - v * sn;
+                b[j] = v * cs + u * sn;
+            }
+            ss += a[j] * a[j] + b[j] * b[j];
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            const int e = rot_dims + lane + 64 * j;
+            rest[j] = e < dk ? in(e) : 0.f;
+            ss += rest[j] * rest[j];
+        }
+        const float f = norm ? 1.0f / sqrtf(wave_sum(ss) / (float)dk + eps) : 1.f;
+        const bool is_q = head < nh;
+        const float* w = is_q ? qw : kw;
+        T* dst = is_q ? q_out + (size_t)t * nh * dk + base
+                      : (slot >= 0 && kcache) ? kcache + (((size_t)pg * nkvh + (head - nh)) * page_size + off) * dk : nullptr;
+        if (!dst) continue;
+        auto put = [&](int e, float v) { dst[e] = from_f32<T>(v * f * (w ? w[e] : 1.f)); };
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int i = lane + 64 * j;
+            if (i < half) { put(i, a[j]); put(i + half, b[j]); }
+        }
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+            const int e = rot_dims + lane + 64 * j;
+            if (e < dk) put(e, rest[j]);
+        }
+    }
+}
+
+IC_EXPORT int ic_conv_rope_norm_store(const void* rows, int row_stride, int dtype, const float* cw, int taps, const int* positions,
+                                      const float* freq, int rot_dims, const float* qw, const float* kw, int norm, float eps,
+                                      void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh, int nkvh, int dk, int dv,
+                                      int page_size, float* state, long long state_stride, const int* token_req, const int* req_start,
+                                      const int* state_slots, int R, int single, hipStream_t stream) {
+    if (T <= 0) return IC_OK;
+    if (nh <= 0 || nkvh <= 0 || dk <= 0 || dv <= 0 || page_size <= 0 || taps < 0 || taps > kConvMaxTaps) return IC_ERR_ARG;
+    if (rot_dims < 0 || rot_dims % 2 || rot_dims > dk || (rot_dims && (!freq || !positions))) return IC_ERR_ARG;
+    if (taps && (!cw || (taps > 1 && !state) || !token_req || !req_start || !state_slots || R <= 0)) return IC_ERR_ARG;
+    if ((qw == nullptr) != (kw == nullptr) || (single && T != R)) return IC_ERR_ARG;
+    const long long n = (long long)(nh + nkvh) * dk + (long long)nkvh * dv;
+    if (row_stride < n) return IC_ERR_ARG;
+    if (dk > 512 || dv > 512) return IC_ERR_TOO_LARGE;
+    const int C = (int)n;
+    dim3 grid(T, (nh + 2 * nkvh + kRopeHeads - 1) / kRopeHeads), block(256), sgrid((C + 255) / 256, R);
+    if (dtype == IC_F32) {
+        hipLaunchKernelGGL(conv_rope_norm_store_kernel<float>, grid, block, 0, stream, (const float*)rows, row_stride, cw, taps, positions,
+                           freq, rot_dims, qw, kw, norm, eps, (float*)q_out, (float*)kcache, (float*)vcache, slots, nh, nkvh, dk, dv,
+                           page_size, state, state_stride, token_req, req_start, state_slots, single);
+        if (taps > 1 && !single)
+            hipLaunchKernelGGL(conv_state_kernel<float>, sgrid, block, 0, stream, (const float*)rows, row_stride, nullptr, taps, C, state,
+                               state_stride, req_start, state_slots);
+    } else if (dtype == IC_BF16) {
+        hipLaunchKernelGGL(conv_rope_norm_store_kernel<bf16>, grid, block, 0, stream, (const bf16*)rows, row_stride, cw, taps, positions,
+                           freq, rot_dims, qw, kw, norm, eps, (bf16*)q_out, (bf16*)kcache, (bf16*)vcache, slots, nh, nkvh, dk, dv,
+                           page_size, state, state_stride, token_req, req_start, state_slots, single);
+        if (taps > 1 && !single)
+            hipLaunchKernelGGL(conv_state_kernel<bf16>, sgrid, block, 0, stream, (const bf16*)rows, row_stride, nullptr, taps, C, state,
+                               state_stride, req_start, state_slots);
+    } else
+        return IC_ERR_UNSUPPORTED;
+    return ic_launch_status();
+}
+
+// ---------------------------------------------------------------------------------------------
+// x[t] = v * rsqrt(mean(v^2) + eps) * w with v = alpha x[t] + sa ya[t] + sb yb[t] (yb null: one result);  copy[t] = x[t] in
+// the results' dtype.  One block per row, four entries a thread and access (one where the row is not made of such pieces);
+// up to kSumKeep pieces a thread wait in registers between the two passes, the rest is read and summed again.
+// ---------------------------------------------------------------------------------------------
+constexpr int kSumKeep = 6;
+
+template <typename T, int N> __device__ __forceinline__ void load_piece(const T* p, float* o) {
+    if (N == 1) o[0] = to_f32(p[0]);
+    else if (sizeof(T) == 4) load_floats<4>((const float*)p, o);
+    else {
+        const uint2 v = *reinterpret_cast<const uint2*>(p);
+        o[0] = __uint_as_float(v.x << 16); o[N > 1 ? 1 : 0] = __uint_as_float(v.x & 0xffff0000u);
+        o[N > 2 ? 2 : 0] = __uint_as_float(v.y << 16); o[N > 3 ? 3 : 0] = __uint_as_float(v.y & 0xffff0000u);
+    }
+}
+template <typename T, int N> __device__ __forceinline__ void store_piece(T* p, const float* o) {
+    if (N == 1) p[0] = from_f32<T>(o[0]);
+    else if (sizeof(T) == 4) *reinterpret_cast<float4*>(p) = make_float4(o[0], o[N > 1 ? 1 : 0], o[N > 2 ? 2 : 0], o[N > 3 ? 3 : 0]);
+    else
+        *reinterpret_cast<uint2*>(p) = uint2{(uint32_t)f32_to_bf16_bits(o[0]) | ((uint32_t)f32_to_bf16_bits(o[N > 1 ? 1 : 0]) << 16),
+                                             (uint32_t)f32_to_bf16_bits(o[N > 2 ? 2 : 0]) | ((uint32_t)f32_to_bf16_bits(o[N > 3 ? 3 : 0]) << 16)};
+}
+
+template <typename T, int N>
+__global__ void __launch_bounds__(256)
+sum_norm_kernel(const T* __restrict__ ya, float sa, const T* __restrict__ yb, float sb, float alpha, const float* __restrict__ w,
+                float* __restrict__ x, T* __restrict__ copy, int d, float eps) {
+    __shared__ float red[16];
+    const int t = blockIdx.x, pieces = d / N, step = blockDim.x;
+    float* xr = x + (size_t)t * d;
+    const T* ar = ya + (size_t)t * d;
+    const T* br = yb ? yb + (size_t)t * d : nullptr;
+    auto sum = [&](int c, float* v) {
+        float y[N];
+        load_piece<float, N>(xr + c * N, v);
+        load_piece<T, N>(ar + c * N, y);
+#pragma unroll
+        for (int i = 0; i < N; ++i) v[i] = alpha * v[i] + sa * y[i];
+        if (br) {
+            load_piece<T, N>(br + c * N, y);
+#pragma unroll
+            for (int i = 0; i < N; ++i) v[i] += sb * y[i];
+        }
+    };
+    float keep[kSumKeep][N];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < kSumKeep; ++j) {
+        const int c = threadIdx.x + j * step;
+        if (c < pieces) {
+            sum(c, keep[j]);
+#pragma unroll
+            for (int i = 0; i < N; ++i) ss += keep[j][i] * keep[j][i];
+        }
+    }
+    for (int c = threadIdx.x + kSumKeep * step; c < pieces; c += step) {
+        float v[N];
+        sum(c, v);
+#pragma unroll
+        for (int i = 0; i < N; ++i) ss += v[i] * v[i];
+    }
+    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)d + eps);
+    auto put = [&](int c, const float* v) {
+        float ws[N], o[N];
+        load_piece<float, N>(w + c * N, ws);
+#pragma unroll
+        for (int i = 0; i < N; ++i) o[i] = v[i] * r * ws[i];
+        store_piece<float, N>(xr + c * N, o);
+        if (copy) store_piece<T, N>(copy + (size_t)t * d + c * N, o);
+    };
+#pragma unroll
+    for (int j = 0; j < kSumKeep; ++j) {
+        const int c = threadIdx.x + j * step;
+        if (c < pieces) put(c, keep[j]);
+    }
+    for (int c = threadIdx.x + kSumKeep * step; c < pieces; c += step) {
+        float v[N];
+        sum(c, v);
+        put(c, v);
+    }
+}
+
+IC_EXPORT int ic_sum_norm(const void* ya, float sa, const void* yb, float sb, int dtype, float alpha, const float* w, float* x,
+                          void* copy, int T, int d, float eps, hipStream_t stream) {
+    if (T <= 0) return IC_OK;
+    if (d <= 0 || !ya || !w || !x) return IC_ERR_ARG;
+    const uintptr_t ptrs = (uintptr_t)ya | (uintptr_t)yb | (uintptr_t)w | (uintptr_t)x | (uintptr_t)copy;
+    const bool vec = d % 4 == 0 && (ptrs & 15) == 0;
+    const int pieces = vec ? d / 4 : d;
+    dim3 grid(T), block(pieces >= 256 ? 256 : (pieces + 63) / 64 * 64);
+#define IC_SN(TT, N)                                                                                                     \
+    hipLaunchKernelGGL((sum_norm_kernel<TT, N>), grid, block, 0, stream, (const TT*)ya, sa, (const TT*)yb, sb, alpha, w, x, \
+                       (TT*)copy, d, eps)
+    if (dtype == IC_F32) { if (vec) IC_SN(float, 4); else IC_SN(float, 1); }
+    else if (dtype == IC_BF16) { if (vec) IC_SN(bf16, 4); else IC_SN(bf16, 1); }
+    else return IC_ERR_UNSUPPORTED;
+#undef IC_SN
     return ic_launch_status();
 }
 

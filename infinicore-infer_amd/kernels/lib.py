@@ -127,6 +127,13 @@ _SIGNATURES = {
     "ic_ssm_scan": [_P, _I, _I, _I, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _P, _P, _LL, _P, _P, _I, _I, _I, _P, _P, _P],
     "ic_gated_group_norm": [_P, _P, _I, _I, _P, _I, _I, _F, _P, _I, _I, _P],
     "ic_blocked_product": [_P, _I, _I, _P, _I, _P, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P],
+    "ic_decay_product": [_P, _I, _P, _I, _P, _I, _P, _P, _I, _F, _I, _I, _I, _P],
+    "ic_conv_rope_norm_store": [_P, _I, _I, _P, _I, _P, _P, _I, _P, _P, _I, _F, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _LL, _P, _P, _P, _I, _I, _P],
+    "ic_sum_norm": [_P, _F, _P, _F, _I, _F, _P, _P, _P, _I, _I, _F, _P],
+    "ic_delta_prep": [_P, _I, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _F, _P, _LL, _P, _P, _P, _I, _I, _I, _P],
+    "ic_memory_gates": [_P, _I, _P, _P, _F, _I, _P, _P, _P, _P, _LL, _P, _P, _I, _P],
+    "ic_matrix_memory": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _P, _I, _I, _I, _I, _I, _F, _P, _P, _P, _LL, _P, _P, _I, _I, _I, _P],
+    "ic_gated_head_norm": [_P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _I, _P],
     "ic_latent_prep": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _P, _P, _P, _P, _I, _P],
     "ic_latent_q_rotate": [_P, _I, _I, _I, _I, _I, _I, _P, _I, _P, _P, _I, _I, _P],
     "ic_attn_latent": [_P, _I, _P, _I, _I, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _I, _P],
@@ -140,11 +147,11 @@ _SIGNATURES = {
     "ic_attn_pooled_decode": [_P, _I, _P, _I, _I, _P, _P, _P, _P, _P, _I, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P],
     "ic_attn_pooled_prefill_supported": [_I, _I, _I],
     "ic_attn_pooled_prefill": [_P, _I, _P, _I, _I, _P, _P, _P, _P, _P, _I, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _F, _I, _I, _P],
-    "ic_moe_route": [_P, _I, _I, _I, _I, _I, _I, _P, _P, _P],
+    "ic_moe_route": [_P, _I, _I, _I, _I, _I, _I, _P, _I, _I, _F, _P, _P, _P],
     "ic_moe_sort": [_P, _I, _I, _P, _P, _P, _P],
     "ic_moe_gather": [_P, _I, _I, _P, _P, _I, _I, _I, _P, _P],
-    "ic_moe_expert_product": [_P, _I, _P, _LL, _I, _P, _P, _I, _I, _I, _I, _I, _I, _P],
-    "ic_moe_combine": [_P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _P, _I, _P],
+    "ic_moe_expert_product": [_P, _I, _P, _LL, _I, _P, _P, _I, _I, _I, _I, _I, _F, _F, _I, _P],
+    "ic_moe_combine": [_P, _I, _I, _P, _P, _P, _I, _P, _I, _P, _I, _I, _I, _P, _I, _P],
     "ic_gated_norm_into_stream": [_P, _P, _I, _I, _P, _P, _P, _P, _I, _I, _I, _F, _P],
     "ic_token_gate": [_P, _I, _P, _I, _I, _P, _I, _I, _P, _I, _P],
     "ic_sample": [_P, _LL, _I, _I, _P, _P, _P, _P, _P, _P],

@@ -758,6 +758,64 @@ def qk_norm_store(rows, bias, q_weight, k_weight, norm_mode: int, eps: float, mi
           "qk_norm_store")
 
 
+def conv_rope_norm_store(rows, conv_w, positions, freq, rot_dims: int, q_weight, k_weight, norm: bool, eps: float, q_out, kcache, vcache,
+                         slots, n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int, page_size: int, state=None,
+                         state_offset: int = 0, token_req=None, req_start=None, state_slots=None, n_requests: int = 0, single: bool = False):
+    """One pass over the projected rows [q | k | v | ..]: a causal convolution per channel (``conv_w`` [channels, taps] with its
+    inputs in ``state``; None: none), a rotation of the halves of the first ``rot_dims`` entries of q and k heads, their norm
+    per head, q to ``q_out``, k and v into the cache planes at ``slots`` (None: no cache write)."""
+    _dev(rows, conv_w, positions, freq, q_weight, k_weight, q_out, kcache, vcache, slots, state, token_req, req_start, state_slots)
+    T = rows.shape[0]
+    nq, nk, nv = n_heads * key_dim, n_kv_heads * key_dim, n_kv_heads * value_dim
+    _need(rows.dim() == 2 and rows.stride(1) == 1 and rows.shape[1] >= nq + nk + nv, "conv_rope_norm_store: rows too short")
+    _need(tuple(q_out.shape) == (T, nq) and q_out.is_contiguous() and q_out.dtype == rows.dtype, "conv_rope_norm_store: q_out layout")
+    taps, sp, stride = 0, None, 0
+    if conv_w is not None:
+        taps = conv_w.shape[1]
+        _need(conv_w.dtype == torch.float32 and conv_w.is_contiguous() and tuple(conv_w.shape) == (nq + nk + nv, taps), "conv_rope_norm_store: convolution")
+        for t, n in ((token_req, "token_req"), (req_start, "req_start"), (state_slots, "state_slots")):
+            _i32(t, n)
+        _need(token_req.numel() >= T and req_start.numel() >= n_requests + 1 and state_slots.numel() >= n_requests, "conv_rope_norm_store: lists")
+        if taps > 1:
+            sp, stride = _state_part(state, state_offset)
+            _need(state_offset + (taps - 1) * (nq + nk + nv) <= stride, "conv_rope_norm_store: state too small")
+    _need(not single or T == n_requests, "conv_rope_norm_store: one token a request")
+    if rot_dims:
+        _i32(positions, "positions")
+        _need(positions.numel() == T and freq.dtype == torch.float32 and freq.is_contiguous() and freq.numel() == rot_dims, "conv_rope_norm_store: angles")
+    for v in (q_weight, k_weight):
+        _need(v is None or (v.dtype == torch.float32 and v.is_contiguous() and v.numel() == key_dim), "conv_rope_norm_store: norm weight")
+    if slots is not None:
+        _i32(slots, "slots")
+        _need(slots.numel() == T and kcache.dtype == rows.dtype and vcache.dtype == rows.dtype and kcache.is_contiguous() and vcache.is_contiguous()
+              and tuple(kcache.shape[1:]) == (n_kv_heads, page_size, key_dim)
+              and tuple(vcache.shape[1:]) == (n_kv_heads, page_size, value_dim) and kcache.shape[0] == vcache.shape[0],
+              "conv_rope_norm_store: cache must be K [pages, kv_heads, page_size, key_dim], V [.., value_dim]")
+    p = lambda t: t.data_ptr() if t is not None else None
+    check(get_lib().ic_conv_rope_norm_store(rows.data_ptr(), rows.stride(0), dtype_code(rows.dtype), p(conv_w), taps, p(positions), p(freq),
+                                            int(rot_dims), p(q_weight), p(k_weight), 1 if norm else 0, float(eps), q_out.data_ptr(),
+                                            p(kcache) if slots is not None else None, p(vcache) if slots is not None else None, p(slots),
+                                            T, n_heads, n_kv_heads, key_dim, value_dim, page_size, sp, stride, p(token_req), p(req_start),
+                                            p(state_slots), n_requests, 1 if single else 0, _stream()), "conv_rope_norm_store")
+
+
+def sum_norm(branches, alpha: float, weight, x, eps: float, copy=None):
+    """x = rmsnorm(alpha x + sum of s_i y_i) * weight, row by row (x float32, in place); ``branches``: one or two (y, s);
+    ``copy`` (optional) receives the new x rounded to the branches' dtype."""
+    (ya, sa), (yb, sb) = branches[0], (branches[1] if len(branches) > 1 else (None, 0.0))
+    _need(1 <= len(branches) <= 2, "sum_norm: one or two results")
+    _dev(ya, yb, weight, x, copy)
+    T, d = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous(), "sum_norm: the stream is float32")
+    for y in (ya, yb, copy):
+        _need(y is None or (tuple(y.shape) == (T, d) and y.is_contiguous() and y.dtype == ya.dtype), "sum_norm: layout")
+    _need(weight.dtype == torch.float32 and weight.numel() == d and weight.is_contiguous(), "sum_norm: weight must be float32 [d]")
+    check(get_lib().ic_sum_norm(ya.data_ptr(), float(sa), yb.data_ptr() if yb is not None else None, float(sb), dtype_code(ya.dtype),
+                                float(alpha), weight.data_ptr(), x.data_ptr(), copy.data_ptr() if copy is not None else None, T, d,
+                                float(eps), _stream()), "sum_norm")
+    return x
+
+
 def activation(x, out, kind: str):
     """out = act(x) element by element (relu2: relu(z)^2, gelu_tanh, silu)."""
     _dev(x, out)
@@ -1075,6 +1133,121 @@ def blocked_product(a, w, out, gate=None):
     return out
 
 
+def decay_product(a, w, out, bias, rate=None, log_scale=None):
+    """Decay factors of a recurrence from a low-rank product: out[m, n] (float32) = exp(-rate[n // per] softplus(a[m] . w[n] +
+    bias[n])) with ``rate`` [N / per], or exp(log_scale * logsigmoid(a[m] . w[n] + bias[n])).  ``a``'s rows may be strided."""
+    _dev(a, w, out, bias, rate)
+    M, K = a.shape
+    N = w.shape[0]
+    _need(tuple(w.shape) == (N, K) and w.is_contiguous() and w.dtype == a.dtype and a.stride(1) == 1, "decay_product: operands")
+    _need(tuple(out.shape) == (M, N) and out.is_contiguous() and out.dtype == torch.float32, "decay_product: out is float32 [M, N]")
+    _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == N, "decay_product: bias")
+    _need((rate is None) != (log_scale is None), "decay_product: a rate or a scale of the logarithm")
+    if rate is not None:
+        _need(rate.dtype == torch.float32 and rate.is_contiguous() and rate.numel() > 0 and N % rate.numel() == 0, "decay_product: rate")
+    check(get_lib().ic_decay_product(a.data_ptr(), a.stride(0), w.data_ptr(), dtype_code(a.dtype), out.data_ptr(), 2 if rate is not None else 3,
+                                     bias.data_ptr(), _ptr(rate), N // rate.numel() if rate is not None else 1,
+                                     float(log_scale) if log_scale is not None else 0.0, M, N, K, _stream()), "decay_product")
+    return out
+
+
+# ---- matrix memories (csrc/matrix_memory.hip) -----------------------------------------------------------------------
+def delta_prep(rows, conv_w, b, out, beta, kv_heads: int, heads: int, key_dim: int, value_dim: int, unit_eps: float, state,
+               state_offset: int, token_req, req_start, state_slots, n_requests: int, single: bool):
+    """rows [T, >= q | k | v] through a convolution (state at ``state_offset``) and silu; q and k heads to unit length: float32
+    ``out`` [T, 2 kv_heads key_dim + heads value_dim]; ``beta`` [T, heads] = sigmoid(b).  ``single``: one token a request."""
+    _dev(rows, conv_w, b, out, beta, state, token_req, req_start, state_slots)
+    T = rows.shape[0]
+    C = 2 * kv_heads * key_dim + heads * value_dim
+    taps = conv_w.shape[1]
+    _need(rows.stride(1) == 1 and rows.shape[1] >= C and b.dtype == rows.dtype and tuple(b.shape) == (T, heads) and b.stride(1) == 1, "delta_prep: rows")
+    _need(conv_w.dtype == torch.float32 and conv_w.is_contiguous() and tuple(conv_w.shape) == (C, taps), "delta_prep: convolution")
+    for v, shape in ((out, (T, C)), (beta, (T, heads))):
+        _need(v.dtype == torch.float32 and v.is_contiguous() and tuple(v.shape) == shape, "delta_prep: results are float32")
+    for t, n in ((token_req, "token_req"), (req_start, "req_start"), (state_slots, "state_slots")):
+        _i32(t, n)
+    _need(token_req.numel() >= T and req_start.numel() >= n_requests + 1 and state_slots.numel() >= n_requests, "delta_prep: lists")
+    _need(not single or T == n_requests, "delta_prep: one token a request")
+    sp, stride = _state_part(state, state_offset)
+    _need(state_offset + (taps - 1) * C <= stride, "delta_prep: state too small")
+    check(get_lib().ic_delta_prep(rows.data_ptr(), rows.stride(0), dtype_code(rows.dtype), conv_w.data_ptr(), taps, b.data_ptr(), b.stride(0),
+                                  out.data_ptr(), beta.data_ptr(), int(kv_heads), int(heads), int(key_dim), int(value_dim), float(unit_eps),
+                                  sp, stride, token_req.data_ptr(), req_start.data_ptr(), state_slots.data_ptr(), T, n_requests,
+                                  1 if single else 0, _stream()), "delta_prep")
+
+
+def memory_gates(z, bias_i, bias_f, cap: float, keep, add, floor, state, state_offset: int, req_start, state_slots, n_requests: int):
+    """Exponential gates against a running maximum (float32, in the state): z [T, 2 H] -> factors ``keep`` and ``add`` and
+    ``floor`` = exp(-maximum), each [T, H]."""
+    _dev(z, bias_i, bias_f, keep, add, floor, state, req_start, state_slots)
+    T, H = keep.shape
+    _need(z.dtype == torch.float32 and tuple(z.shape) == (T, 2 * H) and z.stride(1) == 1, "memory_gates: z")
+    for v in (keep, add, floor):
+        _need(v.dtype == torch.float32 and v.is_contiguous() and tuple(v.shape) == (T, H), "memory_gates: results")
+    for v in (bias_i, bias_f):
+        _need(v.dtype == torch.float32 and v.is_contiguous() and v.numel() == H, "memory_gates: biases")
+    _i32(req_start, "req_start")
+    _i32(state_slots, "state_slots")
+    _need(req_start.numel() >= n_requests + 1 and state_slots.numel() >= n_requests, "memory_gates: lists")
+    sp, stride = _state_part(state, state_offset)
+    _need(state_offset + H <= stride, "memory_gates: state too small")
+    check(get_lib().ic_memory_gates(z.data_ptr(), z.stride(0), bias_i.data_ptr(), bias_f.data_ptr(), float(cap), H, keep.data_ptr(),
+                                    add.data_ptr(), floor.data_ptr(), sp, stride, req_start.data_ptr(), state_slots.data_ptr(), n_requests,
+                                    _stream()), "memory_gates")
+
+
+def matrix_memory(q, k, v, decay, heads: int, kv_heads: int, key_dim: int, value_dim: int, out, state, state_offset: int, req_start,
+                  state_slots, n_requests: int, single: bool, scale=None, delta: bool = False, q_scale: float = 1.0, extra_out=None,
+                  compute_units: int = 256, columns_a_thread=None):
+    """S <- decay S; u = scale (v - S^T k) with ``delta``, else scale v; S <- S + k u^T; out = q_scale S^T q, over every
+    request's rows; the state [heads][value_dim (+ 1)][key_dim] float32 at ``state_offset``.  ``decay`` float32
+    [T, heads * key_dim] or [T, heads]; ``scale`` [T, heads] or None (1).  ``extra_out`` [T, heads]: one more column per head
+    whose v is 1, its read-out.  q, k, v [T, ..] may be views of wider rows.  ``single``: every request brings one token."""
+    _dev(q, k, v, decay, out, state, req_start, state_slots, scale, extra_out)
+    T = q.shape[0]
+    _need(heads % kv_heads == 0, "matrix_memory: heads are not a multiple of the query/key heads")
+    for x, n in ((q, kv_heads * key_dim), (k, kv_heads * key_dim), (v, heads * value_dim)):
+        _need(tuple(x.shape) == (T, n) and x.stride(1) == 1 and x.dtype == q.dtype, "matrix_memory: q, k, v")
+    per_channel = decay.shape[1] == heads * key_dim
+    _need(decay.dtype == torch.float32 and decay.is_contiguous() and decay.shape[0] == T and (per_channel or decay.shape[1] == heads), "matrix_memory: decay")
+    _need(out.dtype == torch.float32 and out.is_contiguous() and tuple(out.shape) == (T, heads * value_dim), "matrix_memory: out")
+    for x in (scale, extra_out):
+        _need(x is None or (x.dtype == torch.float32 and x.is_contiguous() and tuple(x.shape) == (T, heads)), "matrix_memory: per-head rows")
+    _i32(req_start, "req_start")
+    _i32(state_slots, "state_slots")
+    _need(req_start.numel() >= n_requests + 1 and state_slots.numel() >= n_requests, "matrix_memory: lists")
+    _need(not single or T == n_requests, "matrix_memory: one token a request")
+    cols = value_dim + (1 if extra_out is not None else 0)
+    sp, stride = _state_part(state, state_offset)
+    _need(state_offset + heads * cols * key_dim <= stride, "matrix_memory: state too small")
+    if columns_a_thread is None:
+        # two columns a thread halve what a token's vectors cost to read, once one column a thread fills the chip twice
+        columns_a_thread = 2 if -(-cols // 16) * heads * n_requests >= 3 * compute_units else 1
+    check(get_lib().ic_matrix_memory(q.data_ptr(), q.stride(0), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), dtype_code(q.dtype),
+                                     decay.data_ptr(), 1 if per_channel else 0, _ptr(scale), 1 if delta else 0, int(heads),
+                                     heads // kv_heads, int(key_dim), int(value_dim), float(q_scale), out.data_ptr(), _ptr(extra_out), sp,
+                                     stride, req_start.data_ptr(), state_slots.data_ptr(), n_requests, 1 if single else 0,
+                                     int(columns_a_thread), _stream()), "matrix_memory")
+    return out
+
+
+def gated_head_norm(y, z, weight, heads: int, eps: float, out, gate: str = "sigmoid", num=None, floor=None):
+    """out = rms(y / den) * weight * gate(z), head by head (``gate`` "sigmoid" or "silu"); y float32 [T, heads * n], ``weight``
+    [heads * n] or [n] (shared by the heads), den = max(|num|, floor) + 1e-6 with ``num`` and ``floor`` [T, heads], else 1."""
+    _dev(y, z, weight, out, num, floor)
+    T, n = y.shape
+    _need(n % heads == 0 and y.dtype == torch.float32 and y.is_contiguous() and tuple(z.shape) == (T, n) and z.stride(1) == 1
+          and out.dtype == z.dtype and tuple(out.shape) == (T, n) and out.is_contiguous(), "gated_head_norm: layout")
+    _need(weight.dtype == torch.float32 and weight.is_contiguous() and weight.numel() in (n, n // heads), "gated_head_norm: weight")
+    for x in (num, floor):
+        _need(x is None or (x.dtype == torch.float32 and x.is_contiguous() and tuple(x.shape) == (T, heads)), "gated_head_norm: denominators")
+    _need((num is None) == (floor is None), "gated_head_norm: num and floor come together")
+    check(get_lib().ic_gated_head_norm(y.data_ptr(), _ptr(num), _ptr(floor), z.data_ptr(), z.stride(0), dtype_code(z.dtype), weight.data_ptr(),
+                                       1 if weight.numel() != n else 0, T, int(heads), n // heads, float(eps), out.data_ptr(),
+                                       {"sigmoid": 0, "silu": 1}[gate], _stream()), "gated_head_norm")
+    return out
+
+
 # ---- attention through a latent -------------------------------------------------------------------------------------
 def latent_prep(rows, q_rank: int, kv_rank: int, rot_dim: int, qn_w, kvn_w, eps: float, freq, rot_dims: int, positions,
                 cq, cache, slots):
@@ -1333,16 +1506,21 @@ def attention_pooled_prefill(q, out, kcache, vcache, kpool, vpool, block_tables,
 
 
 # ---- routed experts (csrc/moe.hip) ----------------------------------------------------------------------------------------
-def moe_route(logits, top: int, ids, weights, mode: str = "sigmoid", renormalize: bool = False):
+def moe_route(logits, top: int, ids, weights, mode: str = "sigmoid", renormalize: bool = False, correction=None, groups: int = 1,
+              group_keep: int = 1, scale: float = 1.0):
     """ids[t, k], weights[t, k]: the ``top`` experts with the largest scores of float32 ``logits`` [T, E] and their scores
-    (sigmoid of the logit, or the softmax over all experts), renormalised over the chosen ones if asked."""
-    _dev(logits, ids, weights)
+    (sigmoid of the logit, or the softmax over all experts), renormalised over the chosen ones if asked, times ``scale``.
+    ``correction`` [E]: added to the scores for the choice alone.  ``groups``, ``group_keep``: the choice is among the
+    ``group_keep`` best of ``groups`` equal runs of experts (a run is as good as its best corrected score)."""
+    _dev(logits, ids, weights, correction)
     T, E = logits.shape
     _need(logits.dtype == torch.float32 and logits.stride(1) == 1, "moe_route: float32 logits")
     _need(ids.dtype == torch.int32 and ids.is_contiguous() and tuple(ids.shape) == (T, top) and weights.dtype == torch.float32
           and weights.is_contiguous() and tuple(weights.shape) == (T, top), "moe_route: outputs")
+    _need(correction is None or (correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == E), "moe_route: correction")
+    _need(groups >= 1 and E % groups == 0 and 1 <= group_keep <= groups and (groups == 1 or group_keep * (E // groups) >= top), "moe_route: groups")
     check(get_lib().ic_moe_route(logits.data_ptr(), logits.stride(0), T, E, int(top), {"sigmoid": 0, "softmax": 1}[mode],
-                                 1 if renormalize else 0, ids.data_ptr(), weights.data_ptr(), _stream()), "moe_route")
+                                 1 if renormalize else 0, _ptr(correction), int(groups), int(group_keep), float(scale), ids.data_ptr(), weights.data_ptr(), _stream()), "moe_route")
 
 
 def moe_sort(ids, n_experts: int, offsets, order, place):
@@ -1368,33 +1546,42 @@ def moe_gather(h, order, weights, top: int, out):
     return out
 
 
-def moe_expert_product(a, w, offsets, out, glu: bool = False, compute_units: int = 256):
-    """out[s] = a[s] W_e^T for the sorted rows s of every expert e (``offsets`` [E + 1]); ``w`` [E, N or 2N, K].  ``glu``: w
-    holds gate rows then up rows, out = silu(gate) * up.  For few rows: every row chunk streams its expert's matrix."""
+def moe_expert_product(a, w, offsets, out, glu: bool = False, compute_units: int = 256, glu_clamped=None):
+    """out[s] = a[s] W_e^T for the sorted rows s of every expert e (``offsets`` [E + 1] or longer: rows of what lies behind the
+    last expert are left alone); ``w`` [E, N or 2N, K].  ``glu``: w holds gate rows then up rows, out = silu(gate) * up, or with
+    ``glu_clamped`` = (limit, slope) the unit with bounded branches.  For few rows: every row chunk streams its expert's matrix."""
     _dev(a, w, offsets, out)
     E, rows, K = w.shape
     N = rows // 2 if glu else rows
     _need(w.is_contiguous() and a.stride(1) == 1 and a.shape[1] == K and out.stride(1) == 1 and out.shape[1] == N
           and out.shape[0] == a.shape[0] and a.dtype == w.dtype == out.dtype and (not glu or rows % 2 == 0), "moe_expert_product: layout")
     _i32(offsets, "offsets")
-    _need(offsets.numel() == E + 1, "moe_expert_product: offsets")
+    _need(offsets.numel() >= E + 1, "moe_expert_product: offsets")
+    limit, slope = glu_clamped if glu_clamped is not None else (0.0, 0.0)
     check(get_lib().ic_moe_expert_product(a.data_ptr(), a.stride(0), w.data_ptr(), rows * K, dtype_code(a.dtype), offsets.data_ptr(),
-                                          out.data_ptr(), out.stride(0), E, N, K, 1 if glu else 0, int(compute_units), _stream()),
+                                          out.data_ptr(), out.stride(0), E, N, K, 1 if glu else 0, float(limit), float(slope),
+                                          int(compute_units), _stream()),
           "moe_expert_product")
     return out
 
 
-def moe_combine(y, place, weights, shared, top: int, out):
-    """out[t] = sum_k y[place[t * top + k]] * (weights[t * top + k] or 1) + (shared[t] or 0)."""
-    _dev(y, place, weights, shared, out)
+def moe_combine(y, place, weights, shared, top: int, out, own=None, n_routed=None):
+    """out[t] = sum_k y[place[t * top + k]] * (weights[t * top + k] or 1) + (shared[t] or 0); pairs whose place is not below the
+    device integer ``n_routed`` (int32 [1]) take ``own``[t] for y (identity experts)."""
+    _dev(y, place, weights, shared, out, own, n_routed)
     T, d = out.shape
     _need(y.stride(1) == 1 and y.shape[1] == d and out.stride(1) == 1 and y.dtype == out.dtype and place.numel() == T * top
           and y.shape[0] == T * top, "moe_combine: layout")
     _i32(place, "place")
     _need(shared is None or (tuple(shared.shape) == (T, d) and shared.stride(1) == 1 and shared.dtype == out.dtype), "moe_combine: shared")
     _need(weights is None or (weights.dtype == torch.float32 and weights.is_contiguous() and weights.numel() == T * top), "moe_combine: weights")
+    _need((own is None) == (n_routed is None), "moe_combine: own rows come with the number of routed pairs")
+    if own is not None:
+        _need(tuple(own.shape) == (T, d) and own.stride(1) == 1 and own.dtype == out.dtype, "moe_combine: own rows")
+        _i32(n_routed, "n_routed")
     check(get_lib().ic_moe_combine(y.data_ptr(), y.stride(0), dtype_code(y.dtype), place.data_ptr(), _ptr(weights), _ptr(shared),
-                                   shared.stride(0) if shared is not None else 0, T, int(top), d, out.data_ptr(), out.stride(0),
+                                   shared.stride(0) if shared is not None else 0, _ptr(own), own.stride(0) if own is not None else 0,
+                                   _ptr(n_routed), T, int(top), d, out.data_ptr(), out.stride(0),
                                    _stream()), "moe_combine")
     return out
 

@@ -119,6 +119,13 @@ class StreamCopy:
 
 
 @dataclass
+class Branches:
+    """A mixer's result as a sum that is still owed: the (tensor, factor) pairs of its branches.  A mixer with
+    ``yields_branches`` hands it to a block that asks (forward(.., branches=True)) and adds them in its own kernel."""
+    parts: Tuple[Tuple[torch.Tensor, float], ...]
+
+
+@dataclass
 class ResidualTail:
     """What a block asks of a part's LAST projection (a part with ``fuses_tail``): add the part's
     output y to the float32 residual stream, x += alpha * y, and hand back the input of the norm
@@ -128,6 +135,17 @@ class ResidualTail:
     alpha: float
     weight: torch.Tensor
     eps: float
+
+
+def packed_rows(tensors, pack: str, names):
+    """The matrices (or vectors) ``names`` one below the other: as the loader laid them out under ``pack``, or joined here."""
+    packed = tensors.get(pack)
+    if packed is None:
+        mats = [tensors[n] for n in names]
+        if len({m.dtype for m in mats}) > 1:
+            mats = [m.to(torch.float32) for m in mats]
+        packed = torch.cat(mats, dim=0).contiguous()
+    return packed
 
 
 def register_part(category: str, kind: str) -> Callable:
@@ -242,6 +260,12 @@ class Mixer(Part):
     category = "mixer"
     accepts_deferred = False     # forward() takes DeferredRows as h
     fuses_tail = False           # forward() takes tail=ResidualTail and may return DeferredRows
+    yields_branches = False      # forward() takes branches=True and may return Branches
+    # Where a mixer's state begins in its cache slot's state row, and the workspace buffer of its result: a mixer that joins
+    # others sets them for its children.  A mixer that honours both says so with ``relocatable``.
+    relocatable = False
+    state_base = 0
+    out_buffer = "mixer_out"
 
     def cache_need(self) -> CacheNeed:
         return CacheNeed()

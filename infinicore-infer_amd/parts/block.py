@@ -14,7 +14,7 @@ import torch
 
 from ..kernels import ops
 from ..weights.loader import WeightSpec
-from .base import Block, DeferredRows, ResidualTail, StreamCopy, register_part
+from .base import Block, Branches, DeferredRows, ResidualTail, StreamCopy, register_part
 
 
 @register_part("block", "prenorm_residual")
@@ -127,6 +127,47 @@ class OutputNormResidualBlock(Block):
         if self.feed_forward is not None:
             y = self.feed_forward.forward(h, ctx)
             self.feed_forward_norm.forward_into_stream(y, x, copy=copy)
+        return StreamCopy(h)
+
+
+@register_part("block", "sum_norm_residual")
+class SumNormResidualBlock(Block):
+    """x <- norm1(alpha x + mixer(x)); x <- norm2(alpha x + ffn(x)): the norm sits on the residual sum, and the sublayers read
+    the stream itself (the second half only when the layer has a feed-forward).
+
+    The stream is float32.  One row kernel per sublayer (``ops.sum_norm``) forms the sum, its norm, the new stream and the
+    stream's copy in the compute dtype that the next sublayer reads, which the block hands on as ``StreamCopy``.  A mixer
+    of several branches leaves their sum to that kernel (``Branches``)."""
+    graph_safe = True
+    accepts_stream_copy = True
+
+    def __init__(self, name, runtime, mixer=None, mixer_norm=None, feed_forward=None, feed_forward_norm=None, alpha: float = 1.0):
+        super().__init__(name, runtime, mixer, mixer_norm, feed_forward, feed_forward_norm)
+        if mixer is None or mixer_norm is None:
+            raise ValueError("block %s: a block with norms on the sums needs a mixer and its norm" % name)
+        if (feed_forward is None) != (feed_forward_norm is None):
+            raise ValueError("block %s: a feed-forward and its norm come together, or neither" % name)
+        for n in (mixer_norm, feed_forward_norm):
+            if n is not None and n.deferred() is None:
+                raise ValueError("block %s: norm part %s is not a weighted RMS norm" % (name, type(n).__name__))
+        self.alpha = float(alpha)
+
+    def forward(self, x, pending, ctx, cache):
+        copy = None if self.runtime.dtype == x.dtype else ctx.ws.buffer("stream_copy", tuple(x.shape), self.runtime.dtype)
+        if isinstance(pending, StreamCopy):
+            h = pending.values
+        else:
+            if pending is not None:
+                ops.residual_add(x, pending[0], pending[1])
+            h = x if copy is None else copy.copy_(x)
+        y = self.mixer.forward(h, ctx, cache, branches=True) if self.mixer.yields_branches else self.mixer.forward(h, ctx, cache)
+        weight, eps = self.mixer_norm.deferred()
+        ops.sum_norm(y.parts if isinstance(y, Branches) else ((y, 1.0),), self.alpha, weight, x, eps, copy=copy)
+        h = x if copy is None else copy
+        if self.feed_forward is not None:
+            y = self.feed_forward.forward(h, ctx)
+            weight, eps = self.feed_forward_norm.deferred()
+            ops.sum_norm(((y, 1.0),), self.alpha, weight, x, eps, copy=copy)
         return StreamCopy(h)
 
 

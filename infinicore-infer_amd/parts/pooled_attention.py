@@ -21,15 +21,7 @@ from ..kernels import ops
 from ..weights.loader import WeightSpec
 from .base import CacheNeed, Mixer, register_part
 from .linear import linear
-
-
-def pair_frequencies(rot_dims: int, base: float) -> torch.Tensor:
-    """f_i = base^(-2i/rot_dims), i < rot_dims / 2, as float32 [2, rot_dims / 2]: the float64 value rounded, and what the
-    rounding left (the kernel forms the angle from both, so that its error does not grow with the position)."""
-    i = torch.arange(rot_dims // 2, dtype=torch.float64)
-    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / rot_dims)
-    hi = f.to(torch.float32)
-    return torch.stack([hi, (f - hi.double()).to(torch.float32)]).contiguous()
+from .rotary import pair_frequencies
 
 
 @register_part("mixer", "pooled_attention")

@@ -45,6 +45,15 @@ def rotary_tables(head_dim, theta, max_positions, scaling=None, rot_dim=None, mo
     return (torch.cos(ang) * magnitude).to(torch.float32), (torch.sin(ang) * magnitude).to(torch.float32)
 
 
+def pair_frequencies(rot_dims: int, base: float) -> torch.Tensor:
+    """f_i = base^(-2i/rot_dims), i < rot_dims / 2, as float32 [2, rot_dims / 2]: the float64 value rounded, and what the
+    rounding left (the kernel forms the angle from both, so that its error does not grow with the position)."""
+    i = torch.arange(rot_dims // 2, dtype=torch.float64)
+    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / rot_dims)
+    hi = f.to(torch.float32)
+    return torch.stack([hi, (f - hi.double()).to(torch.float32)]).contiguous()
+
+
 _TABLES = {}
 
 

@@ -1,8 +1,10 @@
 """Softmax attention whose keys and values may differ in size per head and whose queries see a span of the
 keys: the last ``window`` keys plus the first ``keep_first`` keys of the sequence (query i sees key j when
-j <= i and (i - j < window or j < keep_first); no window: every earlier key).  Positions do not enter the
-scores.  Options, each a parameter:
+j <= i and (i - j < window or j < keep_first); no window: every earlier key).  Positions enter the scores only with
+a rotation.  Options, each a parameter:
 
+  * a short causal convolution per channel on q, k and v right after the projection (its last inputs are a state per request),
+  * a rotation of the first ``rot_dims`` entries of queries and keys (entry i with entry i + rot_dims / 2), before their norm,
   * biases on the q, k, v projections and on the output projection,
   * a norm on queries and keys to unit root mean square, per head (one weight of the key size, shared by the
     heads, or no weight at all) or over the whole projection before it is cut into heads (a weight of the
@@ -15,15 +17,17 @@ scores.  Options, each a parameter:
   * an output gate: the concatenated heads are multiplied by sigmoid(W_g h) before the output projection.
 
 q, k, v and the gate are rows of ONE projection; a single row kernel then adds the biases, applies the norms,
-mixes the values, and writes keys and values into the paged cache (K and V planes of different widths).  The
+mixes the values, and writes keys and values into the paged cache (K and V planes of different widths); with a
+convolution or a rotation another one applies these, then the norms, and writes the cache.  The
 scores never reach memory: the attention kernels walk the cache with a float32 running softmax.
 """
 import torch
 
 from ..kernels import ops
 from ..weights.loader import WeightSpec
-from .base import CacheNeed, Mixer, register_part
+from .base import CacheNeed, Mixer, packed_rows, register_part
 from .linear import linear
+from .rotary import pair_frequencies
 
 _NORM_MODES = {None: 0, "none": 0, "head": 1, "row": 2}
 _MIX_MODES = {None: 0, "none": 0, "keep": 1, "mix": 2}
@@ -32,18 +36,20 @@ _MIX_MODES = {None: 0, "none": 0, "keep": 1, "mix": 2}
 @register_part("mixer", "span_attention")
 class SpanAttention(Mixer):
     graph_safe = True
+    relocatable = True
     defers_bias = True           # forward(.., defer_bias=True) leaves the output projection's bias to the caller
 
     def __init__(self, name, runtime, hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int,
                  value_dim: int, softmax_scale: float, window=None, keep_first: int = 0, sink: bool = False,
                  qk_norm=None, qk_norm_eps: float = 1e-6, qkv_bias: bool = False, out_bias: bool = False,
                  gate: bool = False, value_mix=None, value_mix_width=None, value_mix_optional: bool = False,
-                 softcap=None, qk_norm_weight: bool = True):
+                 softcap=None, qk_norm_weight: bool = True, conv_taps: int = 0, rot_dims: int = 0, rot_base=None):
         """``sink``: False, True (the constant term exp(0)) or "learned" (one number per head, the tensor ``sink``).
         ``softcap``: None or the cap c > 0.  ``qk_norm_weight`` False: the per-head norm has no weight tensors.
         ``qk_norm``: None, "head" or "row".  ``value_mix``: None, "keep" (this layer's values are the ones later
         layers mix in) or "mix"; all mixing layers of a model have the same kv heads and value size.
-        ``value_mix_optional``: the files may hold the mixing scalar although this layer does not mix."""
+        ``value_mix_optional``: the files may hold the mixing scalar although this layer does not mix.
+        ``conv_taps``: 0 (no convolution) or its taps; ``rot_dims`` / ``rot_base``: the rotation, 0 for none."""
         super().__init__(name, runtime)
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
             raise ValueError("span attention: %d heads are not a multiple of %d kv heads" % (num_heads, num_kv_heads))
@@ -74,13 +80,26 @@ class SpanAttention(Mixer):
         self.qkv_bias, self.out_bias, self.gate = bool(qkv_bias), bool(out_bias), bool(gate)
         self.mix_mode = _MIX_MODES[value_mix]
         self.mix_optional = bool(value_mix_optional)
+        self.taps, self.rot_dims = int(conv_taps or 0), int(rot_dims or 0)
+        if not 0 <= self.taps <= 8:
+            raise ValueError("span attention: at most 8 convolution taps (got %d)" % self.taps)
+        if self.rot_dims < 0 or self.rot_dims % 2 or self.rot_dims > key_dim:
+            raise ValueError("span attention: rot_dims must be even and at most the key size (got %d)" % self.rot_dims)
+        if self.rot_dims and not (rot_base and float(rot_base) > 0):
+            raise ValueError("span attention: a rotation needs a positive base")
+        self.shaped = bool(self.taps or self.rot_dims)
+        if self.shaped and (self.qkv_bias or self.mix_mode or self.norm_mode == 2):
+            raise ValueError("span attention: a convolution or a rotation goes with no norm or the norm per head, without biases and value mixing")
+        self.freq = pair_frequencies(self.rot_dims, rot_base).to(runtime.device) if self.rot_dims else None
+        self.conv_w = None
         self.nq, self.nk, self.nv = self.nh * self.dk, self.nkvh * self.dk, self.nkvh * self.dv
+        self.state_size = max(0, self.taps - 1) * (self.nq + self.nk + self.nv)      # the convolution's last inputs
         self.na = self.nh * self.dv                       # width of the concatenated heads
         self.w_rows = self.w_o = self.b_rows = self.b_o = self.q_norm = self.k_norm = self.mix_lambda = None
 
     def cache_need(self):
-        return CacheNeed("kv", self.nkvh, self.dk, self.window or None, plane_dims=(self.dk, self.dv),
-                         keep_first=self.keep_first)
+        return CacheNeed("kv+state" if self.state_size else "kv", self.nkvh, self.dk, self.window or None, plane_dims=(self.dk, self.dv),
+                         keep_first=self.keep_first, state_shape=(self.state_size,) if self.state_size else ())
 
     def portion_tile_rows(self):
         return ops.attention_prefill_tile_rows()
@@ -103,6 +122,8 @@ class SpanAttention(Mixer):
             specs[n + "v.b"] = WeightSpec((self.nv,), "vector", pack=(bpack, 2), mean=0.0)
         if self.out_bias:
             specs[n + "o.b"] = WeightSpec((d,), "vector", mean=0.0)
+        for i, c in enumerate((self.nq, self.nk, self.nv) if self.taps else ()):
+            specs[n + "qkv"[i] + ".conv"] = WeightSpec((c, self.taps), "vector", pack=(n + "qkv_conv.packed", i), mean=1.0 / self.taps)
         if self.sink_learned:
             specs[n + "sink"] = WeightSpec((self.nh,), "vector", mean=0.0)
         if self.norm_mode and self.norm_weight:
@@ -130,6 +151,8 @@ class SpanAttention(Mixer):
             if b is None:
                 b = torch.cat([tensors[n + s + ".b"].to(torch.float32).reshape(-1) for s in ("q", "k", "v")]).contiguous()
             self.b_rows = b
+        if self.taps:
+            self.conv_w = packed_rows(tensors, n + "qkv_conv.packed", [n + s + ".conv" for s in ("q", "k", "v")])
         self.b_o = tensors[n + "o.b"] if self.out_bias else None
         if self.norm_mode and self.norm_weight:
             self.q_norm, self.k_norm = tensors[n + "q.norm"], tensors[n + "k.norm"]
@@ -149,17 +172,26 @@ class SpanAttention(Mixer):
         linear(h, self.w_rows, rows, rt.gemm_impl, ws=ctx.ws)
         q = ctx.ws.buffer("span_q", (T, self.nq), rt.dtype)
         v_keep = ctx.ws.buffer("value_mix_keep", (T, self.nv), torch.float32) if self.mix_mode else None
-        ops.qk_norm_store(rows, self.b_rows, self.q_norm, self.k_norm, self.norm_mode, self.qk_norm_eps, self.mix_mode,
-                          self.mix_lambda, v_keep, q, cache.k, cache.v, cache.slots if cache.writes else None,
-                          self.nh, self.nkvh, self.dk, self.dv, ctx.page_size)
+        slots = cache.slots if cache.writes else None
+        if self.shaped:
+            ops.conv_rope_norm_store(rows, self.conv_w, ctx.positions, self.freq, self.rot_dims, self.q_norm, self.k_norm,
+                                     self.norm_mode == 1, self.qk_norm_eps, q, cache.k, cache.v, slots, self.nh, self.nkvh, self.dk,
+                                     self.dv, ctx.page_size, cache.state if self.taps else None, self.state_base, ctx.token_req,
+                                     ctx.req_rows, ctx.state_slots, ctx.R, single=ctx.T == ctx.R)
+        else:
+            self._norm_and_store(rows, q, v_keep, ctx, cache, slots)
         out = ctx.ws.buffer("span_out", (T, self.na), rt.dtype)
         gate = rows[:, self.nq + self.nk + self.nv:] if self.gate else None
         self._attend(q, out, gate, ctx, cache)
-        y = ctx.ws.buffer("mixer_out", (T, self.hidden_size), rt.dtype)
+        y = ctx.ws.buffer(self.out_buffer, (T, self.hidden_size), rt.dtype)
         linear(out, self.w_o, y, rt.gemm_impl, ws=ctx.ws)
         if self.b_o is not None and not defer_bias:
             y.add_(self.b_o.to(y.dtype))
         return y
+
+    def _norm_and_store(self, rows, q, v_keep, ctx, cache, slots):
+        ops.qk_norm_store(rows, self.b_rows, self.q_norm, self.k_norm, self.norm_mode, self.qk_norm_eps, self.mix_mode,
+                          self.mix_lambda, v_keep, q, cache.k, cache.v, slots, self.nh, self.nkvh, self.dk, self.dv, ctx.page_size)
 
     def _attend(self, q, out, gate, ctx, cache):
         """Single-token rows go to the split-key kernel, prompt portions to the matrix-core kernel, where the sizes

@@ -23,7 +23,7 @@ import fnmatch
 import glob
 import os
 import time
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Dict, Iterable, List, Optional, Tuple
 
 import torch
@@ -56,6 +56,33 @@ class WeightError(ValueError):
 
 
 @dataclass(frozen=True)
+class FreeDim:
+    """A dimension that the configuration leaves open and the file's tensor decides (the inner size of a low-rank product).
+    All places with the same ``name`` must agree; ``default``: its size where no file is read (random-weights mode)."""
+    name: str
+    default: int
+
+
+def default_shape(shape) -> Tuple[int, ...]:
+    """A spec's shape with every open dimension at its default."""
+    return tuple(s.default if isinstance(s, FreeDim) else int(s) for s in shape)
+
+
+def _resolve_free_dims(specs, stored_shapes):
+    """The specs with every open dimension replaced by what the files hold (its first tensor in the order of the specs decides;
+    a tensor that is absent or of another rank keeps the default, and is reported by the checks that follow)."""
+    sizes: Dict[str, int] = {}
+    for name, spec in specs.items():
+        got = stored_shapes.get(name)
+        if got is not None and len(got) == len(spec.shape):
+            for want, have in zip(spec.shape, got):
+                if isinstance(want, FreeDim):
+                    sizes.setdefault(want.name, int(have))
+    fixed = lambda shape: tuple(sizes.get(s.name, s.default) if isinstance(s, FreeDim) else s for s in shape)
+    return {n: (replace(s, shape=fixed(s.shape)) if any(isinstance(x, FreeDim) for x in s.shape) else s) for n, s in specs.items()}
+
+
+@dataclass(frozen=True)
 class WeightSpec:
     """What a part needs of one tensor.  role: 'matrix' (a GEMM operand or a
     table, keeps its stored dtype), 'vector' (a scale vector, float32) or
@@ -68,7 +95,7 @@ class WeightSpec:
     under that name without copying (fused projections).  ``optional``: the files may lack the
     tensor (it is then absent from the result); when they hold it, it is checked and loaded.
     ``mean``: the value a vector is drawn around in random-weights mode (default 1: a scale; 0 for a bias
-    or a weight stored around zero)."""
+    or a weight stored around zero).  An entry of ``shape`` may be a ``FreeDim``."""
     shape: Tuple[int, ...]
     role: str = "matrix"
     fallback: Optional[str] = None
@@ -180,6 +207,7 @@ def load_weights(model_dir: str, specs: Dict[str, WeightSpec], compute_dtype: to
                 where[name] = path
                 shapes[name] = tuple(sl.get_shape())
                 stored[name] = str(sl.get_dtype())
+    specs = _resolve_free_dims(specs, shapes)
 
     resolved: Dict[str, str] = {}
     missing, wrong, wrong_dtype = [], [], []

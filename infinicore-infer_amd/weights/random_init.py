@@ -25,6 +25,7 @@ import torch
 from safetensors.torch import save_file
 
 from ..config.registry import config_from_dict
+from .loader import default_shape
 
 _M64 = (1 << 64) - 1
 _GOLDEN = 0x9E3779B97F4A7C15
@@ -105,7 +106,7 @@ def random_state_dict(config: dict, seed: int, std: float = 0.02, norm_std: floa
     for name, spec in specs.items():
         if tie and spec.fallback in specs and spec.fallback in out:
             continue                # a tied tensor is not written: the loader takes the tensor it falls back to
-        t = _draw(seed, name, spec.shape, spec.role, std, norm_std, device, spec.mean)
+        t = _draw(seed, name, default_shape(spec.shape), spec.role, std, norm_std, device, spec.mean)
         out[name] = (t if spec.role == "vector" else t.to(dtype)).contiguous()
     return out
 
@@ -121,7 +122,7 @@ def init_random_weights(model, seed: int, std: float = 0.02, norm_std: float = 0
         if tie and spec.fallback in specs and spec.fallback in tensors:
             tensors[name] = tensors[spec.fallback]
             continue
-        t = _draw(seed, name, spec.shape, spec.role, std, norm_std, rt.device, spec.mean)
+        t = _draw(seed, name, default_shape(spec.shape), spec.role, std, norm_std, rt.device, spec.mean)
         tensors[name] = t if spec.role == "vector" else t.to(rt.dtype)
     model.load_weights(tensors)
 

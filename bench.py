@@ -12,7 +12,7 @@ seeded uniform-random token ids.  One JSON line is printed.
   --workload mixed   the 1B shape's workload: 64 requests, prompts of 128..2,048 tokens, portions of 512
   --workload long    the 8B shape's workload: 4 prompts of 16,384 tokens, then decoding
   --direct           decode by calling the step function directly, without the scheduler
-  --workload designs the Fopezen, Mezinex, Daborax and Fizelix decoders beside the MiniCPM decoder at equal layer sizes
+  --workload designs the Fopezen, Mezinex, Daborax, Fizelix and Pekarax decoders beside the MiniCPM decoder at equal layer sizes
                      (a few layers of three real models' sizes): prefill and decode throughput of each, with the fraction
                      of the memory or matrix-core peak it reaches (--only <design>: one of them, for a profiler)
 """
@@ -241,7 +241,21 @@ def _design_configs(z, layers):
     fiz = dict(architecture="Fizelix", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-5), embedding=dict(scale=1.0),
                logit_scale=1.0, token_side=dict(dim=64),
                layers=[dict(type=fiz_kinds[i % 4][0], mixer=fiz_kinds[i % 4][1], mlp=fiz_kinds[i % 4][2]) for i in range(layers)])
-    return {"minicpm": mini, "fopezen": fop, "mezinex": mez, "daborax": dab, "fizelix": fiz}
+    # Pekarax at the same width: the delta rule in as many heads of the row's size, linear attention with half as many heads of
+    # that key size and twice the value size, attention with the row's heads beside a matrix memory of a quarter as many heads
+    # (keys of twice, values of four times the row's head size), the delta rule again; every feed-forward routes, three of
+    # fourteen experts of a quarter of the row's size and two identity experts, out of the two best of four groups
+    dl = dict(heads=z["heads"], kv_heads=z["heads"], dim=z["dim"], vdim=z["dim"], conv=4)
+    gla = dict(heads=z["heads"] // 2, dim=z["dim"], vdim=2 * z["dim"], tau=16.0)
+    par = dict(left=dict(heads=z["heads"], kv_heads=z["kv"], dim=z["dim"], vdim=z["dim"], conv=4, scale=z["dim"] ** -0.5,
+                         rot=dict(base=500000.0, dims=z["dim"])),
+               right=dict(heads=z["heads"] // 4, dim=2 * z["dim"], vdim=4 * z["dim"], gate_cap=15.0), left_scale=0.7, right_scale=0.7)
+    pek_moe = dict(kind="moe", router=dict(experts=14, identity=2, top=3, groups=dict(count=4, keep=2), scale=2.0),
+                   expert=dict(ff=z["ff"] // 4, limit=7.0))
+    pek_kinds = [("channel_delta", dl), ("gla", gla), ("parallel", par), ("channel_delta", dl)]
+    pek = dict(architecture="Pekarax", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-5), postln_alpha=2.0,
+               layers=[dict(type=pek_kinds[i % 4][0], mixer=pek_kinds[i % 4][1], mlp=pek_moe) for i in range(layers)])
+    return {"minicpm": mini, "fopezen": fop, "mezinex": mez, "daborax": dab, "fizelix": fiz, "pekarax": pek}
 
 
 def _design_numbers(design, z, layers, kinds=None):
@@ -254,6 +268,8 @@ def _design_numbers(design, z, layers, kinds=None):
         return _daborax_numbers(z, layers)
     if design == "fizelix":
         return _fizelix_numbers(z, layers)
+    if design == "pekarax":
+        return _pekarax_numbers(z, layers)
     if design == "minicpm":
         per_layer = (H + 2 * G) * dk * d + H * dk * d + 3 * d * ff
         kv = lambda n: 2 * layers * G * dk * eb * n
@@ -372,6 +388,48 @@ def _fizelix_numbers(z, layers):
     kv = lambda n: sum(g * eb * seen(n, w, p) for _, g, w, p in spans) + state_bytes
     flops = lambda T: (T * (per_tok_lin + scan) + sum(2.0 * h * sum(seen(i + 1, w, p) for i in range(T)) for h, _, w, p in spans)
                        + 2.0 * V * d)
+    return weights, kv, flops
+
+
+def _pekarax_numbers(z, layers):
+    """As ``_fizelix_numbers`` for the Pekarax configuration of ``_design_configs`` (low-rank products at their default inner
+    sizes: the key and the value size for the delta rule, 16 for linear attention; identity experts read nothing)."""
+    cfg = _design_configs(z, layers)["pekarax"]
+    d, V, eb = z["width"], z["vocab"], _elem_bytes()
+    fixed, per_tok_lin, scan, state_bytes, heads_kv = V * d, 0.0, 0.0, 0.0, 0
+    pairs = 0.0        # query heads * (key + value size) of the attention
+    routed = []
+    for l in cfg["layers"]:
+        m, r = l["mixer"], l["mlp"]["router"]
+        if l["type"] == "channel_delta":
+            H, G, dk, dv = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            n = (2 * G * dk + H * dv + dk + dv + H) * d + H * dk * dk + H * dv * dv + d * H * dv
+            state_bytes += 2 * 4 * (H * dk * dv + (m["conv"] - 1) * (2 * G * dk + H * dv))
+            scan += 8.0 * H * dk * dv
+        elif l["type"] == "gla":
+            H, dk, dv = m["heads"], m["dim"], m["vdim"]
+            n = (2 * H * dk + 2 * H * dv + 16) * d + 16 * H * dk + d * H * dv
+            state_bytes += 2 * 4 * H * dk * dv
+            scan += 6.0 * H * dk * dv
+        else:
+            a, b = m["left"], m["right"]
+            H, G, dk, dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            n = (H * dk + G * (dk + dv)) * d + d * H * dv
+            heads_kv += G * (dk + dv)
+            pairs += H * (dk + dv)
+            state_bytes += 2 * 4 * (a["conv"] - 1) * (H * dk + G * (dk + dv))
+            H, dk, dv = b["heads"], b["dim"], b["vdim"]
+            n += (2 * H * dk + 2 * H * dv + 2 * H) * d + d * H * dv
+            state_bytes += 2 * 4 * H * dk * (dv + 1)
+            scan += 6.0 * H * dk * (dv + 1)
+        total, one = r["experts"] + r["identity"], 3 * d * l["mlp"]["expert"]["ff"]
+        n += total * d
+        fixed += n
+        per_tok_lin += 2.0 * (n + r["top"] * r["experts"] / total * one)
+        routed.append((r["experts"], r["top"] / total, one))
+    weights = lambda batch: eb * (fixed + sum(E * (1.0 - (1.0 - p) ** batch) * one for E, p, one in routed))
+    kv = lambda n: heads_kv * eb * n + state_bytes
+    flops = lambda T: T * (per_tok_lin + scan) + pairs * 2.0 * (T * (T + 1) / 2) + 2.0 * V * d
     return weights, kv, flops
 
 
@@ -510,7 +568,7 @@ def main():
     ap.add_argument("--layers", type=int, default=0, help="fewer layers than the shape has (0: all)")
     ap.add_argument("--shape", default=None, choices=sorted(SHAPES), help="2b is the benchmark's configuration (default; 1b for --workload mixed)")
     ap.add_argument("--sizes", default=None, help="--workload designs: comma-separated sizes (default: all of 2b-like, 8b-like, 1b-like)")
-    ap.add_argument("--only", default=None, choices=["fopezen", "minicpm", "mezinex", "daborax", "fizelix"], help="--workload designs: one design only")
+    ap.add_argument("--only", default=None, choices=["fopezen", "minicpm", "mezinex", "daborax", "fizelix", "pekarax"], help="--workload designs: one design only")
     ap.add_argument("--workload", default="decode", choices=["decode", "mixed", "long", "designs"],
                     help="decode: the benchmark (prefill of one prompt, decode steps at fixed batches); "
                          "mixed: 64 requests of 128..2048 prompt tokens through the scheduler, --steps tokens generated each; "

@@ -213,19 +213,20 @@ def sum_then_norm(x, y, w, alpha, eps):
     return unit_rms(alpha * x + y, eps) * (1.0 + w)
 
 
-def forward(cfg, W, tokens, dtype=torch.float64, layers_out=None):
-    """Logits [T, vocab] of one whole sequence.  ``layers_out``: a list that receives the residual stream after every layer."""
+def forward(cfg, W, tokens, dtype=torch.float64, layers_out=None, rnd=lambda x: x):
+    """Logits [T, vocab] of one whole sequence.  ``layers_out``: a list that receives the residual stream after every layer.
+    ``rnd``: applied to what every sublayer reads and returns (a rounding shows how far rounding alone moves the logits)."""
     W = {k: (v.to(dtype) if v.is_floating_point() else v) for k, v in W.items()}
     eps, alpha = cfg["norm"]["eps"], cfg["postln_alpha"]
     x = W["embed"][torch.as_tensor(list(tokens), dtype=torch.long)]
     for i, l in enumerate(cfg["layers"]):
         p = "l%d." % i
-        x = sum_then_norm(x, run_mixer(x, W, p + "mix.", l["type"], l["mixer"], eps), W[p + "norm1"], alpha, eps)
+        x = sum_then_norm(x, rnd(run_mixer(rnd(x), W, p + "mix.", l["type"], l["mixer"], eps)), W[p + "norm1"], alpha, eps)
         if l.get("mlp"):
-            x = sum_then_norm(x, routed_experts(x, W, p + "mlp.", l["mlp"]), W[p + "norm2"], alpha, eps)
+            x = sum_then_norm(x, rnd(routed_experts(rnd(x), W, p + "mlp.", l["mlp"])), W[p + "norm2"], alpha, eps)
         if layers_out is not None:
             layers_out.append(x.clone())
-    return (unit_rms(x, eps) * (1.0 + W["final.norm"])) @ W["head"].T
+    return rnd(unit_rms(x, eps) * (1.0 + W["final.norm"])) @ W["head"].T
 
 
 # ---- random weights for the tests -------------------------------------------------------------------------

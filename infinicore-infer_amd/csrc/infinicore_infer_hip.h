@@ -184,7 +184,7 @@ int ic_sum_norm(const void* ya, float sa, const void* yb, float sb, int dtype, f
 
 // ---- matrix_memory.hip: recurrences with a matrix state per head, decays per key channel or per head, the delta rule --------
 int ic_delta_prep(const void* rows, int row_stride, int dtype, const float* w, int taps, const void* b, int b_stride, float* out, float* beta, int G, int H, int dk, int dv, float unit_eps, float* state, long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int T, int R, int single, hipStream_t stream);
-int ic_memory_gates(const float* z, int z_stride, const float* bi, const float* bf, float cap, int H, float* keep, float* add, float* floor_, float* state, long long state_stride, const int* req_start, const int* state_slots, int R, hipStream_t stream);
+int ic_memory_gates(const float* z, int z_stride, const float* bi, const float* bf, float cap, int H, float* keep, float* add, float* floor_, float* state, long long state_stride, const int* req_start, const int* state_slots, int T, int R, hipStream_t stream);
 int ic_matrix_memory(const void* q, int q_stride, const void* k, int k_stride, const void* v, int v_stride, int dtype, const float* decay, int per_channel, const float* scale, int delta, int H, int per, int dk, int dv, float q_scale, float* out, float* extra_out, float* state, long long state_stride, const int* req_start, const int* state_slots, int R, int single, int columns_a_thread, hipStream_t stream);
 int ic_gated_head_norm(const float* y, const float* num, const float* floor_, const void* z, int z_stride, int dtype, const float* w, int w_shared, int T, int H, int dv, float eps, void* out, int gate, hipStream_t stream);
 

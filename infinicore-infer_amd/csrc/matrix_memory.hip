@@ -20,6 +20,9 @@
 __device__ __forceinline__ float mm_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 __device__ __forceinline__ float mm_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float mm_silu(float z) { return z / (1.0f + expf(-z)); }
+// Activations with the hardware's exponential and reciprocal (a last place or two off).
+__device__ __forceinline__ float mm_sigmoid_fast(float z) { return __builtin_amdgcn_rcpf(1.0f + __expf(-z)); }
+__device__ __forceinline__ float mm_silu_fast(float z) { return z * mm_sigmoid_fast(z); }
 
 // ---------------------------------------------------------------------------------------------
 // rows[t] = [q (G dk) | k (G dk) | v (H dv) | ..]: every channel passes the convolution and silu; q and k heads are then
@@ -69,6 +72,101 @@ delta_prep_kernel(const T* __restrict__ rows, int row_stride, const float* __res
     }
 }
 
+// The same for portions: a wave a head and kPrepTile consecutive tokens, two neighbouring channels a lane (n at most 128 NJ,
+// even); every row is read once and waits in registers for the tokens behind it.
+constexpr int kPrepTile = 16;
+
+template <typename T> __device__ __forceinline__ float2 load_pair(const T* p) {
+    if (sizeof(T) == 4) return *reinterpret_cast<const float2*>(p);
+    const uint32_t v = *reinterpret_cast<const uint32_t*>(p);
+    return make_float2(__uint_as_float(v << 16), __uint_as_float(v & 0xffff0000u));
+}
+
+template <typename T, int TMAX, int NJ>
+__global__ void __launch_bounds__(256)
+delta_prep_tile_kernel(const T* __restrict__ rows, int row_stride, const float* __restrict__ w, int taps, const T* __restrict__ b,
+                       int b_stride, float* __restrict__ out, float* __restrict__ beta, int G, int H, int dk, int dv, float unit_eps,
+                       const float* __restrict__ state, long long state_stride, const int* __restrict__ token_req,
+                       const int* __restrict__ req_start, const int* __restrict__ state_slots, int n_tokens) {
+    const int lane = threadIdx.x & 63, head = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int t0 = blockIdx.x * kPrepTile, t1 = min(n_tokens, t0 + kPrepTile);
+    const int C = 2 * G * dk + H * dv;
+    if (head > 2 * G + H) return;
+    if (head == 2 * G + H) {
+        for (int t = t0; t < t1; ++t)
+            for (int i = lane; i < H; i += 64) beta[(size_t)t * H + i] = mm_sigmoid(to_f32(b[(size_t)t * b_stride + i]));
+        return;
+    }
+    const bool unit = head < 2 * G;
+    const int n = unit ? dk : dv, c0 = unit ? head * dk : 2 * G * dk + (head - 2 * G) * dv;
+    ConvWindow<T, TMAX> win[NJ][2];
+#pragma unroll
+    for (int j = 0; j < NJ; ++j) {
+        const int e = 2 * (lane + 64 * j), c = e < n ? c0 + e : c0;
+        win[j][0].weights(w, taps, c);
+        win[j][1].weights(w, taps, c + 1);
+    }
+    int next = t0;                                                   // the row where the window is filled anew
+    constexpr int AHEAD = 8;                                         // rows on their way while others are computed on
+    for (int ta = t0; ta < t1; ta += AHEAD) {
+        float2 in[AHEAD][NJ];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i)
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+                const int e = 2 * (lane + 64 * j);
+                in[i][j] = (ta + i < t1 && e < n) ? load_pair(rows + (size_t)(ta + i) * row_stride + c0 + e) : make_float2(0.f, 0.f);
+            }
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {
+            const int t = ta + i;
+            if (t >= t1) break;
+            if (t == next) {
+                const int r = token_req[t], start = req_start[r];
+                next = req_start[r + 1];
+                const float* st = state + (long long)state_slots[r] * state_stride;
+#pragma unroll
+                for (int j = 0; j < NJ; ++j) {
+                    const int e = 2 * (lane + 64 * j), c = e < n ? c0 + e : c0;
+                    win[j][0].restart(rows, row_stride, taps, C, st, t, start, c);
+                    win[j][1].restart(rows, row_stride, taps, C, st, t, start, c + 1);
+                }
+            }
+            float2 y[NJ];
+            float ss = 0.f;
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+                y[j] = make_float2(mm_silu_fast(win[j][0].next(in[i][j].x)), mm_silu_fast(win[j][1].next(in[i][j].y)));
+                if (2 * (lane + 64 * j) < n) ss += y[j].x * y[j].x + y[j].y * y[j].y;
+            }
+            const float f = unit ? __builtin_amdgcn_rsqf(group_sum<64>(ss) + unit_eps) : 1.f;
+            float* o = out + (size_t)t * C + c0;
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+                const int e = 2 * (lane + 64 * j);
+                if (e < n) *reinterpret_cast<float2*>(o + e) = make_float2(y[j].x * f, y[j].y * f);
+            }
+        }
+    }
+}
+
+// Launches the tile kernel where it takes the sizes.
+template <typename T>
+static bool delta_prep_tiles(const T* rows, int row_stride, const float* w, int taps, const T* b, int b_stride, float* out, float* beta,
+                             int G, int H, int dk, int dv, float unit_eps, const float* state, long long state_stride,
+                             const int* token_req, const int* req_start, const int* state_slots, int T_, hipStream_t stream) {
+    const int n = dk > dv ? dk : dv;
+    if (T_ < 64 || n > 256 || dk % 2 || dv % 2 || row_stride % 2 || (uintptr_t)rows % (2 * sizeof(T)) || (uintptr_t)out % 8) return false;
+    dim3 grid((T_ + kPrepTile - 1) / kPrepTile, (2 * G + H + 1 + 3) / 4), block(256);
+#define IC_DP(TM, NJ_)                                                                                                          \
+    hipLaunchKernelGGL((delta_prep_tile_kernel<T, TM, NJ_>), grid, block, 0, stream, rows, row_stride, w, taps, b, b_stride, out, \
+                       beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, T_)
+    if (taps <= 4) { if (n <= 128) IC_DP(4, 1); else IC_DP(4, 2); }
+    else { if (n <= 128) IC_DP(8, 1); else IC_DP(8, 2); }
+#undef IC_DP
+    return true;
+}
+
 IC_EXPORT int ic_delta_prep(const void* rows, int row_stride, int dtype, const float* w, int taps, const void* b, int b_stride,
                             float* out, float* beta, int G, int H, int dk, int dv, float unit_eps, float* state,
                             long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int T,
@@ -80,13 +178,17 @@ IC_EXPORT int ic_delta_prep(const void* rows, int row_stride, int dtype, const f
     const int C = 2 * G * dk + H * dv;
     dim3 grid(T, (2 * G + H + 1 + 3) / 4), block(256), sgrid((C + 255) / 256, R);
     if (dtype == IC_F32) {
-        hipLaunchKernelGGL(delta_prep_kernel<float>, grid, block, 0, stream, (const float*)rows, row_stride, w, taps, (const float*)b,
+        if (single || !delta_prep_tiles<float>((const float*)rows, row_stride, w, taps, (const float*)b, b_stride, out, beta, G, H, dk, dv, unit_eps,
+                                           state, state_stride, token_req, req_start, state_slots, T, stream))
+            hipLaunchKernelGGL(delta_prep_kernel<float>, grid, block, 0, stream, (const float*)rows, row_stride, w, taps, (const float*)b,
                            b_stride, out, beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, single);
         if (taps > 1 && !single)
             hipLaunchKernelGGL(conv_state_kernel<float>, sgrid, block, 0, stream, (const float*)rows, row_stride, nullptr, taps, C,
                                state, state_stride, req_start, state_slots);
     } else if (dtype == IC_BF16) {
-        hipLaunchKernelGGL(delta_prep_kernel<bf16>, grid, block, 0, stream, (const bf16*)rows, row_stride, w, taps, (const bf16*)b,
+        if (single || !delta_prep_tiles<bf16>((const bf16*)rows, row_stride, w, taps, (const bf16*)b, b_stride, out, beta, G, H, dk, dv, unit_eps,
+                                           state, state_stride, token_req, req_start, state_slots, T, stream))
+            hipLaunchKernelGGL(delta_prep_kernel<bf16>, grid, block, 0, stream, (const bf16*)rows, row_stride, w, taps, (const bf16*)b,
                            b_stride, out, beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, single);
         if (taps > 1 && !single)
             hipLaunchKernelGGL(conv_state_kernel<bf16>, sgrid, block, 0, stream, (const bf16*)rows, row_stride, nullptr, taps, C,
@@ -100,20 +202,23 @@ IC_EXPORT int ic_delta_prep(const void* rows, int row_stride, int dtype, const f
 // Exponential gates.  z [T, 2 H] float32 holds the input gates' pre-activations, then the forget gates'.
 //   i = cap tanh((z_i + b_i) / cap),  f = logsigmoid(cap tanh((z_f + b_f) / cap)),  m_t = max(f_t + m_(t-1), i_t)
 //   keep[t, h] = exp(f_t + m_(t-1) - m_t),  add[t, h] = exp(i_t - m_t),  floor[t, h] = exp(-m_t)
-// A wave per (request, head) takes 64 tokens at a time: the pairs (a, b) = (sum of f, largest i + later f) of a run of
-// tokens combine as (a1 + a2, max(b1 + a2, b2)), and m_t = max(m_0 + a, b).  m_0 lives in the state (zero at the start).
+// A block per (request, head) takes its width in tokens at a time: the pairs (a, b) = (sum of f, largest i + later f) of a
+// run of tokens combine as (a1 + a2, max(b1 + a2, b2)), and m_t = max(m_0 + a, b).  m_0 lives in the state (zero at the start).
 // ---------------------------------------------------------------------------------------------
-__global__ void __launch_bounds__(64)
+template <int WAVES>
+__global__ void __launch_bounds__(64 * WAVES)
 memory_gates_kernel(const float* __restrict__ z, int z_stride, const float* __restrict__ bi, const float* __restrict__ bf, float cap,
                     int H, float* __restrict__ keep, float* __restrict__ add, float* __restrict__ floor_, float* __restrict__ state,
                     long long state_stride, const int* __restrict__ req_start, const int* __restrict__ state_slots) {
-    const int h = blockIdx.x, r = blockIdx.y, lane = threadIdx.x;
+    __shared__ float a_s[2][WAVES], b_s[2][WAVES];
+    const int h = blockIdx.x, r = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int end = req_start[r + 1];
     float* st = state + (long long)state_slots[r] * state_stride + h;
     float m0 = *st;
     const float b_i = bi[h], b_f = bf[h];
-    for (int t0 = req_start[r]; t0 < end; t0 += 64) {
-        const int t = t0 + lane;
+    int half = 0;
+    for (int t0 = req_start[r]; t0 < end; t0 += 64 * WAVES, half ^= 1) {
+        const int t = t0 + threadIdx.x;
         const bool ok = t < end;
         float li = 0.f, lf = 0.f;
         if (ok) {
@@ -130,27 +235,46 @@ memory_gates_kernel(const float* __restrict__ z, int z_stride, const float* __re
                 a = a1 + a;
             }
         }
-        const float m = fmaxf(m0 + a, b);
+        float mw = m0;                                               // the maximum before this wave's tokens, and behind the block's
+        if (WAVES > 1) {
+            if (lane == 63) {
+                a_s[half][wave] = a;
+                b_s[half][wave] = b;
+            }
+            __syncthreads();
+            float all = m0;
+#pragma unroll
+            for (int w = 0; w < WAVES; ++w) {
+                if (w == wave) mw = all;
+                all = fmaxf(all + a_s[half][w], b_s[half][w]);
+            }
+            m0 = all;
+        }
+        const float m = fmaxf(mw + a, b);
         const float before = __shfl_up(m, 1, kWave);
-        const float m_prev = lane ? before : m0;
+        const float m_prev = lane ? before : mw;
         if (ok) {
             const size_t i = (size_t)t * H + h;
             keep[i] = expf(lf + m_prev - m);
             add[i] = expf(li - m);
             floor_[i] = expf(-m);
         }
-        m0 = __shfl(m, min(63, end - 1 - t0), kWave);
+        if (WAVES == 1) m0 = __shfl(m, 63, kWave);
     }
-    if (lane == 0) *st = m0;
+    if (threadIdx.x == 0) *st = m0;
 }
 
 IC_EXPORT int ic_memory_gates(const float* z, int z_stride, const float* bi, const float* bf, float cap, int H, float* keep,
                               float* add, float* floor_, float* state, long long state_stride, const int* req_start,
-                              const int* state_slots, int R, hipStream_t stream) {
+                              const int* state_slots, int T, int R, hipStream_t stream) {
     if (R <= 0) return IC_OK;
-    if (H <= 0 || z_stride < 2 * H || !(cap > 0.f) || !state) return IC_ERR_ARG;
-    hipLaunchKernelGGL(memory_gates_kernel, dim3(H, R), dim3(64), 0, stream, z, z_stride, bi, bf, cap, H, keep, add, floor_, state,
-                       state_stride, req_start, state_slots);
+    if (H <= 0 || R > 65535 || z_stride < 2 * H || !(cap > 0.f) || !state) return IC_ERR_ARG;
+    if (T >= 256)                                                    // (some request brings many tokens, most likely)
+        hipLaunchKernelGGL(memory_gates_kernel<16>, dim3(H, R), dim3(1024), 0, stream, z, z_stride, bi, bf, cap, H, keep, add, floor_, state,
+                           state_stride, req_start, state_slots);
+    else
+        hipLaunchKernelGGL(memory_gates_kernel<1>, dim3(H, R), dim3(64), 0, stream, z, z_stride, bi, bf, cap, H, keep, add, floor_, state,
+                           state_stride, req_start, state_slots);
     return ic_launch_status();
 }
 
@@ -508,7 +632,7 @@ __global__ void __launch_bounds__(256)
 gated_head_norm_kernel(const float* __restrict__ y, const float* __restrict__ num, const float* __restrict__ floor_,
                        const T* __restrict__ z, int z_stride, const float* __restrict__ w, int w_shared, int H, int dv, float eps,
                        T* __restrict__ out, int gate, int n_heads_total) {
-    const int lane = threadIdx.x & 63, item = blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63, item = blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     if (item >= n_heads_total) return;
     const int t = item / H, h = item - t * H;
     const float* yr = y + (size_t)item * dv;
@@ -529,7 +653,7 @@ gated_head_norm_kernel(const float* __restrict__ y, const float* __restrict__ nu
     const float r = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
     auto put = [&](int e, float v) {
         const float g = to_f32(zr[e]);
-        o[e] = from_f32<T>(v * r * wr[e] * (gate ? mm_silu(g) : mm_sigmoid(g)));
+        o[e] = from_f32<T>(v * r * wr[e] * (gate ? mm_silu_fast(g) : mm_sigmoid_fast(g)));
     };
 #pragma unroll
     for (int j = 0; j < KEEP; ++j) {

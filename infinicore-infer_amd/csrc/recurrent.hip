@@ -8,6 +8,12 @@
 #include "short_conv.h"
 
 __device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// The same with the hardware's exponential and logarithm; log(1 + x) = x log(u) / (u - 1) with u = 1 + x as rounded keeps the
+// relative accuracy for small x (Goldberg, "What every computer scientist should know about floating-point arithmetic").
+__device__ __forceinline__ float softplus_fast(float z) {
+    const float x = __expf(-fabsf(z)), u = 1.0f + x, d = u - 1.0f;
+    return fmaxf(z, 0.f) + (d > 0.f ? x * __logf(u) * __frcp_rn(d) : x);
+}
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float gelu_tanh_f(float z) {
@@ -421,8 +427,8 @@ template <typename T> struct BpEpilogue {
         if (kind == 0) return v;
         if (kind == 1) return v * sigmoid_f(to_f32(gate[(size_t)m * gate_stride + at]));
         v += bias[n];
-        if (kind == 2) return expf(-rate[n / per] * softplus_f(v));
-        return expf(-c * softplus_f(-v));
+        if (kind == 2) return __expf(-rate[n / per] * softplus_fast(v));
+        return __expf(-c * softplus_fast(-v));
     }
 };
 
@@ -628,6 +634,36 @@ IC_EXPORT int ic_blocked_product(const void* A, int lda, int a_step, const void*
                                  hipStream_t stream) {
     return blocked_product(A, lda, a_step, W, dtype, C, c_dtype, ldc, c_step, gate ? 1 : 0, gate, gate_stride, nullptr, nullptr, 1, 0.f, M,
                            N, K, B, stream);
+}
+
+// The epilogue alone, in place on a product's float32 results [M, N]: four entries a thread where N is made of such pieces.
+template <int V>
+__global__ void __launch_bounds__(256)
+decay_rows_kernel(float* __restrict__ C, BpEpilogue<float> ep, int M, int N) {
+    const long long i = ((long long)blockIdx.x * 256 + threadIdx.x) * V;
+    if (i >= (long long)M * N) return;
+    const int n = (int)(i % N);
+    if (V == 4) {
+        float4 v = *reinterpret_cast<const float4*>(C + i);
+        v.x = ep(v.x, 0, 0, n);
+        v.y = ep(v.y, 0, 0, n + 1);
+        v.z = ep(v.z, 0, 0, n + 2);
+        v.w = ep(v.w, 0, 0, n + 3);
+        *reinterpret_cast<float4*>(C + i) = v;
+    } else
+        C[i] = ep(C[i], 0, 0, n);
+}
+
+IC_EXPORT int ic_decay_rows(float* C, int kind, const float* bias, const float* rate, int per, float c, int M, int N, hipStream_t stream) {
+    if (M <= 0) return IC_OK;
+    if ((kind != 2 && kind != 3) || !C || !bias || N <= 0 || (kind == 2 && (!rate || per <= 0))) return IC_ERR_ARG;
+    const BpEpilogue<float> ep{kind, nullptr, 0, bias, rate, per > 0 ? per : 1, c};
+    const bool vec = N % 4 == 0 && ((uintptr_t)C & 15) == 0;
+    const long long threads = (long long)M * N / (vec ? 4 : 1), blocks = (threads + 255) / 256;
+    if (blocks > 0x7fffffff) return IC_ERR_TOO_LARGE;
+    if (vec) hipLaunchKernelGGL(decay_rows_kernel<4>, dim3((unsigned)blocks), dim3(256), 0, stream, C, ep, M, N);
+    else hipLaunchKernelGGL(decay_rows_kernel<1>, dim3((unsigned)blocks), dim3(256), 0, stream, C, ep, M, N);
+    return ic_launch_status();
 }
 
 // C[m, n] = the decay factor of A[m] . W[n] (float32): kind 2 or 3 of the epilogues.

@@ -44,3 +44,38 @@ conv_state_kernel(const T* __restrict__ xin, int xin_stride, const float* __rest
     }
     for (int k = 0; k < taps - 1; ++k) st[(size_t)k * C + c] = nv[k];
 }
+
+// One channel's convolution over consecutive tokens, its weights and last inputs in registers (TMAX at least the taps; what a
+// shorter convolution lacks has weight zero).
+template <typename T, int TMAX> struct ConvWindow {
+    float w[TMAX], x[TMAX];
+    __device__ __forceinline__ void weights(const float* __restrict__ cw, int taps, int c) {
+#pragma unroll
+        for (int j = 0; j < TMAX; ++j) {
+            const int k = j - (TMAX - taps);
+            w[j] = k >= 0 ? cw[(size_t)c * taps + k] : 0.f;
+            x[j] = 0.f;
+        }
+    }
+    // The inputs before token t of a request that starts at row `start`: earlier rows of the step, then its state.
+    __device__ __forceinline__ void restart(const T* __restrict__ rows, int stride, int taps, int C, const float* __restrict__ st, int t,
+                                            int start, int c) {
+#pragma unroll
+        for (int j = 1; j < TMAX; ++j) {
+            const int back = TMAX - j, src = t - back;
+            float v = 0.f;
+            if (back < taps) v = src >= start ? to_f32(rows[(size_t)src * stride + c]) : st[(size_t)(taps - 1 - (start - src)) * C + c];
+            x[j] = v;
+        }
+    }
+    __device__ __forceinline__ float next(float v) {
+        float acc = 0.f;
+#pragma unroll
+        for (int j = 0; j + 1 < TMAX; ++j) {
+            x[j] = x[j + 1];
+            acc += w[j] * x[j];
+        }
+        x[TMAX - 1] = v;
+        return acc + w[TMAX - 1] * v;
+    }
+};

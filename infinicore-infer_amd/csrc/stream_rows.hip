@@ -441,10 +441,9 @@ IC_EXPORT int ic_qk_norm_store(const void* rows, int row_stride, int dtype, cons
 //   [2, rot_dims / 2], the frequency and what its rounding left; rot_dims 0: no rotation), then norm 1: unit root mean
 //   square over the head's dk entries, times w[dk] (null: no weight);
 //   q -> q_out[t], k and v -> the cache at slots[t] (null: q only).
-// grid (T, ceil(heads of q, k, v / kRopeHeads)), a wave takes heads in turn: the token's angles are formed once a block.
+// grid (T, ceil(heads of q, k, v / heads_a_block)), a wave takes heads in turn: the token's angles are formed once a block.
 // single: every request brings one token, and the wave moves the convolution's state on itself.
 // ---------------------------------------------------------------------------------------------
-constexpr int kRopeHeads = 16;
 
 template <typename T>
 __global__ void __launch_bounds__(256)
@@ -453,7 +452,7 @@ conv_rope_norm_store_kernel(const T* __restrict__ rows, int row_stride, const fl
                             const float* __restrict__ qw, const float* __restrict__ kw, int norm, float eps, T* __restrict__ q_out,
                             T* __restrict__ kcache, T* __restrict__ vcache, const int* __restrict__ slots, int nh, int nkvh, int dk,
                             int dv, int page_size, float* __restrict__ state, long long state_stride, const int* __restrict__ token_req,
-                            const int* __restrict__ req_start, const int* __restrict__ state_slots, int single) {
+                            const int* __restrict__ req_start, const int* __restrict__ state_slots, int single, int heads_a_block) {
     __shared__ float cs_s[256], sn_s[256];
     const int t = blockIdx.x, lane = threadIdx.x & 63, half = rot_dims / 2;
     const int C = (nh + nkvh) * dk + nkvh * dv;
@@ -471,8 +470,8 @@ conv_rope_norm_store_kernel(const T* __restrict__ rows, int row_stride, const fl
     float* st = taps > 1 ? state + (long long)state_slots[r] * state_stride : nullptr;
     const int slot = slots ? slots[t] : -1;
     const int pg = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot - pg * page_size : 0;
-    const int last = min(nh + 2 * nkvh, (int)(blockIdx.y + 1) * kRopeHeads);
-    for (int head = blockIdx.y * kRopeHeads + (threadIdx.x >> 6); head < last; head += 4) {
+    const int last = min(nh + 2 * nkvh, (int)(blockIdx.y + 1) * heads_a_block);
+    for (int head = blockIdx.y * heads_a_block + (threadIdx.x >> 6); head < last; head += 4) {
         const bool qk = head < nh + nkvh;
         const int base = qk ? head * dk : (nh + nkvh) * dk + (head - nh - nkvh) * dv;
         auto in = [&](int e) {
@@ -528,6 +527,101 @@ conv_rope_norm_store_kernel(const T* __restrict__ rows, int row_stride, const fl
     }
 }
 
+// The same for portions: a wave a head and kRopeTile consecutive tokens; every row is read once and waits in registers for the
+// tokens behind it.  A lane holds two entries: the pair (i, i + half), or two neighbours behind rot_dims (of v heads only
+// those): dk and dv even and at most 128.
+constexpr int kRopeTile = 16;
+
+template <typename T, int TMAX>
+__global__ void __launch_bounds__(256)
+conv_rope_norm_tile_kernel(const T* __restrict__ rows, int row_stride, const float* __restrict__ cw, int taps,
+                           const int* __restrict__ positions, const float* __restrict__ freq, int rot_dims,
+                           const float* __restrict__ qw, const float* __restrict__ kw, int norm, float eps, T* __restrict__ q_out,
+                           T* __restrict__ kcache, T* __restrict__ vcache, const int* __restrict__ slots, int nh, int nkvh, int dk,
+                           int dv, int page_size, const float* __restrict__ state, long long state_stride,
+                           const int* __restrict__ token_req, const int* __restrict__ req_start, const int* __restrict__ state_slots,
+                           int n_tokens) {
+    __shared__ float cs_s[kRopeTile][64], sn_s[kRopeTile][64];
+    __shared__ long long row_s[kRopeTile];                           // a token's place in the cache, in rows of a head (-1: none)
+    const int lane = threadIdx.x & 63, half = rot_dims / 2, C = (nh + nkvh) * dk + nkvh * dv;
+    const int t0 = blockIdx.x * kRopeTile, t1 = min(n_tokens, t0 + kRopeTile);
+    if (threadIdx.x < t1 - t0) {
+        const int slot = slots ? slots[t0 + threadIdx.x] : -1, pg = slot >= 0 ? slot / page_size : 0;
+        row_s[threadIdx.x] = slot >= 0 ? (long long)pg * nkvh * page_size + (slot - pg * page_size) : -1;
+    }
+    for (int i = threadIdx.x; i < (t1 - t0) * 64; i += 256) {
+        const int tt = i >> 6, e = i & 63;
+        float cs = 1.f, sn = 0.f;
+        if (e < half) pair_angle((float)positions[t0 + tt], freq[e], freq[half + e], cs, sn);
+        cs_s[tt][e] = cs;
+        sn_s[tt][e] = sn;
+    }
+    __syncthreads();
+    const int head = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    if (head >= nh + 2 * nkvh) return;
+    const bool qk = head < nh + nkvh, is_q = head < nh, turned = qk && lane < half;
+    const int size = qk ? dk : dv, base = qk ? head * dk : (nh + nkvh) * dk + (head - nh - nkvh) * dv;
+    const int e0 = turned ? lane : qk ? rot_dims + 2 * (lane - half) : 2 * lane, e1 = turned ? lane + half : e0 + 1;
+    const bool has = lane < size / 2;
+    const int c0 = base + (has ? e0 : 0), c1 = base + (has ? e1 : 0);
+    ConvWindow<T, TMAX> win0, win1;
+    win0.weights(cw, taps, c0);
+    win1.weights(cw, taps, c1);
+    const float* w = is_q ? qw : kw;
+    const float w0 = qk && has && w ? w[e0] : 1.f, w1 = qk && has && w ? w[e1] : 1.f, inv_dk = 1.0f / (float)dk;
+    T* cache = qk ? kcache : vcache;
+    const int kv_head = qk ? head - nh : head - nh - nkvh;
+    int next = t0;                                                   // the row where the window is filled anew
+    constexpr int AHEAD = 8;
+    for (int ta = t0; ta < t1; ta += AHEAD) {
+        T in0[AHEAD], in1[AHEAD];
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {
+            const T* row = rows + (size_t)min(ta + i, t1 - 1) * row_stride;
+            in0[i] = row[c0];
+            in1[i] = row[c1];
+        }
+#pragma unroll
+        for (int i = 0; i < AHEAD; ++i) {
+            const int t = ta + i;
+            if (t >= t1) break;
+            if (t == next) {
+                const int r = token_req[t], start = req_start[r];
+                next = req_start[r + 1];
+                const float* st = taps > 1 ? state + (long long)state_slots[r] * state_stride : nullptr;
+                win0.restart(rows, row_stride, taps, C, st, t, start, c0);
+                win1.restart(rows, row_stride, taps, C, st, t, start, c1);
+            }
+            float a = win0.next(to_f32(in0[i])), b = win1.next(to_f32(in1[i]));
+            T* dst;
+            if (is_q) dst = q_out + (size_t)t * nh * dk + base;
+            else {
+                const long long row = row_s[t - t0];
+                dst = row >= 0 && cache ? cache + (row + (long long)kv_head * page_size) * size : nullptr;
+            }
+            if (qk) {
+                if (turned) {
+                    const float cs = cs_s[t - t0][lane], sn = sn_s[t - t0][lane], u = a;
+                    a = u * cs - b * sn;
+                    b = b * cs + u * sn;
+                }
+                if (norm) {
+                    const float f = __builtin_amdgcn_rsqf(group_sum<64>(has ? a * a + b * b : 0.f) * inv_dk + eps);
+                    a *= f * w0;
+                    b *= f * w1;
+                } else {
+                    a *= w0;
+                    b *= w1;
+                }
+            }
+            if (dst && has) {
+                dst[e0] = from_f32<T>(a);
+                dst[e1] = from_f32<T>(b);
+            }
+        }
+    }
+}
+
 IC_EXPORT int ic_conv_rope_norm_store(const void* rows, int row_stride, int dtype, const float* cw, int taps, const int* positions,
                                       const float* freq, int rot_dims, const float* qw, const float* kw, int norm, float eps,
                                       void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh, int nkvh, int dk, int dv,
@@ -542,23 +636,35 @@ IC_EXPORT int ic_conv_rope_norm_store(const void* rows, int row_stride, int dtyp
     if (row_stride < n) return IC_ERR_ARG;
     if (dk > 512 || dv > 512) return IC_ERR_TOO_LARGE;
     const int C = (int)n;
-    dim3 grid(T, (nh + 2 * nkvh + kRopeHeads - 1) / kRopeHeads), block(256), sgrid((C + 255) / 256, R);
+    const int heads = nh + 2 * nkvh, heads_a_block = T >= 256 ? 16 : 4;
+    dim3 grid(T, (heads + heads_a_block - 1) / heads_a_block), block(256), sgrid((C + 255) / 256, R);
+    const bool tiles = taps > 0 && !single && T >= 64 && dk % 2 == 0 && dv % 2 == 0 && dk <= 128 && dv <= 128;
+    dim3 tgrid((T + kRopeTile - 1) / kRopeTile, (heads + 3) / 4);
+#define IC_CRT(TT, TM)                                                                                                         \
+    hipLaunchKernelGGL((conv_rope_norm_tile_kernel<TT, TM>), tgrid, block, 0, stream, (const TT*)rows, row_stride, cw, taps, positions, \
+                       freq, rot_dims, qw, kw, norm, eps, (TT*)q_out, (TT*)kcache, (TT*)vcache, slots, nh, nkvh, dk, dv, page_size, \
+                       state, state_stride, token_req, req_start, state_slots, T)
     if (dtype == IC_F32) {
-        hipLaunchKernelGGL(conv_rope_norm_store_kernel<float>, grid, block, 0, stream, (const float*)rows, row_stride, cw, taps, positions,
+        if (tiles) { if (taps <= 4) IC_CRT(float, 4); else IC_CRT(float, 8); }
+        else
+            hipLaunchKernelGGL(conv_rope_norm_store_kernel<float>, grid, block, 0, stream, (const float*)rows, row_stride, cw, taps, positions,
                            freq, rot_dims, qw, kw, norm, eps, (float*)q_out, (float*)kcache, (float*)vcache, slots, nh, nkvh, dk, dv,
-                           page_size, state, state_stride, token_req, req_start, state_slots, single);
+                           page_size, state, state_stride, token_req, req_start, state_slots, single, heads_a_block);
         if (taps > 1 && !single)
             hipLaunchKernelGGL(conv_state_kernel<float>, sgrid, block, 0, stream, (const float*)rows, row_stride, nullptr, taps, C, state,
                                state_stride, req_start, state_slots);
     } else if (dtype == IC_BF16) {
-        hipLaunchKernelGGL(conv_rope_norm_store_kernel<bf16>, grid, block, 0, stream, (const bf16*)rows, row_stride, cw, taps, positions,
+        if (tiles) { if (taps <= 4) IC_CRT(bf16, 4); else IC_CRT(bf16, 8); }
+        else
+            hipLaunchKernelGGL(conv_rope_norm_store_kernel<bf16>, grid, block, 0, stream, (const bf16*)rows, row_stride, cw, taps, positions,
                            freq, rot_dims, qw, kw, norm, eps, (bf16*)q_out, (bf16*)kcache, (bf16*)vcache, slots, nh, nkvh, dk, dv,
-                           page_size, state, state_stride, token_req, req_start, state_slots, single);
+                           page_size, state, state_stride, token_req, req_start, state_slots, single, heads_a_block);
         if (taps > 1 && !single)
             hipLaunchKernelGGL(conv_state_kernel<bf16>, sgrid, block, 0, stream, (const bf16*)rows, row_stride, nullptr, taps, C, state,
                                state_stride, req_start, state_slots);
     } else
         return IC_ERR_UNSUPPORTED;
+#undef IC_CRT
     return ic_launch_status();
 }
 

@@ -127,11 +127,12 @@ _SIGNATURES = {
     "ic_ssm_scan": [_P, _I, _I, _I, _P, _I, _I, _P, _P, _P, _I, _I, _I, _I, _P, _P, _LL, _P, _P, _I, _I, _I, _P, _P, _P],
     "ic_gated_group_norm": [_P, _P, _I, _I, _P, _I, _I, _F, _P, _I, _I, _P],
     "ic_blocked_product": [_P, _I, _I, _P, _I, _P, _I, _I, _I, _P, _I, _I, _I, _I, _I, _P],
+    "ic_decay_rows": [_P, _I, _P, _P, _I, _F, _I, _I, _P],
     "ic_decay_product": [_P, _I, _P, _I, _P, _I, _P, _P, _I, _F, _I, _I, _I, _P],
     "ic_conv_rope_norm_store": [_P, _I, _I, _P, _I, _P, _P, _I, _P, _P, _I, _F, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _LL, _P, _P, _P, _I, _I, _P],
     "ic_sum_norm": [_P, _F, _P, _F, _I, _F, _P, _P, _P, _I, _I, _F, _P],
     "ic_delta_prep": [_P, _I, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _F, _P, _LL, _P, _P, _P, _I, _I, _I, _P],
-    "ic_memory_gates": [_P, _I, _P, _P, _F, _I, _P, _P, _P, _P, _LL, _P, _P, _I, _P],
+    "ic_memory_gates": [_P, _I, _P, _P, _F, _I, _P, _P, _P, _P, _LL, _P, _P, _I, _I, _P],
     "ic_matrix_memory": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _P, _I, _I, _I, _I, _I, _F, _P, _P, _P, _LL, _P, _P, _I, _I, _I, _P],
     "ic_gated_head_norm": [_P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _I, _P],
     "ic_latent_prep": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _P, _P, _P, _P, _I, _P],

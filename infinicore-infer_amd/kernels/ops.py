@@ -1133,6 +1133,25 @@ def blocked_product(a, w, out, gate=None):
     return out
 
 
+def _decay_args(N: int, bias, rate, log_scale, what: str):
+    _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == N, what + ": bias")
+    _need((rate is None) != (log_scale is None), what + ": a rate or a scale of the logarithm")
+    if rate is None:
+        return 3, 1, float(log_scale)
+    _need(rate.dtype == torch.float32 and rate.is_contiguous() and rate.numel() > 0 and N % rate.numel() == 0, what + ": rate")
+    return 2, N // rate.numel(), 0.0
+
+
+def decay_rows(z, bias, rate=None, log_scale=None):
+    """The decay factors of ``decay_product`` from a product that is there already: z [M, N] float32, in place."""
+    _dev(z, bias, rate)
+    M, N = z.shape
+    _need(z.dtype == torch.float32 and z.is_contiguous(), "decay_rows: z is float32 [M, N]")
+    kind, per, c = _decay_args(N, bias, rate, log_scale, "decay_rows")
+    check(get_lib().ic_decay_rows(z.data_ptr(), kind, bias.data_ptr(), _ptr(rate), per, c, M, N, _stream()), "decay_rows")
+    return z
+
+
 def decay_product(a, w, out, bias, rate=None, log_scale=None):
     """Decay factors of a recurrence from a low-rank product: out[m, n] (float32) = exp(-rate[n // per] softplus(a[m] . w[n] +
     bias[n])) with ``rate`` [N / per], or exp(log_scale * logsigmoid(a[m] . w[n] + bias[n])).  ``a``'s rows may be strided."""
@@ -1141,13 +1160,9 @@ def decay_product(a, w, out, bias, rate=None, log_scale=None):
     N = w.shape[0]
     _need(tuple(w.shape) == (N, K) and w.is_contiguous() and w.dtype == a.dtype and a.stride(1) == 1, "decay_product: operands")
     _need(tuple(out.shape) == (M, N) and out.is_contiguous() and out.dtype == torch.float32, "decay_product: out is float32 [M, N]")
-    _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == N, "decay_product: bias")
-    _need((rate is None) != (log_scale is None), "decay_product: a rate or a scale of the logarithm")
-    if rate is not None:
-        _need(rate.dtype == torch.float32 and rate.is_contiguous() and rate.numel() > 0 and N % rate.numel() == 0, "decay_product: rate")
-    check(get_lib().ic_decay_product(a.data_ptr(), a.stride(0), w.data_ptr(), dtype_code(a.dtype), out.data_ptr(), 2 if rate is not None else 3,
-                                     bias.data_ptr(), _ptr(rate), N // rate.numel() if rate is not None else 1,
-                                     float(log_scale) if log_scale is not None else 0.0, M, N, K, _stream()), "decay_product")
+    kind, per, c = _decay_args(N, bias, rate, log_scale, "decay_product")
+    check(get_lib().ic_decay_product(a.data_ptr(), a.stride(0), w.data_ptr(), dtype_code(a.dtype), out.data_ptr(), kind, bias.data_ptr(),
+                                     _ptr(rate), per, c, M, N, K, _stream()), "decay_product")
     return out
 
 
@@ -1192,7 +1207,7 @@ def memory_gates(z, bias_i, bias_f, cap: float, keep, add, floor, state, state_o
     sp, stride = _state_part(state, state_offset)
     _need(state_offset + H <= stride, "memory_gates: state too small")
     check(get_lib().ic_memory_gates(z.data_ptr(), z.stride(0), bias_i.data_ptr(), bias_f.data_ptr(), float(cap), H, keep.data_ptr(),
-                                    add.data_ptr(), floor.data_ptr(), sp, stride, req_start.data_ptr(), state_slots.data_ptr(), n_requests,
+                                    add.data_ptr(), floor.data_ptr(), sp, stride, req_start.data_ptr(), state_slots.data_ptr(), T, n_requests,
                                     _stream()), "memory_gates")
 
 

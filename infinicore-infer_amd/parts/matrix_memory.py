@@ -14,7 +14,8 @@ The norms over a head's o come before the weight: one of the head's size shared 
 of all heads' size.  S, n, m and the convolution's inputs start at zero and live in one float32 row per request.
 
 The projections that read h are rows of ONE product (the exponential gates have one of their own with a float32 result); the
-second half of a low-rank decay is a product whose epilogue forms the factors (``ops.decay_product``); the recurrences
+second half of a low-rank decay is a product whose epilogue forms the factors (``ops.decay_product``; for many rows the
+library's product with ``ops.decay_rows`` behind it); the recurrences
 run in one kernel (``ops.matrix_memory``), the last step is ``ops.gated_head_norm``.
 """
 import torch
@@ -35,6 +36,9 @@ def _check_sizes(what, heads, kv_heads, key_dim, value_dim):
         raise ValueError("%s: key and value sizes must lie in 1..1024 (got %d, %d)" % (what, key_dim, value_dim))
 
 
+LIBRARY_ROWS = 256         # from so many tokens on the thin products (K an inner size) are the library's
+
+
 class _MatrixMemory(Mixer):
     graph_safe = True
     relocatable = True
@@ -46,6 +50,19 @@ class _MatrixMemory(Mixer):
         y = ctx.ws.buffer(self.out_buffer, (rows.shape[0], self.hidden_size), self.runtime.dtype)
         linear(rows, self.w_o, y, self.runtime.gemm_impl, ws=ctx.ws)
         return y
+
+    def _by_library(self, x):
+        """Whether a thin product over the strided rows ``x`` goes to the library: many rows, whole 16-byte pieces."""
+        piece = 16 // x.element_size()
+        return x.shape[0] >= LIBRARY_ROWS and x.shape[1] % piece == 0 and x.stride(0) % piece == 0 and x.data_ptr() % 16 == 0
+
+    def _decay(self, x, w, bias, ctx, **kind):
+        """The decay factors, float32 [T, heads * key_dim], from the low-rank rows ``x``."""
+        decay = ctx.ws.buffer("memory_decay", (x.shape[0], w.shape[0]), torch.float32)
+        if not self._by_library(x):
+            return ops.decay_product(x, w, decay, bias, **kind)
+        linear(x, w, decay, self.runtime.gemm_impl, ws=ctx.ws)
+        return ops.decay_rows(decay, bias, **kind)
 
     def _project(self, h, ctx):
         rows = ctx.ws.buffer("memory_rows", (h.shape[0], self.w_rows.shape[0]), self.runtime.dtype)
@@ -99,9 +116,12 @@ class GatedDeltaRule(_MatrixMemory):
         rows = self._project(h, ctx)
         a1, g1 = rows[:, c:c + self.ra], rows[:, c + self.ra:c + self.ra + self.rg]
         b = rows[:, c + self.ra + self.rg:]
-        decay = ops.decay_product(a1, self.w_a2, buf("memory_decay", (T, self.heads * self.dk), torch.float32), self.dt_bias, rate=self.rate)
+        decay = self._decay(a1, self.w_a2, self.dt_bias, ctx, rate=self.rate)
         gate = buf("memory_gate", (T, self.nv), rt.dtype)
-        ops.blocked_product(g1.unsqueeze(1), self.w_g2.unsqueeze(0), gate.unsqueeze(1))
+        if self._by_library(g1):
+            linear(g1, self.w_g2, gate, rt.gemm_impl, ws=ctx.ws)
+        else:
+            ops.blocked_product(g1.unsqueeze(1), self.w_g2.unsqueeze(0), gate.unsqueeze(1))
         qkv, beta = buf("memory_qkv", (T, c), torch.float32), buf("memory_beta", (T, self.heads), torch.float32)
         single = ctx.T == ctx.R
         lists = (ctx.req_rows, ctx.state_slots, ctx.R)
@@ -150,8 +170,7 @@ class GatedLinearAttention(_MatrixMemory):
         rt, T, nq, nv = self.runtime, h.shape[0], self.nq, self.nv
         buf = ctx.ws.buffer
         rows = self._project(h, ctx)
-        decay = ops.decay_product(rows[:, 2 * nq + 2 * nv:], self.w_a2, buf("memory_decay", (T, nq), torch.float32), self.b_a2,
-                                  log_scale=1.0 / self.tau)
+        decay = self._decay(rows[:, 2 * nq + 2 * nv:], self.w_a2, self.b_a2, ctx, log_scale=1.0 / self.tau)
         o = buf("memory_o", (T, nv), torch.float32)
         ops.matrix_memory(rows[:, :nq], rows[:, nq:2 * nq], rows[:, 2 * nq:2 * nq + nv], decay, self.heads, self.heads, self.dk, self.dv, o,
                           cache.state, self.state_base, ctx.req_rows, ctx.state_slots, ctx.R, single=ctx.T == ctx.R,

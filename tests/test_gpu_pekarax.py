@@ -26,7 +26,8 @@ def _compare(got, ref, dtype, tol, what, steps=None, rounded=None):
     experts' scores lie closer than 16-bit rounding the choice may fall the other way and move that token's row and, through
     a recurrent state, those behind it (every position is held to the float32 tolerance in the float32 mode, which runs the
     same steps, and the 16-bit kernels are held to theirs one by one).  ``rounded``: the plain implementation's logits with the
-    sublayers' inputs and results rounded to 16 bits; median and mean must then stay within three times what that moves."""
+    sublayers' inputs and results rounded to 16 bits; the median must then stay within three
+    times what that moves (the mean, which a single flipped choice can carry, too if that is more than its own bound)."""
     if dtype == torch.float32 and rounded is None:
         return H.compare(got, ref, tol, what, steps)
     H.compare(got, ref, 5 * tol if dtype == torch.float32 else 1e9, what, steps)        # every wanted place is there and finite
@@ -40,7 +41,8 @@ def _compare(got, ref, dtype, tol, what, steps=None, rounded=None):
     median_most, mean_most, over_most = BF16_MEDIAN, BF16_MEAN, max(1, 0.15 * n)
     if rounded is not None:
         alone = sorted(error(rid, pos, rounded[rid][pos]) for rid, pos in got)
-        median_most, mean_most, over_most = 3 * alone[n // 2], 3 * sum(alone) / n, max(1, 0.02 * n + 3 * sum(e > tol for e in alone))
+        median_most, mean_most = 3 * alone[n // 2], max(mean_most, 3 * sum(alone) / n)
+        over_most = max(1, 0.02 * n + 3 * sum(e > tol for e in alone))
     print("%s: median %.3g (most %.3g) mean %.3g (most %.3g), %d of %d beyond %.3g" % (what, middle, median_most, sum(errs) / n, mean_most, over, n, tol))
     assert over <= over_most, "%s: %d of %d positions beyond %.3g" % (what, over, n, tol)
     assert middle <= median_most, "%s: median error %.3g (allowed %.3g)" % (what, middle, median_most)
@@ -517,11 +519,11 @@ def test_a_forked_request_goes_on_apart(tmp_path_factory):
 
 
 # ---- each mechanism's kernel alone ----------------------------------------------------------------------------------------
-LENS = [83, 40, 9]
+LENS = [203, 40, 9]
 # the requests' tokens cut into steps: whole portions, portions of two, single tokens beside portions, single tokens alone, a
 # request left out of a step
 STEPS = [[(0, 33), (1, 2), (2, 1)], [(1, 16), (0, 1)], [(2, 1), (0, 2), (1, 1)], [(0, 1), (1, 1), (2, 1)], [(1, 18)], [(2, 4), (0, 17)],
-         [(0, 1), (2, 1)], [(0, 26), (1, 1)], [(1, 1), (0, 2), (2, 1)]]
+         [(0, 1), (2, 1)], [(0, 146), (1, 1)], [(1, 1), (0, 2), (2, 1)]]
 SLOTS = [4, 1, 2]                                                  # of five; the others hold NaN
 
 
@@ -771,6 +773,14 @@ def test_decay_factors_from_a_low_rank_product(dtype, M, N, K, heads):
     assert torch.allclose(out.cpu().double(), want, atol=3e-6)
     ops.decay_product(wide.cuda()[:, 3:3 + K], w.cuda(), out, bias.cuda(), log_scale=1 / 16.0)
     assert torch.allclose(out.cpu().double(), torch.sigmoid(z).pow(1 / 16.0), atol=3e-6)
+    # the factors alone, from products that are there already, with arguments far out on both sides
+    zf = (z * 12).float()
+    z2 = zf.clone().cuda()
+    ops.decay_rows(z2, bias.cuda(), rate=rate.cuda())
+    assert torch.allclose(z2.cpu().double(), torch.exp(-rate.double().repeat_interleave(N // heads) * P.softplus(zf.double() + bias)), atol=3e-6)
+    z2 = zf.clone().cuda()
+    ops.decay_rows(z2, bias.cuda(), log_scale=0.25)
+    assert torch.allclose(z2.cpu().double(), torch.sigmoid(zf.double() + bias).pow(0.25), atol=3e-6, rtol=1e-5)
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])

@@ -82,9 +82,15 @@ __device__ __forceinline__ float dpp_add(float v, int) = delete;
 template <int CTRL> __device__ __forceinline__ float dpp_add(float v) {
     return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, true));
 }
+// Lane i gets v[i] + v[i ^ D], D 16 or 32: the two copies of v trade every other run of D lanes.
+template <int D> __device__ __forceinline__ float swap_add(float v) {
+    const unsigned b = (unsigned)__float_as_int(v);
+    const auto r = D == 32 ? __builtin_amdgcn_permlane32_swap(b, b, false, false) : __builtin_amdgcn_permlane16_swap(b, b, false, false);
+    return __int_as_float((int)r[0]) + __int_as_float((int)r[1]);
+}
 template <int LPK> __device__ __forceinline__ float group_sum(float d) {
-    if (LPK >= 64) d += __shfl_xor(d, 32, kWave);
-    if (LPK >= 32) d += __shfl_xor(d, 16, kWave);
+    if (LPK >= 64) d = swap_add<32>(d);
+    if (LPK >= 32) d = swap_add<16>(d);
     if (LPK >= 16) d = dpp_add<0x128>(d);        // row_ror:8      lane i <- lane i ^ 8
     if (LPK >= 8) d = dpp_add<0x141>(d);         // row_half_mirror lane i <- lane 7 - i (of 8)
     if (LPK >= 4) d = dpp_add<0x4E>(d);          // quad_perm [2,3,0,1]

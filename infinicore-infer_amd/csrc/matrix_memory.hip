@@ -536,23 +536,43 @@ __global__ void __launch_bounds__(256) matrix_scan_kernel(MatrixMemoryArgs a) {
         float keep[NC];
 #pragma unroll
         for (int j = 0; j < NC; ++j) keep[j] = 0.f;
-        auto token = [&](int tt) {
-            float k[NI], q[NI], g[NI];
-            rows4(ks[b][tt], k);
-            rows4(qs[b][tt], q);
-            if (CHANNEL) rows4(gs[CHANNEL ? b : 0][CHANNEL ? tt : 0], g);
-            const float4 c = sc[b][tt];
+        // Where the registers suffice a token's vectors are read one token ahead: nothing else hides the way out of LDS from a
+        // wave that is alone on its unit.
+        constexpr bool AHEAD = NI <= 8;
+        float k[2][NI], q[2][NI], g[2][CHANNEL ? NI : 1], v[2][NC];
+        float4 c[2];
+        auto ahead = [&](int tt, int x) {
+            rows4(ks[b][tt], k[x]);
+            if (CHANNEL) rows4(gs[CHANNEL ? b : 0][CHANNEL ? tt : 0], g[x]);
+            rows4(qs[b][tt], q[x]);
+            c[x] = sc[b][tt];
+#pragma unroll
+            for (int j = 0; j < NC; ++j) v[x][j] = vs[b][tt][cg + CG * j];
+            if (AHEAD) __builtin_amdgcn_sched_barrier(0);
+        };
+        auto token = [&](int tt, int x) {
+            if (!AHEAD) ahead(tt, x);
 #pragma unroll
             for (int j = 0; j < NC; ++j) {
-                const float o = mm_token<L, NI, DELTA, CHANNEL>(s[j], k, q, g, c.x, c.y, c.z, vs[b][tt][cg + CG * j]);
+                const float o = mm_token<L, NI, DELTA, CHANNEL>(s[j], k[x], q[x], g[x], c[x].x, c[x].y, c[x].z, v[x][j]);
                 keep[j] = p == tt ? o : keep[j];
             }
         };
+        if (AHEAD) ahead(0, 0);
         if (n == TT) {
 #pragma unroll
-            for (int tt = 0; tt < TT; ++tt) token(tt);
+            for (int tt = 0; tt < TT; ++tt) {
+                if (AHEAD && tt + 1 < TT) ahead(tt + 1, (tt + 1) & 1);
+                token(tt, tt & 1);
+            }
         } else
-            for (int tt = 0; tt < n; ++tt) token(tt);
+            for (int tt = 0; tt < n; tt += 2) {
+                if (AHEAD && tt + 1 < n) ahead(tt + 1, 1);
+                token(tt, 0);
+                if (tt + 1 >= n) break;
+                if (AHEAD && tt + 2 < n) ahead(tt + 2, 0);
+                token(tt + 1, 1);
+            }
         if (p < n) {
 #pragma unroll
             for (int j = 0; j < NC; ++j) {

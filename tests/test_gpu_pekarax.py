@@ -104,7 +104,7 @@ K3 = {"architecture": "Pekarax", "vocab": 300, "width": 128, "norm": {"eps": 1e-
       "layers": [_delta(2, 1, 128, 64, 5, _moe(16, 4, 32, 2.0, (8, 2))),
                  _gla(2, 136, 72, 16.0, _moe(7, 2, 64, 1.2, (2, 1), 1, 2.0)),
                  _parallel((6, 2, 128, 64, 4, 0.25, 64, 300000.0), (2, 160, 96, 8.0), (1.1, 0.9), None),
-                 _parallel((4, 4, 64, 64, 2, 0.125, 64, 1000.0), (4, 32, 16, 15.0), (0.5, 1.5), _moe(4, 4, 24, 1.5)),
+                 _parallel((5, 5, 64, 64, 2, 0.125, 64, 1000.0), (4, 32, 16, 15.0), (0.5, 1.5), _moe(4, 4, 24, 1.5)),
                  _delta(6, 2, 32, 32, 2, None)]}
 SHARP = dict(K1, norm={"eps": 1e-2})
 CONFIGS = {"K1": K1, "K2": K2, "K3": K3}
@@ -559,7 +559,7 @@ def _close(got, want, tol, what):
 
 
 MEMORY_SIZES = [  # heads, query/key heads, key size, value size
-    (4, 2, 24, 40), (3, 3, 6, 9), (2, 1, 128, 64), (1, 1, 200, 33), (2, 1, 300, 24), (1, 1, 600, 20), (6, 6, 32, 32), (8, 4, 64, 128)]
+    (4, 2, 24, 40), (3, 3, 6, 9), (2, 1, 128, 64), (1, 1, 200, 33), (2, 1, 300, 24), (1, 1, 600, 20), (5, 5, 32, 32), (8, 4, 64, 128)]
 
 
 @pytest.mark.parametrize("columns", [1, 2])
@@ -653,13 +653,13 @@ def test_matrix_memory_with_exponential_gates(H_, G, dk, dv, dtype):
 
 @pytest.mark.parametrize("H_", [1, 3, 70])
 def test_exponential_gates_over_long_portions(H_):
-    """More tokens than a wave takes at a time, cut at places inside and at the borders of its runs; the running maximum
+    """More tokens than a wave and than a block takes at a time, cut at places inside and at the borders of its runs; the running maximum
     starts at zero, falls slowly and is overtaken by single strong input gates."""
     from infinicore_infer_amd.kernels import ops
-    T, cap = 700, 9.0
+    T, cap = 2600, 9.0
     g = torch.Generator().manual_seed(H_)
     z = torch.cat([torch.randn(T, H_, generator=g) * 2 - 4, torch.randn(T, H_, generator=g) * 2 + 3], 1)
-    z[300, :H_] = 12.0
+    z[300, :H_] = z[1800, :H_] = 12.0
     bi, bf = torch.randn(H_, generator=g), torch.randn(H_, generator=g)
     li = cap * torch.tanh((z[:, :H_].double() + bi) / cap)
     lf = -P.softplus(-cap * torch.tanh((z[:, H_:].double() + bf) / cap))
@@ -670,7 +670,7 @@ def test_exponential_gates_over_long_portions(H_):
         add.append(torch.exp(li[t] - new))
         floor.append(torch.exp(-new))
         m = new
-    for cuts in ([0, 700], [0, 64, 128, 129, 131, 200, 511, 700], [0, 1, 2, 65, 700]):
+    for cuts in ([0, 2600], [0, 64, 128, 129, 131, 200, 511, 1535, 2600], [0, 1, 2, 65, 2113, 2600]):
         st = torch.zeros(1, H_ + 3, device="cuda")
         outs = [torch.empty(T, H_, device="cuda") for _ in range(3)]
         for a, b in zip(cuts, cuts[1:]):

@@ -8,10 +8,11 @@ from .mezinex import MezinexConfig
 from .daborax import DaboraxConfig
 from .fizelix import FizelixConfig
 from .pekarax import PekaraxConfig
+from .fokinex import FokinexConfig
 
 __all__ = [
     "ConfigError", "config_from_dict", "config_from_dir", "read_config_json",
     "register_architecture", "registered_architectures", "resolve_architecture",
     "ExecEntry", "LayerSpec", "ModelSpec", "PartSpec", "default_schedule",
-    "MiniCPMConfig", "RopeScaling", "FopezenConfig", "MezinexConfig", "DaboraxConfig", "FizelixConfig", "PekaraxConfig",
+    "MiniCPMConfig", "RopeScaling", "FopezenConfig", "MezinexConfig", "DaboraxConfig", "FizelixConfig", "PekaraxConfig", "FokinexConfig",
 ]

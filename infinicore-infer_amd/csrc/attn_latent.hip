@@ -6,9 +6,16 @@
 // the same rows, and leave the two small products per head to the caller.
 //
 // Cache plane: [pages, 1, page_size, R + E].  Rotation: entries (2i, 2i+1) of the first `rot_dims` entries of a
-// rotated part turn by the angle position * freq[i]; the rest pass unchanged.  Angles, scores and the running
-// softmax are float32.
-#include "common.h"
+// rotated part turn by the angle position * freq[i] (freq: float32 [2, rot_dims / 2], the frequency and what its rounding
+// left) and are multiplied by rot_mult; the rest pass unchanged.  Angles, scores and the running softmax are float32.
+// A query at position i sees key j when 0 <= i - j < window (window 0: every j <= i).  `sinks` (nullable, one float32 per
+// head): exp(sinks[h]) joins the softmax's denominator, with no key and no value, not scaled.
+//
+// Prompt portions have two more ways: keys and values of every head made from the request's latent rows and walked by the
+// matrix-core kernel of attn_span_prefill.h (ic_attn_latent_prefill), and two matrix products over the latent rows themselves
+// with a masked softmax between them (ic_latent_gather, ic_latent_softmax).
+#include "attn_span_prefill.h"
+#include "rotation.h"
 
 constexpr int kLatentMaxRank = 512;    // R: a lane holds R / 64 sums per head
 constexpr int kLatentHeads = 4;        // heads that share one walk over the rows
@@ -18,7 +25,7 @@ constexpr int kLatentHeads = 4;        // heads that share one walk over the row
 template <typename T>
 __global__ void __launch_bounds__(256)
 latent_prep_kernel(const T* __restrict__ rows, int ld, int Rq, int R, int E, const float* __restrict__ qn_w,
-                   const float* __restrict__ kvn_w, float eps, const float* __restrict__ freq, int rot_dims,
+                   const float* __restrict__ kvn_w, float eps, const float* __restrict__ freq, int rot_dims, float rot_mult,
                    const int* __restrict__ positions, T* __restrict__ cq, T* __restrict__ cache,
                    const int* __restrict__ slots) {
     __shared__ float red[8];
@@ -43,8 +50,9 @@ latent_prep_kernel(const T* __restrict__ rows, int ld, int Rq, int R, int E, con
     for (int j = threadIdx.x; j < R; j += blockDim.x) dst[j] = from_f32<T>(to_f32(kv[j]) * r * kvn_w[j]);
     const float pos = (float)positions[t];
     for (int i = threadIdx.x; i < rot_dims / 2; i += blockDim.x) {
-        const float a = pos * freq[i];
-        const float c = cosf(a), s = sinf(a);
+        float c, s;
+        pair_angle(pos, freq[i], freq[rot_dims / 2 + i], c, s);
+        c *= rot_mult; s *= rot_mult;
         const float u = to_f32(kv[R + 2 * i]), v = to_f32(kv[R + 2 * i + 1]);
         dst[R + 2 * i] = from_f32<T>(u * c - v * s);
         dst[R + 2 * i + 1] = from_f32<T>(v * c + u * s);
@@ -53,26 +61,27 @@ latent_prep_kernel(const T* __restrict__ rows, int ld, int Rq, int R, int E, con
 }
 
 IC_EXPORT int ic_latent_prep(const void* rows, int ld, int dtype, int Rq, int R, int E, const float* qn_w,
-                             const float* kvn_w, float eps, const float* freq, int rot_dims, const int* positions,
+                             const float* kvn_w, float eps, const float* freq, int rot_dims, float rot_mult, const int* positions,
                              void* cq, void* cache, const int* slots, int T, hipStream_t stream) {
     if (T <= 0) return IC_OK;
-    if (Rq <= 0 || R <= 0 || E < 0 || rot_dims < 0 || rot_dims > E || rot_dims % 2) return IC_ERR_ARG;
+    if (Rq <= 0 || R <= 0 || E < 0 || (slots && (!kvn_w || !cache)) || rot_dims < 0 || rot_dims > E || rot_dims % 2) return IC_ERR_ARG;
     if (dtype == IC_F32)
         hipLaunchKernelGGL(latent_prep_kernel<float>, dim3(T), dim3(256), 0, stream, (const float*)rows, ld, Rq, R, E, qn_w,
-                           kvn_w, eps, freq, rot_dims, positions, (float*)cq, (float*)cache, slots);
+                           kvn_w, eps, freq, rot_dims, rot_mult, positions, (float*)cq, (float*)cache, slots);
     else if (dtype == IC_BF16)
         hipLaunchKernelGGL(latent_prep_kernel<bf16>, dim3(T), dim3(256), 0, stream, (const bf16*)rows, ld, Rq, R, E, qn_w,
-                           kvn_w, eps, freq, rot_dims, positions, (bf16*)cq, (bf16*)cache, slots);
+                           kvn_w, eps, freq, rot_dims, rot_mult, positions, (bf16*)cq, (bf16*)cache, slots);
     else
         return IC_ERR_UNSUPPORTED;
     return ic_launch_status();
 }
 
-// ---- the queries' rotated parts: q[t, h, dim:dim+E] rotated into qa[t, h, R:R+E] -----------------------------------
+// ---- the queries' rotated parts: q[t, h, dim:dim+E] rotated into qa[t, h, R:R+E] (q itself with R = dim: a thread reads its
+// entries before it writes them, and no two threads share one) ---------------------------------------------------------
 template <typename T>
 __global__ void __launch_bounds__(256)
-latent_q_rotate_kernel(const T* __restrict__ q, int q_stride, int dim, int E, int R, int H, const float* __restrict__ freq,
-                       int rot_dims, const int* __restrict__ positions, T* __restrict__ qa, int qa_stride) {
+latent_q_rotate_kernel(const T* q, int q_stride, int dim, int E, int R, int H, const float* __restrict__ freq,
+                       int rot_dims, float rot_mult, const int* __restrict__ positions, T* qa, int qa_stride) {
     const int t = blockIdx.x;
     const float pos = (float)positions[t];
     const int half = rot_dims / 2, rest = E - rot_dims, per = half + rest;
@@ -81,8 +90,9 @@ latent_q_rotate_kernel(const T* __restrict__ q, int q_stride, int dim, int E, in
         const T* src = q + (size_t)t * q_stride + (size_t)h * (dim + E) + dim;
         T* dst = qa + (size_t)t * qa_stride + (size_t)h * (R + E) + R;
         if (i < half) {
-            const float a = pos * freq[i];
-            const float c = cosf(a), s = sinf(a);
+            float c, s;
+            pair_angle(pos, freq[i], freq[half + i], c, s);
+            c *= rot_mult; s *= rot_mult;
             const float u = to_f32(src[2 * i]), v = to_f32(src[2 * i + 1]);
             dst[2 * i] = from_f32<T>(u * c - v * s);
             dst[2 * i + 1] = from_f32<T>(v * c + u * s);
@@ -93,15 +103,15 @@ latent_q_rotate_kernel(const T* __restrict__ q, int q_stride, int dim, int E, in
 }
 
 IC_EXPORT int ic_latent_q_rotate(const void* q, int q_stride, int dtype, int dim, int E, int R, int H, const float* freq,
-                                 int rot_dims, const int* positions, void* qa, int qa_stride, int T, hipStream_t stream) {
+                                 int rot_dims, float rot_mult, const int* positions, void* qa, int qa_stride, int T, hipStream_t stream) {
     if (T <= 0 || E == 0) return IC_OK;
     if (dim < 0 || E < 0 || R <= 0 || H <= 0 || rot_dims < 0 || rot_dims > E || rot_dims % 2) return IC_ERR_ARG;
     if (dtype == IC_F32)
         hipLaunchKernelGGL(latent_q_rotate_kernel<float>, dim3(T), dim3(256), 0, stream, (const float*)q, q_stride, dim, E,
-                           R, H, freq, rot_dims, positions, (float*)qa, qa_stride);
+                           R, H, freq, rot_dims, rot_mult, positions, (float*)qa, qa_stride);
     else if (dtype == IC_BF16)
         hipLaunchKernelGGL(latent_q_rotate_kernel<bf16>, dim3(T), dim3(256), 0, stream, (const bf16*)q, q_stride, dim, E, R,
-                           H, freq, rot_dims, positions, (bf16*)qa, qa_stride);
+                           H, freq, rot_dims, rot_mult, positions, (bf16*)qa, qa_stride);
     else
         return IC_ERR_UNSUPPORTED;
     return ic_launch_status();
@@ -118,7 +128,8 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
                    const T* __restrict__ cache, const int* __restrict__ block_tables, int bt_stride,
                    const int* __restrict__ token_req, const int* __restrict__ positions,
                    const int* __restrict__ row_list, int H, int R, int E,
-                   int page_size, float scale, int n_split, float* __restrict__ part_acc, float* __restrict__ part_ml) {
+                   int page_size, float scale, int window, const float* __restrict__ sinks, int n_split,
+                   float* __restrict__ part_acc, float* __restrict__ part_ml) {
     constexpr int HG = kLatentHeads, NP = kLatentMaxRank / 64 / VEC;   // pieces of VEC columns a lane owns
     extern __shared__ float qs[];                 // HG * (R + E) floats
     __shared__ float ps[HG][64];
@@ -135,10 +146,11 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
         qs[e] = g < nh ? to_f32(qa[(size_t)t * qa_stride + (size_t)(h0 + g) * D + d]) : 0.f;
     }
     __syncthreads();
-    // this split's share of the keys 0..pos, in whole chunks of 64
-    const int n_chunks = (pos + 64) / 64;
+    // this split's share of the keys lo..pos, in whole chunks of 64
+    const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    const int first_chunk = lo / 64, n_chunks = pos / 64 + 1 - first_chunk;
     const int per = (n_chunks + n_split - 1) / n_split;
-    const int c_lo = split * per, c_hi = (c_lo + per < n_chunks) ? c_lo + per : n_chunks;
+    const int c_lo = first_chunk + split * per, c_hi = (split * per + per < n_chunks) ? c_lo + per : first_chunk + n_chunks;
 
     float acc[HG][NP][VEC];
 #pragma unroll
@@ -153,7 +165,7 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
 
     for (int ch = c_lo; ch < c_hi; ++ch) {
         const int key = ch * 64 + lane;
-        const bool valid = key <= pos;
+        const bool valid = key >= lo && key <= pos;
         float s[HG];
 #pragma unroll
         for (int g = 0; g < HG; ++g) s[g] = 0.f;
@@ -177,7 +189,7 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
 #pragma unroll
         for (int g = 0; g < HG; ++g) {
             const float sv = valid ? s[g] * scale : -INFINITY;
-            const float m_new = fmaxf(m[g], wave_max(sv));      // the chunk's first key is always visible
+            const float m_new = fmaxf(m[g], wave_max(sv));      // finite: some key of every chunk is visible
             const float p = valid ? expf(sv - m_new) : 0.f;
             corr[g] = expf(m[g] - m_new);
             l[g] = l[g] * corr[g] + wave_sum(p);
@@ -186,14 +198,14 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
         }
         krow[lane] = base;
         __syncthreads();
-        const int nk = (pos - ch * 64 + 1 < 64) ? pos - ch * 64 + 1 : 64;
+        const int k0 = (lo > ch * 64) ? lo - ch * 64 : 0, nk = (pos - ch * 64 + 1 < 64) ? pos - ch * 64 + 1 : 64;
 #pragma unroll
         for (int g = 0; g < HG; ++g)
 #pragma unroll
             for (int i = 0; i < NP; ++i)
 #pragma unroll
                 for (int v = 0; v < VEC; ++v) acc[g][i][v] *= corr[g];
-        for (int kk = 0; kk < nk; ++kk) {
+        for (int kk = k0; kk < nk; ++kk) {
             const T* cp = cache + krow[kk];
             float pk[HG];
 #pragma unroll
@@ -221,7 +233,11 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
         if (g >= nh) continue;
         const int h = h0 + g;
         if (n_split == 1) {
-            const float inv = 1.0f / l[g];
+            float inv = 1.0f / l[g];
+            if (sinks) {
+                const float mf = fmaxf(m[g], sinks[h]), c = expf(m[g] - mf);
+                inv = c / (l[g] * c + expf(sinks[h] - mf));
+            }
 #pragma unroll
             for (int i = 0; i < NP; ++i) {
                 const int col = (lane + 64 * i) * VEC;
@@ -254,7 +270,7 @@ attn_latent_kernel(const T* __restrict__ qa, int qa_stride, T* __restrict__ out,
 // operand of O^T = V^T P^T, whose A operand (the first R values of the same LDS rows, transposed) comes out of LDS
 // through the transposing read.  Operand layout (lane l, h = l / 32): A[i = l % 32][k = 8h..8h+7],
 // B[k = 8h..8h+7][j = l % 32], D[i = 8(r / 4) + 4h + r % 4][j = l % 32] for the 16 accumulators r.
-// A key beyond the token's position is replaced by the position's own row when loaded, and masked.
+// A key outside the token's window or beyond its position is replaced by the nearest one inside when loaded, and masked.
 typedef __bf16 lat_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float lat_v16f __attribute__((ext_vector_type(16)));
 typedef float lat_v8f __attribute__((ext_vector_type(8)));
@@ -265,8 +281,9 @@ __global__ void __launch_bounds__(64 * (R >= 128 ? 4 : R / 32))
 attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __restrict__ out, int out_stride,
                         const bf16* __restrict__ cache, const int* __restrict__ block_tables, int bt_stride,
                         const int* __restrict__ token_req, const int* __restrict__ positions,
-                        const int* __restrict__ row_list, int H, int page_size, float scale, int n_split,
-                        float* __restrict__ part_acc, float* __restrict__ part_ml) {
+                        const int* __restrict__ row_list, int H, int page_size, float scale, int window,
+                        const float* __restrict__ sinks, int n_split, float* __restrict__ part_acc,
+                        float* __restrict__ part_ml) {
     // The block's waves share a step's rows in LDS; each computes the (same) scores and owns ND / WAVES of the
     // 32-column tiles of the result.
     constexpr int D = R + E, NC = D / 16, ND = R / 32, PK = D + 8, PIECES = D / 8;
@@ -296,9 +313,10 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
             else qf[c] = __builtin_bit_cast(lat_bf16x8, v);
         }
     }
-    const int n_steps = pos / 32 + 1;
+    const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    const int first_step = lo / 32, n_steps = pos / 32 + 1 - first_step;
     const int per = (n_steps + n_split - 1) / n_split;
-    const int s_lo = split * per, s_hi = (s_lo + per < n_steps) ? s_lo + per : n_steps;
+    const int s_lo = first_step + split * per, s_hi = (split * per + per < n_steps) ? s_lo + per : first_step + n_steps;
 
     lat_v16f oacc[NDW];
 #pragma unroll
@@ -319,7 +337,7 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
             const int e = threadIdx.x + THREADS * k;
             if (e < 32 * PIECES) {
                 const int row = e / PIECES, piece = e % PIECES;
-                const int key = (kb + row < pos) ? kb + row : pos;
+                const int key = (kb + row < lo) ? lo : (kb + row < pos) ? kb + row : pos;
                 got[k] = *reinterpret_cast<const uint4*>(cache + ((long long)bt[key / page_size] * page_size + key % page_size) * D + piece * 8);
             }
         }
@@ -346,16 +364,18 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
         }
 #pragma unroll
         for (int r = 0; r < 16; ++r) sacc[r] += sacc2[r];
-        if (kb + 31 > pos) {
+        if (kb + 31 > pos || kb < lo) {
 #pragma unroll
-            for (int r = 0; r < 16; ++r)
-                if (kb + 8 * (r >> 2) + 4 * half + (r & 3) > pos) sacc[r] = -INFINITY;
+            for (int r = 0; r < 16; ++r) {
+                const int key = kb + 8 * (r >> 2) + 4 * half + (r & 3);
+                if (key > pos || key < lo) sacc[r] = -INFINITY;
+            }
         }
         float mloc = sacc[0];
 #pragma unroll
         for (int r = 1; r < 16; ++r) mloc = fmaxf(mloc, sacc[r]);
         mloc = fmaxf(mloc, __shfl_xor(mloc, 32, kWave));
-        const float m_new = fmaxf(m, mloc);                     // finite: the step's first key is visible
+        const float m_new = fmaxf(m, mloc);                     // finite: some key of every step is visible
         const float mc = m_new * scale_log2e;
         const float corr = (m == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(m * scale_log2e - mc);
         float rs = 0.f;
@@ -391,7 +411,11 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
     }
     if (!row_ok) return;
     if (n_split == 1) {
-        const float inv = 1.0f / l;
+        float inv = 1.0f / l;
+        if (sinks) {                              // the term exp(sink) joins the denominator (exponents base 2)
+            const float sv = sinks[head] * kLog2e, ms = m * scale_log2e, mf = fmaxf(ms, sv), c = __builtin_amdgcn_exp2f(ms - mf);
+            inv = c / (l * c + __builtin_amdgcn_exp2f(sv - mf));
+        }
         bf16* op = out + (size_t)t * out_stride + (size_t)head * R + 32 * wave * NDW;
 #pragma unroll
         for (int dt = 0; dt < NDW; ++dt)
@@ -411,11 +435,11 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
 template <int R, int E>
 static void latent_mfma_launch(dim3 grid, hipStream_t stream, const void* qa, int qa_stride, void* out, int out_stride,
                                const void* cache, const int* block_tables, int bt_stride, const int* token_req,
-                               const int* positions, const int* row_list, int H, int page_size, float scale, int n_split,
-                               float* part_acc, float* part_ml) {
+                               const int* positions, const int* row_list, int H, int page_size, float scale, int window,
+                               const float* sinks, int n_split, float* part_acc, float* part_ml) {
     hipLaunchKernelGGL((attn_latent_mfma_kernel<R, E>), grid, dim3(64 * (R >= 128 ? 4 : R / 32)), 0, stream, (const bf16*)qa, qa_stride, (bf16*)out,
                        out_stride, (const bf16*)cache, block_tables, bt_stride, token_req, positions, row_list, H, page_size,
-                       scale, n_split, part_acc, part_ml);
+                       scale, window, sinks, n_split, part_acc, part_ml);
 }
 
 // Sizes the matrix-core walk is built for: the latent 64, 128, 256 or 512 wide, the rotated part 16, 32 or 64.
@@ -427,7 +451,7 @@ IC_EXPORT int ic_attn_latent_on_matrix_cores(int dtype, int R, int E) {
 template <typename T>
 __global__ void __launch_bounds__(256)
 attn_latent_merge_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml, int n_split, int H, int R,
-                         T* __restrict__ out, int out_stride, const int* __restrict__ row_list) {
+                         T* __restrict__ out, int out_stride, const int* __restrict__ row_list, const float* __restrict__ sinks) {
     const int h = blockIdx.x % H, t = row_list ? row_list[blockIdx.x / H] : blockIdx.x / H;
     const size_t p0 = ((size_t)t * H + h) * n_split;
     __shared__ float wgt[64];                 // a split's share of the result: exp(m_s - m) / l
@@ -435,9 +459,10 @@ attn_latent_merge_kernel(const float* __restrict__ part_acc, const float* __rest
         const int sp = threadIdx.x;
         const float ms = sp < n_split ? part_ml[2 * (p0 + sp)] : -INFINITY;
         const float ls = sp < n_split ? part_ml[2 * (p0 + sp) + 1] : 0.f;
-        const float m = wave_max(ms);
+        float m = wave_max(ms);
+        if (sinks) m = fmaxf(m, sinks[h]);
         const float e = ms > -INFINITY ? expf(ms - m) : 0.f;
-        const float l = wave_sum(ls * e);
+        const float l = wave_sum(ls * e) + (sinks ? expf(sinks[h] - m) : 0.f);
         wgt[sp] = e / l;
     }
     __syncthreads();
@@ -451,10 +476,11 @@ attn_latent_merge_kernel(const float* __restrict__ part_acc, const float* __rest
 
 IC_EXPORT int ic_attn_latent(const void* qa, int qa_stride, void* out, int out_stride, int dtype, const void* cache,
                              const int* block_tables, int bt_stride, const int* token_req, const int* positions,
-                             const int* row_list, int T, int H, int R, int E, int page_size, float scale, int n_split,
+                             const int* row_list, int T, int H, int R, int E, int page_size, float scale, int window,
+                             const float* sinks, int n_split,
                              float* part_acc, float* part_ml, int force_vector, hipStream_t stream) {
     if (T <= 0) return IC_OK;
-    if (H <= 0 || R <= 0 || R > kLatentMaxRank || E < 0 || page_size <= 0 || n_split < 1 || n_split > 64) return IC_ERR_ARG;
+    if (H <= 0 || R <= 0 || R > kLatentMaxRank || E < 0 || page_size <= 0 || window < 0 || n_split < 1 || n_split > 64) return IC_ERR_ARG;
     if (n_split > 1 && (!part_acc || !part_ml)) return IC_ERR_ARG;
     const int D = R + E;
     const size_t lds = (size_t)kLatentHeads * D * sizeof(float);
@@ -466,13 +492,13 @@ IC_EXPORT int ic_attn_latent(const void* qa, int qa_stride, void* out, int out_s
 #define IC_LATM(RR, EE)                                                                                                  \
     if (R == RR && E == EE)                                                                                              \
         latent_mfma_launch<RR, EE>(wide, stream, qa, qa_stride, out, out_stride, cache, block_tables, bt_stride, token_req, \
-                                   positions, row_list, H, page_size, scale, n_split, part_acc, part_ml);
+                                   positions, row_list, H, page_size, scale, window, sinks, n_split, part_acc, part_ml);
         IC_LATM(64, 16) IC_LATM(64, 32) IC_LATM(64, 64) IC_LATM(128, 16) IC_LATM(128, 32) IC_LATM(128, 64)
         IC_LATM(256, 16) IC_LATM(256, 32) IC_LATM(256, 64) IC_LATM(512, 16) IC_LATM(512, 32) IC_LATM(512, 64)
 #undef IC_LATM
         if (n_split > 1)
             hipLaunchKernelGGL(attn_latent_merge_kernel<bf16>, dim3(T * H), dim3(256), 0, stream, part_acc, part_ml, n_split, H,
-                               R, (bf16*)out, out_stride, row_list);
+                               R, (bf16*)out, out_stride, row_list, sinks);
         return ic_launch_status();
     }
     const int n_groups = (H + kLatentHeads - 1) / kLatentHeads;
@@ -481,7 +507,7 @@ IC_EXPORT int ic_attn_latent(const void* qa, int qa_stride, void* out, int out_s
 #define IC_LAT(TT, VV)                                                                                                 \
     hipLaunchKernelGGL((attn_latent_kernel<TT, VV>), grid, block, lds, stream, (const TT*)qa, qa_stride, (TT*)out,     \
                        out_stride, (const TT*)cache, block_tables, bt_stride, token_req, positions, row_list, H, R, E,  \
-                       page_size, scale, n_split, part_acc, part_ml)
+                       page_size, scale, window, sinks, n_split, part_acc, part_ml)
     if (dtype == IC_F32) {
         if (R % 4 == 0 && E % 4 == 0) IC_LAT(float, 4); else IC_LAT(float, 1);
     } else if (dtype == IC_BF16) {
@@ -492,12 +518,50 @@ IC_EXPORT int ic_attn_latent(const void* qa, int qa_stride, void* out, int out_s
     if (n_split > 1) {
         if (dtype == IC_F32)
             hipLaunchKernelGGL(attn_latent_merge_kernel<float>, dim3(T * H), dim3(256), 0, stream, part_acc, part_ml, n_split,
-                               H, R, (float*)out, out_stride, row_list);
+                               H, R, (float*)out, out_stride, row_list, sinks);
         else
             hipLaunchKernelGGL(attn_latent_merge_kernel<bf16>, dim3(T * H), dim3(256), 0, stream, part_acc, part_ml, n_split,
-                               H, R, (bf16*)out, out_stride, row_list);
+                               H, R, (bf16*)out, out_stride, row_list, sinks);
     }
     return ic_launch_status();
+}
+
+// ---- prompt portions: keys and values made per head --------------------------------------------------------------------
+// `kv` holds one row per key from key0 on, every head's key part and, from column v_off on, every head's value (a product of
+// the gathered latent rows); `rows` the gathered rows themselves, whose last E columns are the shared rotated key part.  The
+// portion's tokens are rows row0 .. row0 + n - 1 of q (rotated in place), out and gate, at positions pos0 and up.
+// Key sizes dim + E up to 192 and values up to 128, each made of whole 16-byte pieces.
+IC_EXPORT int ic_attn_latent_prefill_supported(int dtype, int dim, int E, int dv) {
+    return dtype == IC_BF16 && dim > 0 && E >= 0 && dv > 0 && dim % 8 == 0 && E % 8 == 0 && dv % 8 == 0 && dim + E <= 192 && dv <= 128;
+}
+
+IC_EXPORT int ic_attn_latent_prefill(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype,
+                                     const void* kv, int kv_stride, int v_off, const void* rows, int rows_stride, int R, int key0,
+                                     int row0, int n, int pos0, int H, int dim, int E, int dv, float scale, int window,
+                                     const float* sinks, hipStream_t stream) {
+    if (n <= 0) return IC_OK;
+    if (!ic_attn_latent_prefill_supported(dtype, dim, E, dv)) return IC_ERR_UNSUPPORTED;
+    const int first = (window > 0 && pos0 - window + 1 > 0) ? pos0 - window + 1 : 0;
+    if (H <= 0 || R < 0 || window < 0 || row0 < 0 || pos0 < 0 || key0 < 0 || key0 > first || !(scale > 0.f)) return IC_ERR_ARG;
+    const uint16_t* krot = (const uint16_t*)rows + R;
+    if ((q_stride | kv_stride | v_off | rows_stride) & 7 || (out_stride & 3) || (gate && (gate_stride & 3)) ||
+        ((uintptr_t)q & 15) || ((uintptr_t)kv & 15) || ((uintptr_t)krot & 15) || ((uintptr_t)out & 7) || ((uintptr_t)gate & 7))
+        return IC_ERR_ARG;
+    const long long blocks = (long long)((n + kSpRows - 1) / kSpRows) * H;
+    if (blocks > 0x7fffffffLL) return IC_ERR_ARG;
+    const SpanSizes z{dim + E, dv, E, kv_stride, v_off, key0, rows_stride, krot, int4{0, row0, n, pos0}};
+    const int dk = dim + E;
+#define IC_LATP(K, V)                                                                                                        \
+    if (dk <= K && dv <= V) {                                                                                                \
+        hipLaunchKernelGGL((attn_span_prefill_kernel<K, V, kSpanLatent>), dim3((unsigned)blocks), dim3(256), 0, stream,       \
+                           (const uint16_t*)q, q_stride, (uint16_t*)out, out_stride, (const uint16_t*)gate, gate_stride,      \
+                           (const uint16_t*)kv, nullptr, nullptr, 0, nullptr, H, H, 0, scale * kLog2e, window, 0,             \
+                           sinks ? 1 : 0, sinks, 0.f, nullptr, z);                                                           \
+        return ic_launch_status();                                                                                           \
+    }
+    IC_LATP(64, 64) IC_LATP(64, 96) IC_LATP(96, 64) IC_LATP(96, 96) IC_LATP(128, 64) IC_LATP(128, 128) IC_LATP(192, 64) IC_LATP(192, 128)
+#undef IC_LATP
+    return IC_ERR_UNSUPPORTED;
 }
 
 // ---- prompt portions through matrix products -------------------------------------------------------------------------
@@ -505,28 +569,29 @@ IC_EXPORT int ic_attn_latent(const void* qa, int qa_stride, void* out, int out_s
 // scores = Q' C^T and result = P C[:, :R].  The request's latent rows are gathered out of their pages into one
 // matrix (and its first R columns transposed, for the second product), the scores pass a masked softmax.
 
-// rows[j] = cache row of key j (j < L), zeros for L <= j < L_pad; rows_t[c, j] = rows[j, c] for c < R.
+// Row j of `rows` is key key0 + j.  rows[j] = the cache row of its key for first <= key < L, zeros for the other keys up to
+// L_pad rows; rows_t[c, j] = rows[j, c] for c < R (rows_t null: left out).
 template <typename T>
 __global__ void __launch_bounds__(256)
-latent_gather_kernel(const T* __restrict__ cache, const int* __restrict__ table, int page_size, int D, int R, int L,
-                     int L_pad, T* __restrict__ rows, T* __restrict__ rows_t) {
+latent_gather_kernel(const T* __restrict__ cache, const int* __restrict__ table, int page_size, int D, int R, int key0, int first,
+                     int L, int L_pad, T* __restrict__ rows, T* __restrict__ rows_t) {
     // blockIdx.y == 0: 64 keys' rows as they are; blockIdx.y = 1 + i: columns 64 i .. 64 i + 63 of the same keys, transposed
     __shared__ T tile[64][65];
     const int j0 = blockIdx.x * 64, lane = threadIdx.x % 64, w = threadIdx.x / 64;
     if (blockIdx.y == 0) {
         for (int jj = w; jj < 64; jj += 4) {
-            const int j = j0 + jj;
+            const int j = j0 + jj, key = key0 + j;
             if (j >= L_pad) break;
-            const T* src = j < L ? cache + ((long long)table[j / page_size] * page_size + j % page_size) * D : nullptr;
+            const T* src = (key >= first && key < L) ? cache + ((long long)table[key / page_size] * page_size + key % page_size) * D : nullptr;
             for (int c = lane; c < D; c += 64) rows[(size_t)j * D + c] = src ? src[c] : from_f32<T>(0.f);
         }
         return;
     }
     const int c0 = 64 * (blockIdx.y - 1);
     for (int jj = w; jj < 64; jj += 4) {
-        const int j = j0 + jj, c = c0 + lane;
+        const int j = j0 + jj, key = key0 + j, c = c0 + lane;
         T v = from_f32<T>(0.f);
-        if (j < L && c < R) v = cache[((long long)table[j / page_size] * page_size + j % page_size) * D + c];
+        if (j < L_pad && key >= first && key < L && c < R) v = cache[((long long)table[key / page_size] * page_size + key % page_size) * D + c];
         tile[jj][lane] = v;
     }
     __syncthreads();
@@ -536,50 +601,54 @@ latent_gather_kernel(const T* __restrict__ cache, const int* __restrict__ table,
     }
 }
 
-IC_EXPORT int ic_latent_gather(const void* cache, int dtype, const int* table, int page_size, int D, int R, int L, int L_pad,
-                               void* rows, void* rows_t, hipStream_t stream) {
+IC_EXPORT int ic_latent_gather(const void* cache, int dtype, const int* table, int page_size, int D, int R, int key0, int first, int L,
+                               int L_pad, void* rows, void* rows_t, hipStream_t stream) {
     if (L <= 0) return IC_OK;
-    if (page_size <= 0 || D <= 0 || R <= 0 || R > D || L_pad < L) return IC_ERR_ARG;
-    dim3 grid((L_pad + 63) / 64, 1 + (R + 63) / 64), block(256);
+    if (page_size <= 0 || D <= 0 || R <= 0 || R > D || key0 < 0 || first < key0 || L <= first || L_pad < L - key0) return IC_ERR_ARG;
+    dim3 grid((L_pad + 63) / 64, rows_t ? 1 + (R + 63) / 64 : 1), block(256);
     if (dtype == IC_F32)
-        hipLaunchKernelGGL(latent_gather_kernel<float>, grid, block, 0, stream, (const float*)cache, table, page_size, D, R, L,
-                           L_pad, (float*)rows, (float*)rows_t);
+        hipLaunchKernelGGL(latent_gather_kernel<float>, grid, block, 0, stream, (const float*)cache, table, page_size, D, R, key0, first,
+                           L, L_pad, (float*)rows, (float*)rows_t);
     else if (dtype == IC_BF16)
-        hipLaunchKernelGGL(latent_gather_kernel<bf16>, grid, block, 0, stream, (const bf16*)cache, table, page_size, D, R, L,
-                           L_pad, (bf16*)rows, (bf16*)rows_t);
+        hipLaunchKernelGGL(latent_gather_kernel<bf16>, grid, block, 0, stream, (const bf16*)cache, table, page_size, D, R, key0, first,
+                           L, L_pad, (bf16*)rows, (bf16*)rows_t);
     else
         return IC_ERR_UNSUPPORTED;
     return ic_launch_status();
 }
 
-// Row m belongs to token m / H of the portion, which sees keys 0 .. first_limit + m / H.  p = softmax(scale * s) over
-// them, zero beyond (up to n_cols).  One block per row; the scores are float32.
+// Column j of a row is key key0 + j.  Row m belongs to token m / H of the portion, at position pos0 + m / H, and head m % H;
+// p = softmax(scale * s) over the keys it sees (window, sinks: see above), zero elsewhere.  One block per row; the scores are
+// float32.
 template <typename T>
 __global__ void __launch_bounds__(256)
-latent_softmax_kernel(const float* __restrict__ s, int lds, T* __restrict__ p, int ldp, int H, int n_cols, int first_limit,
-                      float scale) {
+latent_softmax_kernel(const float* __restrict__ s, int lds, T* __restrict__ p, int ldp, int H, int n_cols, int key0, int pos0,
+                      float scale, int window, const float* __restrict__ sinks) {
     __shared__ float red[8];
-    const int m = blockIdx.x;
-    const int n = min(first_limit + m / H + 1, n_cols);
+    const int m = blockIdx.x, pos = pos0 + m / H;
+    const int n = min(pos - key0 + 1, n_cols);                       // columns lo .. n - 1 are seen
+    const int lo = window > 0 ? max(pos - window + 1 - key0, 0) : 0;
     const float* row = s + (size_t)m * lds;
     T* out = p + (size_t)m * ldp;
+    const float sink = sinks ? sinks[m % H] : -INFINITY;
     if (n_cols <= 16 * 256) {                 // the row is read once and waits in registers
         float v[16];
         float mx = -INFINITY;
 #pragma unroll
         for (int k = 0; k < 16; ++k) {
             const int j = threadIdx.x + 256 * k;
-            v[k] = j < n ? row[j] : -INFINITY;
+            v[k] = (j >= lo && j < n) ? row[j] : -INFINITY;
             mx = fmaxf(mx, v[k]);
         }
-        mx = block_max(mx, red) * scale;
+        mx = fmaxf(block_max(mx, red) * scale, sink);
         float sum = 0.f;
 #pragma unroll
         for (int k = 0; k < 16; ++k) {
-            v[k] = expf(v[k] * scale - mx);       // exp(-inf) = 0 beyond the visible keys
+            v[k] = expf(v[k] * scale - mx);       // exp(-inf) = 0 for the keys that are not seen
             sum += v[k];
         }
-        const float inv = 1.0f / block_sum(sum, red);
+        sum = block_sum(sum, red);
+        const float inv = 1.0f / (sum + (sinks ? expf(sink - mx) : 0.f));
 #pragma unroll
         for (int k = 0; k < 16; ++k) {
             const int j = threadIdx.x + 256 * k;
@@ -588,25 +657,26 @@ latent_softmax_kernel(const float* __restrict__ s, int lds, T* __restrict__ p, i
         return;
     }
     float mx = -INFINITY;
-    for (int j = threadIdx.x; j < n; j += blockDim.x) mx = fmaxf(mx, row[j]);
-    mx = block_max(mx, red) * scale;
+    for (int j = lo + threadIdx.x; j < n; j += blockDim.x) mx = fmaxf(mx, row[j]);
+    mx = fmaxf(block_max(mx, red) * scale, sink);
     float sum = 0.f;
-    for (int j = threadIdx.x; j < n; j += blockDim.x) sum += expf(row[j] * scale - mx);
-    const float inv = 1.0f / block_sum(sum, red);
+    for (int j = lo + threadIdx.x; j < n; j += blockDim.x) sum += expf(row[j] * scale - mx);
+    sum = block_sum(sum, red);
+    const float inv = 1.0f / (sum + (sinks ? expf(sink - mx) : 0.f));
     for (int j = threadIdx.x; j < n_cols; j += blockDim.x)
-        out[j] = from_f32<T>(j < n ? expf(row[j] * scale - mx) * inv : 0.f);
+        out[j] = from_f32<T>((j >= lo && j < n) ? expf(row[j] * scale - mx) * inv : 0.f);
 }
 
-IC_EXPORT int ic_latent_softmax(const float* s, int lds, void* p, int ldp, int dtype, int M, int H, int n_cols,
-                                int first_limit, float scale, hipStream_t stream) {
+IC_EXPORT int ic_latent_softmax(const float* s, int lds, void* p, int ldp, int dtype, int M, int H, int n_cols, int key0, int pos0,
+                                float scale, int window, const float* sinks, hipStream_t stream) {
     if (M <= 0) return IC_OK;
-    if (H <= 0 || n_cols <= 0 || first_limit < 0 || scale <= 0.f) return IC_ERR_ARG;
+    if (H <= 0 || n_cols <= 0 || pos0 < key0 || key0 < 0 || window < 0 || scale <= 0.f) return IC_ERR_ARG;
     if (dtype == IC_F32)
-        hipLaunchKernelGGL(latent_softmax_kernel<float>, dim3(M), dim3(256), 0, stream, s, lds, (float*)p, ldp, H, n_cols,
-                           first_limit, scale);
+        hipLaunchKernelGGL(latent_softmax_kernel<float>, dim3(M), dim3(256), 0, stream, s, lds, (float*)p, ldp, H, n_cols, key0,
+                           pos0, scale, window, sinks);
     else if (dtype == IC_BF16)
-        hipLaunchKernelGGL(latent_softmax_kernel<bf16>, dim3(M), dim3(256), 0, stream, s, lds, (bf16*)p, ldp, H, n_cols,
-                           first_limit, scale);
+        hipLaunchKernelGGL(latent_softmax_kernel<bf16>, dim3(M), dim3(256), 0, stream, s, lds, (bf16*)p, ldp, H, n_cols, key0,
+                           pos0, scale, window, sinks);
     else
         return IC_ERR_UNSUPPORTED;
     return ic_launch_status();

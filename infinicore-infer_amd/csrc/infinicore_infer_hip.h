@@ -74,24 +74,25 @@ int ic_embed_sinusoid(const int* tokens, const int* positions, const void* table
 int ic_norm_into_stream(const void* y, int y_dtype, const float* bias, const float* w, float* x, void* copy, int copy_dtype, int T, int d, float eps, hipStream_t stream);
 // A token's projected row [q | k | v | ..]: bias, query/key norm (norm_mode 0 none, 1 per head with w[dk], 2 whole row with w[nh dk] / w[nkvh dk]),
 // value mixing (mix_mode 0 none, 1 keep v in v_keep float32 [T, nkvh dv], 2 v = (1 - lambda[0]) v + lambda[0] v_keep), q to q_out [T, nh dk],
-// k and v to the cache planes at slots[t] (K [pages, nkvh, page_size, dk], V [.., dv]).
-int ic_qk_norm_store(const void* rows, int row_stride, int dtype, const float* bias, const float* qw, const float* kw, int norm_mode, float eps, int mix_mode, const float* lambda, float* v_keep, void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh, int nkvh, int dk, int dv, int page_size, hipStream_t stream);
+// k and v to the cache planes at slots[t] (K [pages, nkvh, page_size, dk], V [.., dv]).  v_from: the column of the row where the
+// values begin ((nh + nkvh) dk; nh dk: the values are the keys as projected).
+int ic_qk_norm_store(const void* rows, int row_stride, int dtype, const float* bias, const float* qw, const float* kw, int norm_mode, float eps, int mix_mode, const float* lambda, float* v_keep, void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh, int nkvh, int dk, int dv, int page_size, int v_from, hipStream_t stream);
 // out = act(in) element by element; kind 0: relu(z)^2, 1: gelu_tanh(z), 2: silu(z).
 int ic_activation(const void* in, void* out, int dtype, long long n, int kind, hipStream_t stream);
 
 // ---- attn_span.hip: keys and values of different sizes, a window plus kept first keys, a sink, an output gate --------
 // Query at position i sees key j when j <= i and (window == 0 or i - j < window or j < keep_first); sink: 1 joins the
-// softmax's denominator; gate (nullable): out *= sigmoid(gate[t, h dv + d]).
-int ic_attn_span_generic(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype, const void* kcache, const void* vcache, const int* block_tables, int bt_stride, const int* token_req, const int* positions, int T, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int keep_first, int sink, const float* sinks, float softcap, hipStream_t stream);
+// softmax's denominator; gate (nullable): out *= sigmoid(gate[t, h dv + d]).  slopes (nullable, float32 [nh]): slopes[h] (i - j) is taken off the scaled, capped score.
+int ic_attn_span_generic(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype, const void* kcache, const void* vcache, const int* block_tables, int bt_stride, const int* token_req, const int* positions, int T, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int keep_first, int sink, const float* sinks, float softcap, const float* slopes, hipStream_t stream);
 
-// Single new tokens, split over the visible keys (key and value sizes 32, 64, 128; float32 or bfloat16).  tok_list (nullable): the rows that are
+// Single new tokens, split over the visible keys (key and value sizes of whole 16-byte pieces up to 128; float32 or bfloat16).  tok_list (nullable): the rows that are
 // single tokens.  part_acc: float32 [n_tok, nh, nsplit, dv]; part_ml: float32 [n_tok, nh, nsplit, 2]; nsplit <= 32 (1: no second pass, no scratch).
 int ic_attn_span_decode_supported(int dtype, int dk, int dv);
 int ic_attn_span_decode_splits(int n_rows, int n_kv_heads, int max_keys, int compute_units);
-int ic_attn_span_decode(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype, const void* kcache, const void* vcache, const int* block_tables, int bt_stride, const int* tok_list, const int* token_req, const int* positions, float* part_acc, float* part_ml, int n_tok, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int keep_first, int sink, const float* sinks, float softcap, int nsplit, hipStream_t stream);
-// Prompt portions on the matrix cores (bfloat16; key and value sizes 32, 64, 128; scale > 0).  tiles as for ic_attn_prefill, rows <= 128.
+int ic_attn_span_decode(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype, const void* kcache, const void* vcache, const int* block_tables, int bt_stride, const int* tok_list, const int* token_req, const int* positions, float* part_acc, float* part_ml, int n_tok, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int keep_first, int sink, const float* sinks, float softcap, const float* slopes, int nsplit, hipStream_t stream);
+// Prompt portions on the matrix cores (bfloat16; key and value sizes multiples of 8 up to 128; scale > 0).  tiles as for ic_attn_prefill, rows <= 128.
 int ic_attn_span_prefill_supported(int dtype, int dk, int dv);
-int ic_attn_span_prefill(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype, const void* kcache, const void* vcache, const int* block_tables, int bt_stride, const int* tiles, int n_tiles, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int keep_first, int sink, const float* sinks, float softcap, hipStream_t stream);
+int ic_attn_span_prefill(const void* q, int q_stride, void* out, int out_stride, const void* gate, int gate_stride, int dtype, const void* kcache, const void* vcache, const int* block_tables, int bt_stride, const int* tiles, int n_tiles, int nh, int nkvh, int dk, int dv, int page_size, float scale, int window, int keep_first, int sink, const float* sinks, float softcap, const float* slopes, hipStream_t stream);
 
 // ---- gemm.hip ---------------------------------------------------------------------------------------
 // A norm y = x * rsqrt(mean(x^2) + eps) * w between two products of M <= 16 rows can be split over them: the
@@ -181,9 +182,11 @@ int ic_token_gate(const void* z, int z_stride, const void* table, int table_stri
 int ic_conv_rope_norm_store(const void* rows, int row_stride, int dtype, const float* cw, int taps, const int* positions, const float* freq, int rot_dims, const float* qw, const float* kw, int norm, float eps, void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh, int nkvh, int dk, int dv, int page_size, float* state, long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int R, int single, hipStream_t stream);
 // x = rmsnorm(alpha x + sa ya + sb yb) * w, the norm on the sum; copy: the new x in the results' dtype.
 int ic_sum_norm(const void* ya, float sa, const void* yb, float sb, int dtype, float alpha, const float* w, float* x, void* copy, int T, int d, float eps, hipStream_t stream);
+// x += s0 y0 (+ s1 y1 (+ s2 y2)), n of them; h (nullable) = rmsnorm(x) * w, in the results' dtype.
+int ic_branches_norm(const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, int n, int dtype, const float* w, float* x, void* h, int T, int d, float eps, hipStream_t stream);
 
 // ---- matrix_memory.hip: recurrences with a matrix state per head, decays per key channel or per head, the delta rule --------
-int ic_delta_prep(const void* rows, int row_stride, int dtype, const float* w, int taps, const void* b, int b_stride, float* out, float* beta, int G, int H, int dk, int dv, float unit_eps, float* state, long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int T, int R, int single, hipStream_t stream);
+int ic_delta_prep(const void* rows, int row_stride, int dtype, const float* w, int taps, const void* b, int b_stride, float* out, float* beta, int G, int H, int dk, int dv, float unit_eps, float* state, long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int T, int R, int single, const void* a, int a_stride, const float* rate, const float* a_bias, float* decay, hipStream_t stream);
 int ic_memory_gates(const float* z, int z_stride, const float* bi, const float* bf, float cap, int H, float* keep, float* add, float* floor_, float* state, long long state_stride, const int* req_start, const int* state_slots, int T, int R, hipStream_t stream);
 int ic_matrix_memory(const void* q, int q_stride, const void* k, int k_stride, const void* v, int v_stride, int dtype, const float* decay, int per_channel, const float* scale, int delta, int H, int per, int dk, int dv, float q_scale, float* out, float* extra_out, float* state, long long state_stride, const int* req_start, const int* state_slots, int R, int single, int columns_a_thread, hipStream_t stream);
 int ic_gated_head_norm(const float* y, const float* num, const float* floor_, const void* z, int z_stride, int dtype, const float* w, int w_shared, int T, int H, int dv, float eps, void* out, int gate, hipStream_t stream);

@@ -7,7 +7,7 @@
 // decayed keys against q) normalises the others.
 //
 //   * ic_delta_prep: the delta rule's rows: convolution and silu on q, k, v, unit length per head for q and k, the step
-//     sizes sigmoid(b), and the convolution's state,
+//     sizes sigmoid(b), one decay per head where the rule has that, and the convolution's state,
 //   * ic_memory_gates: exponential input and forget gates held in logarithms against a running maximum, as factors,
 //   * ic_matrix_step: one token per request, ic_matrix_scan: portions,
 //   * ic_gated_head_norm: o per head to unit root mean square, a weight, a gate.
@@ -26,23 +26,36 @@ __device__ __forceinline__ float mm_silu_fast(float z) { return z * mm_sigmoid_f
 
 // ---------------------------------------------------------------------------------------------
 // rows[t] = [q (G dk) | k (G dk) | v (H dv) | ..]: every channel passes the convolution and silu; q and k heads are then
-// divided by sqrt(sum of squares + unit_eps).  out [T, 2 G dk + H dv] float32; beta[t, h] = sigmoid(b[t, h]).
+// divided by sqrt(sum of squares + unit_eps).  out [T, 2 G dk + H dv] float32; beta[t, h] = sigmoid(b[t, h]);
+// with d.a: d.decay[t, h] = exp(-d.rate[h] softplus(a[t, h] + d.bias[h])), one decay factor per head.
 // grid (T, ceil((2 G + H + 1) / 4)), a wave a head (the last one: the step sizes).  single: every request brings one
 // token, and the wave moves the convolution's state on itself.
 // ---------------------------------------------------------------------------------------------
 constexpr int kPrepMaxPerLane = 16;
+
+struct HeadDecay { const void* a; int a_stride; const float *rate, *bias; float* decay; };
+
+// The step sizes and decay factors of tokens t0 .. t1 - 1, by one wave.
+template <typename T>
+__device__ __forceinline__ void head_steps(const T* b, int b_stride, float* beta, const HeadDecay& d, int H, int t0, int t1, int lane) {
+    for (int e = t0 * H + lane; e < t1 * H; e += 64) {
+        const int t = e / H, h = e - t * H;
+        beta[e] = mm_sigmoid(to_f32(b[(size_t)t * b_stride + h]));
+        if (d.a) d.decay[e] = expf(-d.rate[h] * mm_softplus(to_f32(((const T*)d.a)[(size_t)t * d.a_stride + h]) + d.bias[h]));
+    }
+}
 
 template <typename T>
 __global__ void __launch_bounds__(256)
 delta_prep_kernel(const T* __restrict__ rows, int row_stride, const float* __restrict__ w, int taps, const T* __restrict__ b,
                   int b_stride, float* __restrict__ out, float* __restrict__ beta, int G, int H, int dk, int dv,
                   float unit_eps, float* __restrict__ state, long long state_stride, const int* __restrict__ token_req,
-                  const int* __restrict__ req_start, const int* __restrict__ state_slots, int single) {
+                  const int* __restrict__ req_start, const int* __restrict__ state_slots, int single, HeadDecay d) {
     const int t = blockIdx.x, lane = threadIdx.x & 63, head = blockIdx.y * 4 + (threadIdx.x >> 6);
     const int C = 2 * G * dk + H * dv;
     if (head > 2 * G + H) return;
     if (head == 2 * G + H) {
-        for (int i = lane; i < H; i += 64) beta[(size_t)t * H + i] = mm_sigmoid(to_f32(b[(size_t)t * b_stride + i]));
+        head_steps<T>(b, b_stride, beta, d, H, t, t + 1, lane);
         return;
     }
     const int r = token_req[t], start = req_start[r];
@@ -87,14 +100,13 @@ __global__ void __launch_bounds__(256)
 delta_prep_tile_kernel(const T* __restrict__ rows, int row_stride, const float* __restrict__ w, int taps, const T* __restrict__ b,
                        int b_stride, float* __restrict__ out, float* __restrict__ beta, int G, int H, int dk, int dv, float unit_eps,
                        const float* __restrict__ state, long long state_stride, const int* __restrict__ token_req,
-                       const int* __restrict__ req_start, const int* __restrict__ state_slots, int n_tokens) {
+                       const int* __restrict__ req_start, const int* __restrict__ state_slots, int n_tokens, HeadDecay d) {
     const int lane = threadIdx.x & 63, head = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int t0 = blockIdx.x * kPrepTile, t1 = min(n_tokens, t0 + kPrepTile);
     const int C = 2 * G * dk + H * dv;
     if (head > 2 * G + H) return;
     if (head == 2 * G + H) {
-        for (int t = t0; t < t1; ++t)
-            for (int i = lane; i < H; i += 64) beta[(size_t)t * H + i] = mm_sigmoid(to_f32(b[(size_t)t * b_stride + i]));
+        head_steps<T>(b, b_stride, beta, d, H, t0, t1, lane);
         return;
     }
     const bool unit = head < 2 * G;
@@ -154,13 +166,13 @@ delta_prep_tile_kernel(const T* __restrict__ rows, int row_stride, const float* 
 template <typename T>
 static bool delta_prep_tiles(const T* rows, int row_stride, const float* w, int taps, const T* b, int b_stride, float* out, float* beta,
                              int G, int H, int dk, int dv, float unit_eps, const float* state, long long state_stride,
-                             const int* token_req, const int* req_start, const int* state_slots, int T_, hipStream_t stream) {
+                             const int* token_req, const int* req_start, const int* state_slots, int T_, const HeadDecay& d, hipStream_t stream) {
     const int n = dk > dv ? dk : dv;
     if (T_ < 64 || n > 256 || dk % 2 || dv % 2 || row_stride % 2 || (uintptr_t)rows % (2 * sizeof(T)) || (uintptr_t)out % 8) return false;
     dim3 grid((T_ + kPrepTile - 1) / kPrepTile, (2 * G + H + 1 + 3) / 4), block(256);
 #define IC_DP(TM, NJ_)                                                                                                          \
     hipLaunchKernelGGL((delta_prep_tile_kernel<T, TM, NJ_>), grid, block, 0, stream, rows, row_stride, w, taps, b, b_stride, out, \
-                       beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, T_)
+                       beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, T_, d)
     if (taps <= 4) { if (n <= 128) IC_DP(4, 1); else IC_DP(4, 2); }
     else { if (n <= 128) IC_DP(8, 1); else IC_DP(8, 2); }
 #undef IC_DP
@@ -170,8 +182,12 @@ static bool delta_prep_tiles(const T* rows, int row_stride, const float* w, int 
 IC_EXPORT int ic_delta_prep(const void* rows, int row_stride, int dtype, const float* w, int taps, const void* b, int b_stride,
                             float* out, float* beta, int G, int H, int dk, int dv, float unit_eps, float* state,
                             long long state_stride, const int* token_req, const int* req_start, const int* state_slots, int T,
-                            int R, int single, hipStream_t stream) {
+                            int R, int single, const void* a, int a_stride, const float* rate, const float* a_bias, float* decay,
+                            hipStream_t stream) {
     if (T <= 0) return IC_OK;
+    if (a && (!rate || !a_bias || !decay)) return IC_ERR_ARG;
+    if ((long long)T * H > 0x7fffffff) return IC_ERR_TOO_LARGE;
+    const HeadDecay d{a, a_stride, rate, a_bias, decay};
     if (G <= 0 || H <= 0 || dk <= 0 || dv <= 0 || taps < 1 || taps > kConvMaxTaps || R <= 0 || !state || !w) return IC_ERR_ARG;
     if (dk > 64 * kPrepMaxPerLane || dv > 64 * kPrepMaxPerLane) return IC_ERR_TOO_LARGE;
     if (single && T != R) return IC_ERR_ARG;
@@ -179,17 +195,17 @@ IC_EXPORT int ic_delta_prep(const void* rows, int row_stride, int dtype, const f
     dim3 grid(T, (2 * G + H + 1 + 3) / 4), block(256), sgrid((C + 255) / 256, R);
     if (dtype == IC_F32) {
         if (single || !delta_prep_tiles<float>((const float*)rows, row_stride, w, taps, (const float*)b, b_stride, out, beta, G, H, dk, dv, unit_eps,
-                                           state, state_stride, token_req, req_start, state_slots, T, stream))
+                                           state, state_stride, token_req, req_start, state_slots, T, d, stream))
             hipLaunchKernelGGL(delta_prep_kernel<float>, grid, block, 0, stream, (const float*)rows, row_stride, w, taps, (const float*)b,
-                           b_stride, out, beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, single);
+                           b_stride, out, beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, single, d);
         if (taps > 1 && !single)
             hipLaunchKernelGGL(conv_state_kernel<float>, sgrid, block, 0, stream, (const float*)rows, row_stride, nullptr, taps, C,
                                state, state_stride, req_start, state_slots);
     } else if (dtype == IC_BF16) {
         if (single || !delta_prep_tiles<bf16>((const bf16*)rows, row_stride, w, taps, (const bf16*)b, b_stride, out, beta, G, H, dk, dv, unit_eps,
-                                           state, state_stride, token_req, req_start, state_slots, T, stream))
+                                           state, state_stride, token_req, req_start, state_slots, T, d, stream))
             hipLaunchKernelGGL(delta_prep_kernel<bf16>, grid, block, 0, stream, (const bf16*)rows, row_stride, w, taps, (const bf16*)b,
-                           b_stride, out, beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, single);
+                           b_stride, out, beta, G, H, dk, dv, unit_eps, state, state_stride, token_req, req_start, state_slots, single, d);
         if (taps > 1 && !single)
             hipLaunchKernelGGL(conv_state_kernel<bf16>, sgrid, block, 0, stream, (const bf16*)rows, row_stride, nullptr, taps, C,
                                state, state_stride, req_start, state_slots);
@@ -631,8 +647,9 @@ IC_EXPORT int ic_matrix_memory(const void* q, int q_stride, const void* k, int k
     a.vec = dk % (16 / es) == 0 && dk % 4 == 0 && aligned(q, q_stride, es) && aligned(k, k_stride, es) && aligned(state, state_stride, 4) &&
             (!per_channel || aligned(decay, (long long)H * dk, 4));
     if (delta) {
-        if (dtype != IC_F32 || !per_channel || extra_out) return IC_ERR_UNSUPPORTED;
-        return matrix_memory_launch<float, true, true>(a, R, single, columns_a_thread, stream);
+        if (dtype != IC_F32 || extra_out) return IC_ERR_UNSUPPORTED;
+        return per_channel ? matrix_memory_launch<float, true, true>(a, R, single, columns_a_thread, stream)
+                           : matrix_memory_launch<float, true, false>(a, R, single, columns_a_thread, stream);
     }
     if (dtype == IC_F32)
         return per_channel ? matrix_memory_launch<float, false, true>(a, R, single, columns_a_thread, stream)

@@ -158,6 +158,7 @@ IC_EXPORT int ic_norm_into_stream(const void* y, int y_dtype, const float* bias,
 // norm_mode 0: none; 1: every head's dk entries to unit root mean square, times w[dk] (shared by the heads; qw and kw both
 // null: no weight);
 // 2: the whole of q (or k) to unit root mean square, times w[nh * dk] (or w[nkvh * dk]).
+// The value heads are read from column v_from on (nq + nk: behind the keys; nq: the values are the keys as projected).
 // One wave per (token, head of q, k or v); head sizes up to 512.
 // ---------------------------------------------------------------------------------------------
 template <typename T>
@@ -166,12 +167,12 @@ qk_norm_store_kernel(const T* __restrict__ rows, int row_stride, const float* __
                      const float* __restrict__ qw, const float* __restrict__ kw, int norm_mode, float eps,
                      int mix_mode, const float* __restrict__ lambda, float* __restrict__ v_keep,
                      T* __restrict__ q_out, T* __restrict__ kcache, T* __restrict__ vcache,
-                     const int* __restrict__ slots, int nh, int nkvh, int dk, int dv, int page_size) {
+                     const int* __restrict__ slots, int nh, int nkvh, int dk, int dv, int page_size, int v_from) {
     // Grid (tokens, ceil(heads / 4)): one wave per head of q, k or v; a lane holds up to 8 of the head's entries.
     const int t = blockIdx.x, lane = threadIdx.x & 63;
     const int head = blockIdx.y * 4 + (threadIdx.x >> 6);
     if (head >= nh + 2 * nkvh) return;
-    const int nq = nh * dk, nk = nkvh * dk, nv = nkvh * dv;
+    const int nq = nh * dk, nv = nkvh * dv;
     const T* src = rows + (size_t)t * row_stride;
     const int slot = slots ? slots[t] : -1;
     const int pg = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot - pg * page_size : 0;
@@ -193,7 +194,7 @@ qk_norm_store_kernel(const T* __restrict__ rows, int row_stride, const float* __
 #pragma unroll
             for (int j = 0; j < 8; ++j) { const int e = lane + 64 * j; if (e < dk) val[j] = val[j] * r * (w ? w[e] : 1.f); }
         } else if (norm_mode == 2) {                      // the sum runs over the whole of q (or k), which every wave reads
-            const int p0 = is_q ? 0 : nq, pn = is_q ? nq : nk;
+            const int p0 = is_q ? 0 : nq, pn = is_q ? nq : nkvh * dk;
             float ss = 0.f;
             for (int i = lane; i < pn; i += 64) { const float v = to_f32(src[p0 + i]) + (bias ? bias[p0 + i] : 0.f); ss += v * v; }
             const float r = 1.0f / sqrtf(wave_sum(ss) / (float)pn + eps);
@@ -209,7 +210,7 @@ qk_norm_store_kernel(const T* __restrict__ rows, int row_stride, const float* __
         }
         return;
     }
-    const int vh = head - nh - nkvh, base = nq + nk + vh * dv;
+    const int vh = head - nh - nkvh, base = v_from + vh * dv;
     const float lam = (mix_mode == 2) ? lambda[0] : 0.f;
     T* dst = (slot >= 0 && vcache) ? vcache + (((size_t)pg * nkvh + vh) * page_size + off) * dv : nullptr;
 #pragma unroll
@@ -234,7 +235,7 @@ qk_norm_store_vec_kernel(const T* __restrict__ rows, int row_stride, const float
                          const float* __restrict__ qw, const float* __restrict__ kw, int norm_mode, float eps,
                          int mix_mode, const float* __restrict__ lambda, float* __restrict__ v_keep,
                          T* __restrict__ q_out, T* __restrict__ kcache, T* __restrict__ vcache,
-                         const int* __restrict__ slots, int nh, int nkvh, int dk, int dv, int page_size, int qk_items_padded) {
+                         const int* __restrict__ slots, int nh, int nkvh, int dk, int dv, int page_size, int qk_items_padded, int v_from) {
     constexpr int N = RowPack<T>::N;
     const int t = blockIdx.x, lane = threadIdx.x & 63;
     const int item = blockIdx.y * 256 + threadIdx.x;
@@ -279,10 +280,10 @@ qk_norm_store_vec_kernel(const T* __restrict__ rows, int row_stride, const float
     const int vi = item - qk_items_padded;
     if (vi >= nv / N) return;
     const int e0 = vi * N, vh = e0 / dv, j0 = e0 - vh * dv;
-    RowPack<T>::load(src + nq + nk + e0, val);
+    RowPack<T>::load(src + v_from + e0, val);
     if (bias) {
         float b[N];
-        load_floats<N>(bias + nq + nk + e0, b);
+        load_floats<N>(bias + v_from + e0, b);
 #pragma unroll
         for (int i = 0; i < N; ++i) val[i] += b[i];
     }
@@ -309,7 +310,7 @@ qk_norm_store_whole_kernel(const T* __restrict__ rows, int row_stride, const flo
                            const float* __restrict__ qw, const float* __restrict__ kw, float eps,
                            int mix_mode, const float* __restrict__ lambda, float* __restrict__ v_keep,
                            T* __restrict__ q_out, T* __restrict__ kcache, T* __restrict__ vcache,
-                           const int* __restrict__ slots, int nh, int nkvh, int dk, int dv, int page_size) {
+                           const int* __restrict__ slots, int nh, int nkvh, int dk, int dv, int page_size, int v_from) {
     constexpr int N = RowPack<T>::N;
     __shared__ float red[16];
     const int t = blockIdx.x, tid = threadIdx.x;
@@ -351,8 +352,8 @@ qk_norm_store_whole_kernel(const T* __restrict__ rows, int row_stride, const flo
     for (int vi = tid; vi < nv / N; vi += blockDim.x) {
         const int e0 = vi * N, vh = e0 / dv, j0 = e0 - vh * dv;
         float v[N], b[N], kv[N];
-        RowPack<T>::load(src + nq + nk + e0, v);
-        if (bias) load_floats<N>(bias + nq + nk + e0, b);
+        RowPack<T>::load(src + v_from + e0, v);
+        if (bias) load_floats<N>(bias + v_from + e0, b);
         float* keep = v_keep + (size_t)t * nv + e0;
         if (mix_mode == 2) load_floats<N>(keep, kv);
 #pragma unroll
@@ -371,17 +372,16 @@ qk_norm_store_whole_kernel(const T* __restrict__ rows, int row_stride, const flo
 IC_EXPORT int ic_qk_norm_store(const void* rows, int row_stride, int dtype, const float* bias, const float* qw,
                                const float* kw, int norm_mode, float eps, int mix_mode, const float* lambda,
                                float* v_keep, void* q_out, void* kcache, void* vcache, const int* slots, int T, int nh,
-                               int nkvh, int dk, int dv, int page_size, hipStream_t stream) {
+                               int nkvh, int dk, int dv, int page_size, int v_from, hipStream_t stream) {
     if (T <= 0) return IC_OK;
-    if (nh <= 0 || nkvh <= 0 || dk <= 0 || dv <= 0 || page_size <= 0 || norm_mode < 0 || norm_mode > 2 || mix_mode < 0 ||
+    if (nh <= 0 || nkvh <= 0 || dk <= 0 || dv <= 0 || page_size <= 0 || v_from < 0 || norm_mode < 0 || norm_mode > 2 || mix_mode < 0 ||
         mix_mode > 2)
         return IC_ERR_ARG;
     if ((qw == nullptr) != (kw == nullptr)) return IC_ERR_ARG;
     if (norm_mode == 2 && qw == nullptr) return IC_ERR_ARG;       // the per-head norm (1) may come without weights
     if (mix_mode != 0 && v_keep == nullptr) return IC_ERR_ARG;
     if (mix_mode == 2 && lambda == nullptr) return IC_ERR_ARG;
-    const long long n = (long long)(nh + nkvh) * dk + (long long)nkvh * dv;
-    if (row_stride < n) return IC_ERR_ARG;
+    if (row_stride < (long long)(nh + nkvh) * dk || row_stride < v_from + (long long)nkvh * dv) return IC_ERR_ARG;
     if (dk > 512 || dv > 512) return IC_ERR_TOO_LARGE;
     const size_t lds = 0;
     {
@@ -392,17 +392,18 @@ IC_EXPORT int ic_qk_norm_store(const void* rows, int row_stride, int dtype, cons
         const bool pow2 = lph > 0 && lph <= 64 && (lph & (lph - 1)) == 0;
         const uintptr_t ptrs = (uintptr_t)rows | (uintptr_t)q_out | (uintptr_t)kcache | (uintptr_t)vcache | (uintptr_t)bias |
                                (uintptr_t)qw | (uintptr_t)kw | (uintptr_t)v_keep;
-        if ((dtype == IC_F32 || dtype == IC_BF16) && pow2 && dv % pack == 0 && row_stride % pack == 0 && (ptrs & 15) == 0) {
+        if ((dtype == IC_F32 || dtype == IC_BF16) && (pow2 || (norm_mode == 2 && lph > 0)) && dv % pack == 0 && row_stride % pack == 0 &&
+            v_from % pack == 0 && (ptrs & 15) == 0) {
             if (norm_mode == 2) {
                 const int threads = ((long long)(nh + nkvh) * dk / pack > 512) ? 1024 : 256;
                 if (dtype == IC_F32)
                     hipLaunchKernelGGL(qk_norm_store_whole_kernel<float>, dim3(T), dim3(threads), 0, stream, (const float*)rows, row_stride,
                                        bias, qw, kw, eps, mix_mode, lambda, v_keep, (float*)q_out, (float*)kcache, (float*)vcache, slots,
-                                       nh, nkvh, dk, dv, page_size);
+                                       nh, nkvh, dk, dv, page_size, v_from);
                 else
                     hipLaunchKernelGGL(qk_norm_store_whole_kernel<bf16>, dim3(T), dim3(threads), 0, stream, (const bf16*)rows, row_stride,
                                        bias, qw, kw, eps, mix_mode, lambda, v_keep, (bf16*)q_out, (bf16*)kcache, (bf16*)vcache, slots, nh,
-                                       nkvh, dk, dv, page_size);
+                                       nkvh, dk, dv, page_size, v_from);
                 return ic_launch_status();
             }
             const int qk_items = (int)(((long long)(nh + nkvh) * dk) / pack);
@@ -412,11 +413,11 @@ IC_EXPORT int ic_qk_norm_store(const void* rows, int row_stride, int dtype, cons
             if (dtype == IC_F32)
                 hipLaunchKernelGGL(qk_norm_store_vec_kernel<float>, vgrid, vblock, 0, stream, (const float*)rows, row_stride, bias, qw,
                                    kw, norm_mode, eps, mix_mode, lambda, v_keep, (float*)q_out, (float*)kcache, (float*)vcache, slots,
-                                   nh, nkvh, dk, dv, page_size, qk_padded);
+                                   nh, nkvh, dk, dv, page_size, qk_padded, v_from);
             else
                 hipLaunchKernelGGL(qk_norm_store_vec_kernel<bf16>, vgrid, vblock, 0, stream, (const bf16*)rows, row_stride, bias, qw, kw,
                                    norm_mode, eps, mix_mode, lambda, v_keep, (bf16*)q_out, (bf16*)kcache, (bf16*)vcache, slots, nh,
-                                   nkvh, dk, dv, page_size, qk_padded);
+                                   nkvh, dk, dv, page_size, qk_padded, v_from);
             return ic_launch_status();
         }
     }
@@ -424,11 +425,11 @@ IC_EXPORT int ic_qk_norm_store(const void* rows, int row_stride, int dtype, cons
     if (dtype == IC_F32)
         hipLaunchKernelGGL(qk_norm_store_kernel<float>, grid, block, lds, stream, (const float*)rows, row_stride, bias, qw,
                            kw, norm_mode, eps, mix_mode, lambda, v_keep, (float*)q_out, (float*)kcache, (float*)vcache,
-                           slots, nh, nkvh, dk, dv, page_size);
+                           slots, nh, nkvh, dk, dv, page_size, v_from);
     else if (dtype == IC_BF16)
         hipLaunchKernelGGL(qk_norm_store_kernel<bf16>, grid, block, lds, stream, (const bf16*)rows, row_stride, bias, qw, kw,
                            norm_mode, eps, mix_mode, lambda, v_keep, (bf16*)q_out, (bf16*)kcache, (bf16*)vcache, slots, nh,
-                           nkvh, dk, dv, page_size);
+                           nkvh, dk, dv, page_size, v_from);
     else
         return IC_ERR_UNSUPPORTED;
     return ic_launch_status();
@@ -766,6 +767,90 @@ IC_EXPORT int ic_sum_norm(const void* ya, float sa, const void* yb, float sb, in
     else if (dtype == IC_BF16) { if (vec) IC_SN(bf16, 4); else IC_SN(bf16, 1); }
     else return IC_ERR_UNSUPPORTED;
 #undef IC_SN
+    return ic_launch_status();
+}
+
+// ---------------------------------------------------------------------------------------------
+// x[t] += the sum of up to three s_i y_i[t] (sublayers that read one norm's output, or the branches of one sublayer); h[t]
+// (nullable) = the new x to unit root mean square times w, in h's type.  A block per row; the row waits in registers.
+// ---------------------------------------------------------------------------------------------
+struct BranchSum { const void* y[3]; float s[3]; int n; };
+
+template <typename T, int N>
+__global__ void __launch_bounds__(256)
+branches_norm_kernel(BranchSum b, const float* __restrict__ w, float* __restrict__ x, T* __restrict__ h, int d, float eps) {
+    __shared__ float red[16];
+    const int t = blockIdx.x, pieces = d / N, step = blockDim.x;
+    float* xr = x + (size_t)t * d;
+    auto sum = [&](int c, float* v) {
+        float y[3][N];
+        load_piece<float, N>(xr + c * N, v);
+#pragma unroll
+        for (int k = 0; k < 3; ++k)
+            if (k < b.n) load_piece<T, N>((const T*)b.y[k] + (size_t)t * d + c * N, y[k]);
+#pragma unroll
+        for (int k = 0; k < 3; ++k)
+            if (k < b.n)
+#pragma unroll
+                for (int i = 0; i < N; ++i) v[i] += b.s[k] * y[k][i];
+        store_piece<float, N>(xr + c * N, v);
+    };
+    float keep[kSumKeep][N];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < kSumKeep; ++j) {
+        const int c = threadIdx.x + j * step;
+        if (c < pieces) {
+            sum(c, keep[j]);
+#pragma unroll
+            for (int i = 0; i < N; ++i) ss += keep[j][i] * keep[j][i];
+        }
+    }
+    for (int c = threadIdx.x + kSumKeep * step; c < pieces; c += step) {
+        float v[N];
+        sum(c, v);                                   // (stored: the same thread reads it back below)
+#pragma unroll
+        for (int i = 0; i < N; ++i) ss += v[i] * v[i];
+    }
+    if (!h) return;
+    const float r = 1.0f / sqrtf(block_sum(ss, red) / (float)d + eps);
+    auto put = [&](int c, const float* v) {
+        float ws[N], o[N];
+        load_piece<float, N>(w + c * N, ws);
+#pragma unroll
+        for (int i = 0; i < N; ++i) o[i] = v[i] * r * ws[i];
+        store_piece<T, N>(h + (size_t)t * d + c * N, o);
+    };
+#pragma unroll
+    for (int j = 0; j < kSumKeep; ++j) {
+        const int c = threadIdx.x + j * step;
+        if (c < pieces) put(c, keep[j]);
+    }
+    for (int c = threadIdx.x + kSumKeep * step; c < pieces; c += step) {
+        float v[N];
+        load_piece<float, N>(xr + c * N, v);
+        put(c, v);
+    }
+}
+
+IC_EXPORT int ic_branches_norm(const void* y0, float s0, const void* y1, float s1, const void* y2, float s2, int n, int dtype,
+                               const float* w, float* x, void* h, int T, int d, float eps, hipStream_t stream) {
+    if (T <= 0) return IC_OK;
+    if (d <= 0 || n < 1 || n > 3 || !x || (h && !w)) return IC_ERR_ARG;
+    const BranchSum b{{y0, y1, y2}, {s0, s1, s2}, n};
+    uintptr_t ptrs = (uintptr_t)w | (uintptr_t)x | (uintptr_t)h;
+    for (int k = 0; k < n; ++k) {
+        if (!b.y[k]) return IC_ERR_ARG;
+        ptrs |= (uintptr_t)b.y[k];
+    }
+    const bool vec = d % 4 == 0 && (ptrs & 15) == 0;
+    const int pieces = vec ? d / 4 : d;
+    dim3 grid(T), block(pieces >= 256 ? 256 : (pieces + 63) / 64 * 64);
+#define IC_BN(TT, N) hipLaunchKernelGGL((branches_norm_kernel<TT, N>), grid, block, 0, stream, b, w, x, (TT*)h, d, eps)
+    if (dtype == IC_F32) { if (vec) IC_BN(float, 4); else IC_BN(float, 1); }
+    else if (dtype == IC_BF16) { if (vec) IC_BN(bf16, 4); else IC_BN(bf16, 1); }
+    else return IC_ERR_UNSUPPORTED;
+#undef IC_BN
     return ic_launch_status();
 }
 

@@ -111,14 +111,14 @@ _SIGNATURES = {
     "ic_attn_prefill_counter_ints": [],
     "ic_embed_sinusoid": [_P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _F, _P],
     "ic_norm_into_stream": [_P, _I, _P, _P, _P, _P, _I, _I, _I, _F, _P],
-    "ic_qk_norm_store": [_P, _I, _I, _P, _P, _P, _I, _F, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
+    "ic_qk_norm_store": [_P, _I, _I, _P, _P, _P, _I, _F, _I, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "ic_activation": [_P, _P, _I, _LL, _I, _P],
-    "ic_attn_span_generic": [_P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _F, _P],
+    "ic_attn_span_generic": [_P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _F, _P, _P],
     "ic_attn_span_decode_supported": [_I, _I, _I],
     "ic_attn_span_decode_splits": [_I, _I, _I, _I],
-    "ic_attn_span_decode": [_P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _F, _I, _P],
+    "ic_attn_span_decode": [_P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _I, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _F, _P, _I, _P],
     "ic_attn_span_prefill_supported": [_I, _I, _I],
-    "ic_attn_span_prefill": [_P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _F, _P],
+    "ic_attn_span_prefill": [_P, _I, _P, _I, _P, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _P, _F, _P, _P],
     "ic_pair_rows": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P],
     "ic_embed_streams": [_P, _P, _P, _P, _I, _P, _I, _I, _I, _P, _P, _P, _P],
     "ic_hc_step": [_P, _I, _I, _I, _P, _I, _P, _P, _P, _P, _F, _P, _I, _P],
@@ -131,16 +131,19 @@ _SIGNATURES = {
     "ic_decay_product": [_P, _I, _P, _I, _P, _I, _P, _P, _I, _F, _I, _I, _I, _P],
     "ic_conv_rope_norm_store": [_P, _I, _I, _P, _I, _P, _P, _I, _P, _P, _I, _F, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _LL, _P, _P, _P, _I, _I, _P],
     "ic_sum_norm": [_P, _F, _P, _F, _I, _F, _P, _P, _P, _I, _I, _F, _P],
-    "ic_delta_prep": [_P, _I, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _F, _P, _LL, _P, _P, _P, _I, _I, _I, _P],
+    "ic_branches_norm": [_P, _F, _P, _F, _P, _F, _I, _I, _P, _P, _P, _I, _I, _F, _P],
+    "ic_delta_prep": [_P, _I, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _F, _P, _LL, _P, _P, _P, _I, _I, _I, _P, _I, _P, _P, _P, _P],
     "ic_memory_gates": [_P, _I, _P, _P, _F, _I, _P, _P, _P, _P, _LL, _P, _P, _I, _I, _P],
     "ic_matrix_memory": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _P, _I, _I, _I, _I, _I, _F, _P, _P, _P, _LL, _P, _P, _I, _I, _I, _P],
     "ic_gated_head_norm": [_P, _P, _P, _P, _I, _I, _P, _I, _I, _I, _I, _F, _P, _I, _P],
-    "ic_latent_prep": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _P, _P, _P, _P, _I, _P],
-    "ic_latent_q_rotate": [_P, _I, _I, _I, _I, _I, _I, _P, _I, _P, _P, _I, _I, _P],
-    "ic_attn_latent": [_P, _I, _P, _I, _I, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _I, _P],
+    "ic_latent_prep": [_P, _I, _I, _I, _I, _I, _P, _P, _F, _P, _I, _F, _P, _P, _P, _P, _I, _P],
+    "ic_latent_q_rotate": [_P, _I, _I, _I, _I, _I, _I, _P, _I, _F, _P, _P, _I, _I, _P],
+    "ic_attn_latent": [_P, _I, _P, _I, _I, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _I, _P, _P, _I, _P],
     "ic_attn_latent_on_matrix_cores": [_I, _I, _I],
-    "ic_latent_gather": [_P, _I, _P, _I, _I, _I, _I, _I, _P, _P, _P],
-    "ic_latent_softmax": [_P, _I, _P, _I, _I, _I, _I, _I, _I, _F, _P],
+    "ic_attn_latent_prefill_supported": [_I, _I, _I, _I],
+    "ic_attn_latent_prefill": [_P, _I, _P, _I, _P, _I, _I, _P, _I, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P],
+    "ic_latent_gather": [_P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P, _P],
+    "ic_latent_softmax": [_P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P, _P],
     "ic_rope_pairs_store": [_P, _I, _I, _P, _P, _I, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "ic_pool_blocks": [_P, _P, _P, _P, _I, _P, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "ic_attn_pooled_generic": [_P, _I, _P, _I, _I, _P, _P, _P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _F, _I, _I, _P],

@@ -723,17 +723,21 @@ def norm_into_stream(y, weight, x, eps: float, bias=None, copy=None):
 
 
 def qk_norm_store(rows, bias, q_weight, k_weight, norm_mode: int, eps: float, mix_mode: int, mix_lambda, v_keep, q_out,
-                  kcache, vcache, slots, n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int, page_size: int):
+                  kcache, vcache, slots, n_heads: int, n_kv_heads: int, key_dim: int, value_dim: int, page_size: int,
+                  values_from_keys: bool = False):
     """One pass over the projected rows [q | k | v | ..]: bias, query/key norm (0 none, 1 per head, with weights or with
     both None to unit root mean square alone, 2 whole row), value
     mixing (0 none, 1 keep the values in ``v_keep``, 2 mix with ``v_keep`` by ``mix_lambda``), q to ``q_out``, k and v
-    into the cache planes at ``slots`` (None: no cache write)."""
+    into the cache planes at ``slots`` (None: no cache write).  ``values_from_keys``: the rows are [q | k | ..] and the values are
+    the keys as projected (with their bias, before their norm)."""
     _dev(rows, bias, q_weight, k_weight, mix_lambda, v_keep, q_out, kcache, vcache, slots)
     T = rows.shape[0]
     nq, nk, nv = n_heads * key_dim, n_kv_heads * key_dim, n_kv_heads * value_dim
-    _need(rows.dim() == 2 and rows.stride(1) == 1 and rows.shape[1] >= nq + nk + nv, "qk_norm_store: rows too short")
+    _need(not values_from_keys or value_dim == key_dim, "qk_norm_store: values that are keys have their size")
+    v_from = nq if values_from_keys else nq + nk
+    _need(rows.dim() == 2 and rows.stride(1) == 1 and rows.shape[1] >= v_from + nv, "qk_norm_store: rows too short")
     _need(tuple(q_out.shape) == (T, nq) and q_out.is_contiguous() and q_out.dtype == rows.dtype, "qk_norm_store: q_out layout")
-    for v, n, what in ((bias, nq + nk + nv, "bias"), (q_weight, (key_dim, nq)[norm_mode == 2], "q weight"),
+    for v, n, what in ((bias, v_from + nv, "bias"), (q_weight, (key_dim, nq)[norm_mode == 2], "q weight"),
                        (k_weight, (key_dim, nk)[norm_mode == 2], "k weight"), (mix_lambda, 1, "lambda")):
         if v is not None:
             _need(v.dtype == torch.float32 and v.is_contiguous() and v.numel() == n, "qk_norm_store: %s must be float32 [%d]" % (what, n))
@@ -754,7 +758,7 @@ def qk_norm_store(rows, bias, q_weight, k_weight, norm_mode: int, eps: float, mi
     check(get_lib().ic_qk_norm_store(rows.data_ptr(), rows.stride(0), dtype_code(rows.dtype), p(bias), p(q_weight), p(k_weight),
                                      int(norm_mode), float(eps), int(mix_mode), p(mix_lambda), p(v_keep), q_out.data_ptr(),
                                      p(kcache) if slots is not None else None, p(vcache) if slots is not None else None,
-                                     p(slots), T, n_heads, n_kv_heads, key_dim, value_dim, page_size, _stream()),
+                                     p(slots), T, n_heads, n_kv_heads, key_dim, value_dim, page_size, v_from, _stream()),
           "qk_norm_store")
 
 
@@ -816,6 +820,25 @@ def sum_norm(branches, alpha: float, weight, x, eps: float, copy=None):
     return x
 
 
+def branches_norm(branches, weight, x, eps: float, out=None):
+    """x += the sum of s_i y_i, row by row (x float32, in place); ``branches``: one to three (y, s); ``out`` (optional)
+    receives rmsnorm(x) * weight in the branches' dtype."""
+    _need(1 <= len(branches) <= 3, "branches_norm: one to three results")
+    T, d = x.shape
+    _dev(x, weight, out, *[y for y, _ in branches])
+    _need(x.dtype == torch.float32 and x.is_contiguous(), "branches_norm: the stream is float32")
+    first = branches[0][0]
+    for y in [y for y, _ in branches] + ([out] if out is not None else []):
+        _need(tuple(y.shape) == (T, d) and y.is_contiguous() and y.dtype == first.dtype, "branches_norm: layout")
+    if out is not None:
+        _need(weight.dtype == torch.float32 and weight.numel() == d and weight.is_contiguous(), "branches_norm: weight must be float32 [d]")
+    three = [(y.data_ptr(), float(f)) for y, f in branches] + [(None, 0.0)] * (3 - len(branches))
+    check(get_lib().ic_branches_norm(*[a for pair in three for a in pair], len(branches), dtype_code(first.dtype),
+                                     _ptr(weight) if out is not None else None, x.data_ptr(), _ptr(out), T, d, float(eps), _stream()),
+          "branches_norm")
+    return out
+
+
 def activation(x, out, kind: str):
     """out = act(x) element by element (relu2: relu(z)^2, gelu_tanh, silu)."""
     _dev(x, out)
@@ -854,11 +877,21 @@ def _sink_args(sink, n_heads: int):
     return int(bool(sink)), None
 
 
+def _slopes_arg(slopes, n_heads: int):
+    """Pointer of a distance bias's slopes (float32 [n_heads], None: no bias)."""
+    if slopes is None:
+        return None
+    _dev(slopes)
+    _need(slopes.dtype == torch.float32 and slopes.is_contiguous() and slopes.numel() == n_heads, "span attention: slopes must be float32 [heads]")
+    return slopes.data_ptr()
+
+
 def attention_span_generic(q, out, gate, kcache, vcache, block_tables, token_req, positions, n_heads, n_kv_heads, key_dim,
                            value_dim, page_size, scale: float, window: int = 0, keep_first: int = 0, sink=False,
-                           softcap: float = 0.0):
+                           softcap: float = 0.0, slopes=None):
     """out[t, h] = sum_j p_j V_j over the keys j <= positions[t] with positions[t] - j < window or j < keep_first
-    (window 0: all), p = softmax of s_j = scale * q . K_j (``softcap`` c > 0: s_j <- c tanh(s_j / c)) with the sink's
+    (window 0: all), p = softmax of s_j = scale * q . K_j (``softcap`` c > 0: s_j <- c tanh(s_j / c); ``slopes``, float32
+    [n_heads]: then s_j <- s_j - slopes[h] (positions[t] - j)) with the sink's
     term added to the denominator (``sink``: see ``_sink_args``); times sigmoid(gate)."""
     sink_flag, sink_ptr = _sink_args(sink, n_heads)
     _span_common(q, out, gate, kcache, vcache, block_tables, n_heads, n_kv_heads, key_dim, value_dim, page_size)
@@ -872,7 +905,7 @@ def attention_span_generic(q, out, gate, kcache, vcache, block_tables, token_req
         gate.stride(0) if gate is not None else 0, dtype_code(q.dtype), kcache.data_ptr(), vcache.data_ptr(),
         block_tables.data_ptr(), block_tables.stride(0), token_req.data_ptr(), positions.data_ptr(), T, n_heads, n_kv_heads,
         key_dim, value_dim, page_size, float(scale), int(window or 0), int(keep_first or 0), sink_flag, sink_ptr,
-        float(softcap or 0.0), _stream()),
+        float(softcap or 0.0), _slopes_arg(slopes, n_heads), _stream()),
         "attention_span_generic")
 
 
@@ -887,7 +920,7 @@ def attention_span_decode_splits(n_rows: int, n_kv_heads: int, max_keys: int, co
 
 def attention_span_decode(q, out, gate, kcache, vcache, block_tables, tok_list, n_tok, token_req, positions, part_acc,
                           part_ml, n_heads, n_kv_heads, key_dim, value_dim, page_size, scale: float, window: int = 0,
-                          keep_first: int = 0, sink=False, softcap: float = 0.0, n_split: int = 1):
+                          keep_first: int = 0, sink=False, softcap: float = 0.0, slopes=None, n_split: int = 1):
     """The rows ``tok_list`` (None: rows 0..n_tok-1) of q, each a request's single new token, split ``n_split`` ways
     over their visible keys.  part_acc / part_ml: float32 scratch of n_tok * heads * n_split * (value_dim / 2) elements."""
     _span_common(q, out, gate, kcache, vcache, block_tables, n_heads, n_kv_heads, key_dim, value_dim, page_size)
@@ -911,8 +944,8 @@ def attention_span_decode(q, out, gate, kcache, vcache, block_tables, tok_list, 
         block_tables.data_ptr(), block_tables.stride(0), tok_list.data_ptr() if tok_list is not None else None,
         token_req.data_ptr(), positions.data_ptr(), part_acc.data_ptr() if n_split > 1 else None,
         part_ml.data_ptr() if n_split > 1 else None, n_tok, n_heads, n_kv_heads, key_dim, value_dim, page_size,
-        float(scale), int(window or 0), int(keep_first or 0), sink_flag, sink_ptr, float(softcap or 0.0), int(n_split),
-        _stream()),
+        float(scale), int(window or 0), int(keep_first or 0), sink_flag, sink_ptr, float(softcap or 0.0), _slopes_arg(slopes, n_heads),
+        int(n_split), _stream()),
         "attention_span_decode")
 
 
@@ -923,7 +956,7 @@ def attention_span_prefill_supported(dtype, key_dim: int, value_dim: int) -> boo
 
 def attention_span_prefill(q, out, gate, kcache, vcache, block_tables, tiles, n_tiles, n_heads, n_kv_heads, key_dim,
                            value_dim, page_size, scale: float, window: int = 0, keep_first: int = 0, sink=False,
-                           softcap: float = 0.0):
+                           softcap: float = 0.0, slopes=None):
     """Prompt portions listed as tiles int32 [n_tiles, 4] (request row, first token row, rows, first position)."""
     sink_flag, sink_ptr = _sink_args(sink, n_heads)
     _span_common(q, out, gate, kcache, vcache, block_tables, n_heads, n_kv_heads, key_dim, value_dim, page_size)
@@ -935,7 +968,7 @@ def attention_span_prefill(q, out, gate, kcache, vcache, block_tables, tiles, n_
         gate.stride(0) if gate is not None else 0, dtype_code(q.dtype), kcache.data_ptr(), vcache.data_ptr(),
         block_tables.data_ptr(), block_tables.stride(0), tiles.data_ptr(), n_tiles, n_heads, n_kv_heads, key_dim, value_dim,
         page_size, float(scale), int(window or 0), int(keep_first or 0), sink_flag, sink_ptr, float(softcap or 0.0),
-        _stream()),
+        _slopes_arg(slopes, n_heads), _stream()),
         "attention_span_prefill")
 
 
@@ -1168,9 +1201,11 @@ def decay_product(a, w, out, bias, rate=None, log_scale=None):
 
 # ---- matrix memories (csrc/matrix_memory.hip) -----------------------------------------------------------------------
 def delta_prep(rows, conv_w, b, out, beta, kv_heads: int, heads: int, key_dim: int, value_dim: int, unit_eps: float, state,
-               state_offset: int, token_req, req_start, state_slots, n_requests: int, single: bool):
+               state_offset: int, token_req, req_start, state_slots, n_requests: int, single: bool, head_decay=None):
     """rows [T, >= q | k | v] through a convolution (state at ``state_offset``) and silu; q and k heads to unit length: float32
-    ``out`` [T, 2 kv_heads key_dim + heads value_dim]; ``beta`` [T, heads] = sigmoid(b).  ``single``: one token a request."""
+    ``out`` [T, 2 kv_heads key_dim + heads value_dim]; ``beta`` [T, heads] = sigmoid(b).  ``single``: one token a request.
+    ``head_decay``: (a [T, heads] in the rows' dtype, rate [heads], bias [heads], decay [T, heads] float32), and then
+    decay = exp(-rate softplus(a + bias))."""
     _dev(rows, conv_w, b, out, beta, state, token_req, req_start, state_slots)
     T = rows.shape[0]
     C = 2 * kv_heads * key_dim + heads * value_dim
@@ -1185,10 +1220,18 @@ def delta_prep(rows, conv_w, b, out, beta, kv_heads: int, heads: int, key_dim: i
     _need(not single or T == n_requests, "delta_prep: one token a request")
     sp, stride = _state_part(state, state_offset)
     _need(state_offset + (taps - 1) * C <= stride, "delta_prep: state too small")
+    a = rate = a_bias = decay = None
+    if head_decay is not None:
+        a, rate, a_bias, decay = head_decay
+        _dev(a, rate, a_bias, decay)
+        _need(tuple(a.shape) == (T, heads) and a.stride(1) == 1 and a.dtype == rows.dtype, "delta_prep: decay rows")
+        for v, shape in ((rate, (heads,)), (a_bias, (heads,)), (decay, (T, heads))):
+            _need(v.dtype == torch.float32 and v.is_contiguous() and tuple(v.shape) == shape, "delta_prep: decay vectors")
     check(get_lib().ic_delta_prep(rows.data_ptr(), rows.stride(0), dtype_code(rows.dtype), conv_w.data_ptr(), taps, b.data_ptr(), b.stride(0),
                                   out.data_ptr(), beta.data_ptr(), int(kv_heads), int(heads), int(key_dim), int(value_dim), float(unit_eps),
                                   sp, stride, token_req.data_ptr(), req_start.data_ptr(), state_slots.data_ptr(), T, n_requests,
-                                  1 if single else 0, _stream()), "delta_prep")
+                                  1 if single else 0, _ptr(a), a.stride(0) if a is not None else 0, _ptr(rate), _ptr(a_bias), _ptr(decay),
+                                  _stream()), "delta_prep")
 
 
 def memory_gates(z, bias_i, bias_f, cap: float, keep, add, floor, state, state_offset: int, req_start, state_slots, n_requests: int):
@@ -1264,35 +1307,43 @@ def gated_head_norm(y, z, weight, heads: int, eps: float, out, gate: str = "sigm
 
 
 # ---- attention through a latent -------------------------------------------------------------------------------------
+def _angles(freq, rot_dims: int, what: str):
+    _need(freq.dtype == torch.float32 and freq.is_contiguous() and freq.numel() >= rot_dims, what + ": angles are float32 [2, rot_dims / 2]")
+
+
 def latent_prep(rows, q_rank: int, kv_rank: int, rot_dim: int, qn_w, kvn_w, eps: float, freq, rot_dims: int, positions,
-                cq, cache, slots):
-    """cq = rms(rows[:, :q_rank]) * qn_w; cache[slots[t]] = [rms(next kv_rank columns) * kvn_w | the next rot_dim rotated]."""
+                cq, cache, slots, rot_mult: float = 1.0):
+    """cq = rms(rows[:, :q_rank]) * qn_w; cache[slots[t]] = [rms(next kv_rank columns) * kvn_w | the next rot_dim rotated and
+    times rot_mult].  ``slots`` None: only cq (the rows may then end behind the query latent and kvn_w be None)."""
     _dev(rows, qn_w, kvn_w, freq, positions, cq, cache, slots)
     T = rows.shape[0]
-    _need(rows.stride(1) == 1 and rows.shape[1] >= q_rank + kv_rank + rot_dim, "latent_prep: rows")
+    _need(rows.stride(1) == 1 and rows.shape[1] >= q_rank + (kv_rank + rot_dim if slots is not None else 0), "latent_prep: rows")
     _need(cq.dtype == rows.dtype and tuple(cq.shape) == (T, q_rank) and cq.is_contiguous(), "latent_prep: cq")
-    for v, n in ((qn_w, q_rank), (kvn_w, kv_rank), (freq, rot_dims // 2)):
-        _need(v.dtype == torch.float32 and v.numel() >= n and v.is_contiguous(), "latent_prep: vectors")
+    for v, n in ((qn_w, q_rank),) + (((kvn_w, kv_rank),) if slots is not None else ()):
+        _need(v is not None and v.dtype == torch.float32 and v.numel() >= n and v.is_contiguous(), "latent_prep: vectors")
+    _angles(freq, rot_dims, "latent_prep")
     _i32(positions, "positions")
     if slots is not None:
         _i32(slots, "slots")
         _need(cache.dtype == rows.dtype and cache.is_contiguous() and cache.shape[-1] == kv_rank + rot_dim and cache.shape[1] == 1,
               "latent_prep: cache plane")
     check(get_lib().ic_latent_prep(rows.data_ptr(), rows.stride(0), dtype_code(rows.dtype), q_rank, kv_rank, rot_dim,
-                                   qn_w.data_ptr(), kvn_w.data_ptr(), float(eps), freq.data_ptr(), int(rot_dims),
+                                   qn_w.data_ptr(), _ptr(kvn_w), float(eps), freq.data_ptr(), int(rot_dims), float(rot_mult),
                                    positions.data_ptr(), cq.data_ptr(), _ptr(cache), _ptr(slots), T, _stream()), "latent_prep")
 
 
-def latent_q_rotate(q, dim: int, rot_dim: int, kv_rank: int, heads: int, freq, rot_dims: int, positions, qa):
-    """qa[t, h, kv_rank:] = the rotated part q[t, h, dim:] turned by its position's angles."""
+def latent_q_rotate(q, dim: int, rot_dim: int, kv_rank: int, heads: int, freq, rot_dims: int, positions, qa, rot_mult: float = 1.0):
+    """qa[t, h, kv_rank:] = the rotated part q[t, h, dim:] turned by its position's angles and times rot_mult.  In place with
+    qa = q and kv_rank = dim."""
     _dev(q, freq, positions, qa)
     T = q.shape[0]
     _need(q.shape[1] == heads * (dim + rot_dim) and q.stride(1) == 1 and qa.dtype == q.dtype
           and tuple(qa.shape) == (T, heads * (kv_rank + rot_dim)) and qa.stride(1) == 1, "latent_q_rotate: layout")
+    _angles(freq, rot_dims, "latent_q_rotate")
     _i32(positions, "positions")
     check(get_lib().ic_latent_q_rotate(q.data_ptr(), q.stride(0), dtype_code(q.dtype), dim, rot_dim, kv_rank, heads,
-                                       freq.data_ptr(), int(rot_dims), positions.data_ptr(), qa.data_ptr(), qa.stride(0), T,
-                                       _stream()), "latent_q_rotate")
+                                       freq.data_ptr(), int(rot_dims), float(rot_mult), positions.data_ptr(), qa.data_ptr(), qa.stride(0),
+                                       T, _stream()), "latent_q_rotate")
 
 
 LATENT_MAX_RANK = 512
@@ -1304,11 +1355,20 @@ def attention_latent_on_matrix_cores(dtype, kv_rank: int, rot_dim: int) -> bool:
     return code is not None and bool(get_lib().ic_attn_latent_on_matrix_cores(code, kv_rank, rot_dim))
 
 
+def _head_sinks(sinks, heads: int, what: str):
+    if sinks is None:
+        return None
+    _dev(sinks)
+    _need(sinks.dtype == torch.float32 and sinks.is_contiguous() and sinks.numel() == heads, what + ": sinks must be float32 [heads]")
+    return sinks.data_ptr()
+
+
 def attention_latent(qa, out, cache, block_tables, token_req, positions, heads: int, kv_rank: int, rot_dim: int,
                      page_size: int, scale: float, n_split: int = 1, part_acc=None, part_ml=None, row_list=None, n_rows=None,
-                     vector_units: bool = False):
-    """out[t, h, :kv_rank] = sum_j p_j c_j over the cached rows [c | k_rot] j <= positions[t] of the token's request,
-    p = softmax(scale * qa[t, h] . row_j): every head walks the same rows.  ``row_list`` (int32, ``n_rows`` of them): the
+                     vector_units: bool = False, window: int = 0, sinks=None):
+    """out[t, h, :kv_rank] = sum_j p_j c_j over the cached rows [c | k_rot] j <= positions[t] of the token's request
+    (``window`` > 0: of the last ``window`` of them), p = softmax(scale * qa[t, h] . row_j): every head walks the same rows.
+    ``sinks`` (float32 [heads]): exp(sinks[h]) joins the denominator.  ``row_list`` (int32, ``n_rows`` of them): the
     rows t to compute; None: all.  bfloat16 with a latent of 64..512 and a rotated part of 16..64 values runs on the
     matrix cores unless ``vector_units`` asks for the general kernel."""
     _dev(qa, out, cache, block_tables, token_req, positions, part_acc, part_ml, row_list)
@@ -1333,33 +1393,66 @@ def attention_latent(qa, out, cache, block_tables, token_req, positions, heads: 
     check(get_lib().ic_attn_latent(qa.data_ptr(), qa.stride(0), out.data_ptr(), out.stride(0), dtype_code(qa.dtype),
                                    cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), token_req.data_ptr(),
                                    positions.data_ptr(), _ptr(row_list), n_launch, heads, kv_rank, rot_dim, page_size,
-                                   float(scale), int(n_split), _ptr(part_acc), _ptr(part_ml), int(bool(vector_units)), _stream()),
+                                   float(scale), int(window or 0), _head_sinks(sinks, heads, "attention_latent"), int(n_split),
+                                   _ptr(part_acc), _ptr(part_ml), int(bool(vector_units)), _stream()),
           "attention_latent")
     return out
 
 
-def latent_gather(cache, table_row, n_keys: int, n_padded: int, page_size: int, kv_rank: int, rows, rows_t):
-    """rows[j] = the cached row of key j of the request whose block-table row is ``table_row`` (zeros from n_keys to
-    n_padded); rows_t[c, j] = rows[j, c] for the first kv_rank columns."""
+def attention_latent_prefill_supported(dtype, dim: int, rot_dim: int, value_dim: int) -> bool:
+    code = _code_or_none(dtype)
+    return code is not None and bool(get_lib().ic_attn_latent_prefill_supported(code, dim, rot_dim, value_dim))
+
+
+def attention_latent_prefill(q, out, gate, kv, rows, kv_rank: int, key0: int, row0: int, n: int, pos0: int, heads: int, dim: int,
+                             rot_dim: int, value_dim: int, scale: float, window: int = 0, sinks=None):
+    """One request's portion, rows row0 .. row0 + n - 1 of q [T, heads (dim + rot_dim)] (rotated), out and gate (nullable)
+    [T, heads value_dim], at positions pos0 and up: softmax attention over keys and values made per head.  ``kv`` [keys, heads dim
+    + heads value_dim] and ``rows`` [keys, kv_rank + rot_dim] (``latent_gather``) hold keys key0 .. pos0 + n - 1."""
+    _dev(q, out, gate, kv, rows)
+    _need(n > 0 and row0 >= 0 and row0 + n <= q.shape[0] and q.shape[1] == heads * (dim + rot_dim) and q.stride(1) == 1, "latent prefill: q")
+    _need(out.shape[0] >= row0 + n and out.shape[1] == heads * value_dim and out.stride(1) == 1, "latent prefill: out")
+    _need(gate is None or (gate.shape[0] >= row0 + n and gate.shape[1] >= heads * value_dim and gate.stride(1) == 1), "latent prefill: gate")
+    keys = pos0 + n - key0
+    _need(kv.shape[0] >= keys and kv.shape[1] == heads * (dim + value_dim) and kv.stride(1) == 1
+          and rows.shape[0] >= keys and rows.shape[1] == kv_rank + rot_dim and rows.stride(1) == 1, "latent prefill: keys and values")
+    for t in (out, gate, kv, rows):
+        _need(t is None or t.dtype == q.dtype, "latent prefill: one dtype")
+    check(get_lib().ic_attn_latent_prefill(q.data_ptr(), q.stride(0), out.data_ptr(), out.stride(0), _ptr(gate), gate.stride(0) if gate is not None else 0,
+                                           dtype_code(q.dtype), kv.data_ptr(), kv.stride(0), heads * dim, rows.data_ptr(), rows.stride(0),
+                                           kv_rank, int(key0), int(row0), int(n), int(pos0), heads, dim, rot_dim, value_dim, float(scale),
+                                           int(window or 0), _head_sinks(sinks, heads, "latent prefill"), _stream()), "attention_latent_prefill")
+    return out
+
+
+def latent_gather(cache, table_row, n_keys: int, n_padded: int, page_size: int, kv_rank: int, rows, rows_t=None, key0: int = 0, first: int = 0):
+    """rows[j] = the cached row of key key0 + j of the request whose block-table row is ``table_row``, zeros for keys before
+    ``first`` (they may have been given back) and from n_keys on, ``n_padded`` rows; rows_t[c, j] = rows[j, c] for the first
+    kv_rank columns (None: left out)."""
     _dev(cache, table_row, rows, rows_t)
     D = cache.shape[-1]
+    first = max(first, key0)
     _need(table_row.dtype == torch.int32 and table_row.stride(-1) == 1 and table_row.numel() * page_size >= n_keys,
           "latent_gather: block table")
     _need(cache.is_contiguous() and cache.shape[1] == 1 and cache.shape[2] == page_size, "latent_gather: cache plane")
-    _need(rows.dtype == cache.dtype and rows_t.dtype == cache.dtype and tuple(rows.shape) == (n_padded, D) and rows.is_contiguous()
-          and tuple(rows_t.shape) == (kv_rank, n_padded) and rows_t.is_contiguous() and n_padded >= n_keys, "latent_gather: outputs")
+    _need(rows.dtype == cache.dtype and tuple(rows.shape) == (n_padded, D) and rows.is_contiguous() and key0 >= 0
+          and n_padded >= n_keys - key0, "latent_gather: outputs")
+    _need(rows_t is None or (rows_t.dtype == cache.dtype and tuple(rows_t.shape) == (kv_rank, n_padded) and rows_t.is_contiguous()),
+          "latent_gather: transposed output")
     check(get_lib().ic_latent_gather(cache.data_ptr(), dtype_code(cache.dtype), table_row.data_ptr(), page_size, D, kv_rank,
-                                     int(n_keys), int(n_padded), rows.data_ptr(), rows_t.data_ptr(), _stream()), "latent_gather")
+                                     int(key0), int(first), int(n_keys), int(n_padded), rows.data_ptr(), _ptr(rows_t), _stream()), "latent_gather")
 
 
-def latent_softmax(scores, probs, heads: int, first_limit: int, scale: float):
-    """probs[m] = softmax(scale * scores[m, :n]) with n = first_limit + m // heads + 1 visible keys, zeros beyond."""
+def latent_softmax(scores, probs, heads: int, first_limit: int, scale: float, window: int = 0, sinks=None, key0: int = 0):
+    """Column j is key key0 + j.  probs[m] = softmax(scale * scores[m]) over the keys that position first_limit + m // heads sees
+    (the last ``window`` of them when > 0), with head m % heads' sink in the denominator, zeros elsewhere."""
     _dev(scores, probs)
     M, n_cols = scores.shape
     _need(scores.dtype == torch.float32 and scores.stride(1) == 1 and tuple(probs.shape) == (M, n_cols) and probs.stride(1) == 1,
           "latent_softmax: layout")
     check(get_lib().ic_latent_softmax(scores.data_ptr(), scores.stride(0), probs.data_ptr(), probs.stride(0), dtype_code(probs.dtype),
-                                      M, heads, n_cols, int(first_limit), float(scale), _stream()), "latent_softmax")
+                                      M, heads, n_cols, int(key0), int(first_limit), float(scale), int(window or 0),
+                                      _head_sinks(sinks, heads, "latent_softmax"), _stream()), "latent_softmax")
     return probs
 
 

@@ -307,6 +307,9 @@ class Block(Part):
     # the norm a block applies to the incoming stream when it takes DeferredRows as ``pending``.
     fuses_successor = False
 
+    # Kinds of owed update (objects with ``settle(x, ctx)``) that the block takes as ``pending``; others are settled first.
+    accepts_owed_update = ()
+
     def entry_norm(self):
         return None
 

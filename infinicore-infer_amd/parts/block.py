@@ -191,7 +191,7 @@ class HyperConnectionBlock(Block):
     ``hc<q>.mix`` [S, S] ([from, to]), held in float32.  One row kernel per sublayer does the write owed by the
     sublayer before, the read, and the norm."""
     graph_safe = True
-    accepts_owed_update = True
+    accepts_owed_update = (OwedStreamWrite,)
 
     def __init__(self, name, runtime, mixer=None, mixer_norm=None, feed_forward=None, feed_forward_norm=None, streams: int = 2):
         super().__init__(name, runtime, mixer, mixer_norm, feed_forward, feed_forward_norm)
@@ -254,6 +254,49 @@ class HyperConnectionBlock(Block):
             y = self.feed_forward.forward(h, ctx)
             pending = OwedStreamWrite(y, self.hc[2][2], self.hc[2][1])
         return pending
+
+
+class OwedBranches:
+    """Results that are still to be added to the residual stream, as (tensor, factor) pairs: the next block of the same kind
+    adds them in the kernel that forms its norm.  Whoever cannot, settles it."""
+
+    def __init__(self, parts):
+        self.parts = tuple(parts)
+
+    def settle(self, x, ctx=None):
+        ops.branches_norm(self.parts, None, x, 0.0)
+        return None
+
+
+@register_part("block", "shared_norm_residual")
+class SharedNormResidualBlock(Block):
+    """h = norm(x); x += mixer(h) + ff(h): one norm, whose output both sublayers read (the second term only when the layer has a
+    feed-forward).  The stream is float32; both results (and the branches of a mixer that yields them) stay owed, and one row
+    kernel of the next block adds them all and forms its norm."""
+    graph_safe = True
+    accepts_owed_update = (OwedBranches,)
+
+    def __init__(self, name, runtime, mixer=None, mixer_norm=None, feed_forward=None, feed_forward_norm=None):
+        super().__init__(name, runtime, mixer, mixer_norm, feed_forward, feed_forward_norm)
+        if mixer is None or mixer_norm is None or feed_forward_norm is not None:
+            raise ValueError("block %s: a block of one norm needs a mixer and that norm, as the mixer's" % name)
+        if mixer_norm.deferred() is None:
+            raise ValueError("block %s: norm part %s is not a weighted RMS norm" % (name, type(mixer_norm).__name__))
+
+    def forward(self, x, pending, ctx, cache):
+        h = ctx.ws.buffer("normed", tuple(x.shape), self.runtime.dtype)
+        weight, eps = self.mixer_norm.deferred()
+        if isinstance(pending, OwedBranches):
+            ops.branches_norm(pending.parts, weight, x, eps, out=h)
+        elif pending is None or isinstance(pending, StreamCopy):
+            self.mixer_norm.forward(x, h)
+        else:
+            self.mixer_norm.forward_add(x, pending[0], pending[1], h)
+        y = self.mixer.forward(h, ctx, cache, branches=True) if self.mixer.yields_branches else self.mixer.forward(h, ctx, cache)
+        owed = y.parts if isinstance(y, Branches) else ((y, 1.0),)
+        if self.feed_forward is not None:
+            owed += ((self.feed_forward.forward(h, ctx), 1.0),)
+        return OwedBranches(owed)
 
 
 @register_part("block", "sandwich_gated")

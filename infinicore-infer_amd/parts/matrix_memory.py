@@ -1,9 +1,10 @@
 """Mixers whose state is a matrix S [key size, value size] per head that keys and values write and queries read, in float32.
 
-``gated_delta``: the delta rule with a decay per head and key channel.  q, k (``kv_heads`` heads), v pass a causal convolution
+``gated_delta``: the delta rule with a decay per head and key channel (or per head alone).  q, k (``kv_heads`` heads), v pass a causal convolution
     per channel and silu; q and k heads are brought to unit length, q is multiplied by key_dim^(-1/2);
     g = exp(-exp(A_log) softplus(W_a2 W_a1 h + dt_bias)), beta = sigmoid(W_b h);
     S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q;   out = W_o (rms(o) * w * sigmoid(W_g2 W_g1 h)).
+    ``decay="head"``: one decay per head, g = exp(-exp(A_log) softplus(W_a h + dt_bias)), and a dense gate, silu(W_g h).
 ``gated_linear_attention``: g = sigmoid(W_a2 W_a1 h + a2.b)^(1/tau) per head and key channel, no delta rule and no convolution:
     S <- g S + k v^T,  o = S^T q with q = W_q h key_dim^(-1/2);   out = W_o (rms(o) * w * silu(W_g h)).
 ``exponential_memory``: one decay per head from exponential gates.  i = cap tanh((W_i h + i.b) / cap), f = logsigmoid(cap
@@ -73,11 +74,15 @@ class _MatrixMemory(Mixer):
 @register_part("mixer", "gated_delta")
 class GatedDeltaRule(_MatrixMemory):
     def __init__(self, name, runtime, hidden_size: int, heads: int, kv_heads: int, key_dim: int, value_dim: int, conv_taps: int,
-                 norm_eps: float):
+                 norm_eps: float, decay: str = "channel"):
+        """``decay``: "channel" (low-rank decay and gate projections, a sigmoid gate) or "head" (dense ones, a silu gate)."""
         super().__init__(name, runtime)
         _check_sizes("gated delta rule", heads, kv_heads, key_dim, value_dim)
         if not 1 <= conv_taps <= 8:
             raise ValueError("gated delta rule: 1..8 convolution taps (got %d)" % conv_taps)
+        if decay not in ("channel", "head"):
+            raise ValueError("gated delta rule: the decay is per channel or per head (got %r)" % (decay,))
+        self.per_head = decay == "head"
         self.hidden_size, self.heads, self.kvh = int(hidden_size), int(heads), int(kv_heads)
         self.dk, self.dv, self.taps, self.eps = int(key_dim), int(value_dim), int(conv_taps), float(norm_eps)
         self.nq, self.nv = self.kvh * self.dk, self.heads * self.dv
@@ -86,53 +91,70 @@ class GatedDeltaRule(_MatrixMemory):
         self.state_size = self.conv_offset + (self.taps - 1) * self.channels
         self.ranks = (FreeDim(name + "a.rank", self.dk), FreeDim(name + "g.rank", self.dv))
 
+    def _row_names(self):
+        """What reads h, in the order of the packed projection's rows."""
+        return ("q", "k", "v") + (("g", "b", "a") if self.per_head else ("a1", "g1", "b"))
+
     def weight_specs(self):
         n, d, (ra, rg) = self.name, self.hidden_size, self.ranks
-        pack, cpack = n + "rows.packed", n + "conv.packed"
+        cpack = n + "conv.packed"
         conv = lambda c, i: WeightSpec((c, self.taps), "vector", pack=(cpack, i), mean=1.0 / self.taps)
-        return {
-            n + "q": WeightSpec((self.nq, d), pack=(pack, 0)), n + "k": WeightSpec((self.nq, d), pack=(pack, 1)),
-            n + "v": WeightSpec((self.nv, d), pack=(pack, 2)), n + "a1": WeightSpec((ra, d), pack=(pack, 3)),
-            n + "g1": WeightSpec((rg, d), pack=(pack, 4)), n + "b": WeightSpec((self.heads, d), pack=(pack, 5)),
+        rows = {"q": self.nq, "k": self.nq, "v": self.nv, "b": self.heads, "a1": ra, "g1": rg, "g": self.nv, "a": self.heads}
+        n_decays = self.heads if self.per_head else self.heads * self.dk
+        specs = {n + x: WeightSpec((rows[x], d), pack=(n + "rows.packed", i)) for i, x in enumerate(self._row_names())}
+        specs.update({
             n + "q.conv": conv(self.nq, 0), n + "k.conv": conv(self.nq, 1), n + "v.conv": conv(self.nv, 2),
-            n + "A_log": WeightSpec((self.heads,), "vector", mean=0.0),
-            n + "a2": WeightSpec((self.heads * self.dk, ra)), n + "dt_bias": WeightSpec((self.heads * self.dk,), "vector", mean=0.0),
-            n + "g2": WeightSpec((self.nv, rg)),
+            n + "A_log": WeightSpec((self.heads,), "vector", mean=0.0), n + "dt_bias": WeightSpec((n_decays,), "vector", mean=0.0),
             n + "norm": WeightSpec((self.dv,), "vector"), n + "o": WeightSpec((d, self.nv)),
-        }
+        })
+        if not self.per_head:
+            specs[n + "a2"], specs[n + "g2"] = WeightSpec((self.heads * self.dk, ra)), WeightSpec((self.nv, rg))
+        return specs
 
     def load_weights(self, tensors):
         n, dt = self.name, self.runtime.dtype
-        self.w_rows = packed_rows(tensors, n + "rows.packed", [n + s for s in ("q", "k", "v", "a1", "g1", "b")])
+        self.w_rows = packed_rows(tensors, n + "rows.packed", [n + s for s in self._row_names()])
         self.conv_w = packed_rows(tensors, n + "conv.packed", [n + s + ".conv" for s in ("q", "k", "v")])
-        self.ra, self.rg = tensors[n + "a2"].shape[1], tensors[n + "g2"].shape[1]
-        self.w_a2, self.w_g2 = tensors[n + "a2"].to(dt).contiguous(), tensors[n + "g2"].to(dt).contiguous()
+        if not self.per_head:
+            self.ra, self.rg = tensors[n + "a2"].shape[1], tensors[n + "g2"].shape[1]
+            self.w_a2, self.w_g2 = tensors[n + "a2"].to(dt).contiguous(), tensors[n + "g2"].to(dt).contiguous()
         self.rate = torch.exp(tensors[n + "A_log"].to(torch.float64)).to(torch.float32).contiguous()
         self.dt_bias, self.norm_w, self.w_o = tensors[n + "dt_bias"], tensors[n + "norm"], tensors[n + "o"]
+
+    def _channel_parts(self, rows, ctx):
+        """(the step sizes' rows, the decay factors, the gate's rows) from the low-rank rows."""
+        rt, T, c = self.runtime, rows.shape[0], self.channels
+        a1, g1 = rows[:, c:c + self.ra], rows[:, c + self.ra:c + self.ra + self.rg]
+        decay = self._decay(a1, self.w_a2, self.dt_bias, ctx, rate=self.rate)
+        gate = ctx.ws.buffer("memory_gate", (T, self.nv), rt.dtype)
+        if self._by_library(g1):
+            linear(g1, self.w_g2, gate, rt.gemm_impl, ws=ctx.ws)
+        else:
+            ops.blocked_product(g1.unsqueeze(1), self.w_g2.unsqueeze(0), gate.unsqueeze(1))
+        return rows[:, c + self.ra + self.rg:], decay, gate
 
     def forward(self, h, ctx, cache):
         rt, T, c = self.runtime, h.shape[0], self.channels
         buf = ctx.ws.buffer
         rows = self._project(h, ctx)
-        a1, g1 = rows[:, c:c + self.ra], rows[:, c + self.ra:c + self.ra + self.rg]
-        b = rows[:, c + self.ra + self.rg:]
-        decay = self._decay(a1, self.w_a2, self.dt_bias, ctx, rate=self.rate)
-        gate = buf("memory_gate", (T, self.nv), rt.dtype)
-        if self._by_library(g1):
-            linear(g1, self.w_g2, gate, rt.gemm_impl, ws=ctx.ws)
+        head_decay = None
+        if self.per_head:
+            gate, b, a = rows[:, c:c + self.nv], rows[:, c + self.nv:c + self.nv + self.heads], rows[:, c + self.nv + self.heads:]
+            decay = buf("memory_decay", (T, self.heads), torch.float32)
+            head_decay = (a, self.rate, self.dt_bias, decay)             # formed beside the step sizes
         else:
-            ops.blocked_product(g1.unsqueeze(1), self.w_g2.unsqueeze(0), gate.unsqueeze(1))
+            b, decay, gate = self._channel_parts(rows, ctx)
         qkv, beta = buf("memory_qkv", (T, c), torch.float32), buf("memory_beta", (T, self.heads), torch.float32)
         single = ctx.T == ctx.R
         lists = (ctx.req_rows, ctx.state_slots, ctx.R)
         ops.delta_prep(rows[:, :c], self.conv_w, b, qkv, beta, self.kvh, self.heads, self.dk, self.dv, UNIT_EPS, cache.state,
-                       self.state_base + self.conv_offset, ctx.token_req, *lists, single=single)
+                       self.state_base + self.conv_offset, ctx.token_req, *lists, single=single, head_decay=head_decay)
         o = buf("memory_o", (T, self.nv), torch.float32)
         ops.matrix_memory(qkv[:, :self.nq], qkv[:, self.nq:2 * self.nq], qkv[:, 2 * self.nq:], decay, self.heads, self.kvh, self.dk, self.dv,
                           o, cache.state, self.state_base, *lists, single=single, scale=beta, delta=True, q_scale=self.dk ** -0.5,
                           compute_units=ctx.cu_count)
         g = buf("memory_gated", (T, self.nv), rt.dtype)
-        ops.gated_head_norm(o, gate, self.norm_w, self.heads, self.eps, g)
+        ops.gated_head_norm(o, gate, self.norm_w, self.heads, self.eps, g, gate="silu" if self.per_head else "sigmoid")
         return self._result(g, ctx)
 
 

@@ -6,6 +6,7 @@ reference's): gather embeddings into the float32 residual stream, run the
 schedule, settle the last residual add, then normalise and project only the
 rows whose logits are wanted.
 """
+from dataclasses import replace
 from typing import Dict, List
 
 import torch
@@ -57,9 +58,8 @@ class DecoderModel:
             for l in self.layers:
                 if getattr(l, "streams", 1) != self.streams:
                     raise ValueError("block %s keeps %d residual streams, the model %d" % (l.name, getattr(l, "streams", 1), self.streams))
-        # an entry that reads another entry's cache must fit what the writer keeps: the same heads and
-        # head size, and no more keys than the writer's window holds (pages behind a window are given
-        # back and their block-table entries are reused)
+        # an entry that reads another entry's cache must fit what the writer keeps: the same heads and head size (how many keys
+        # the slot keeps is the widest window of all its entries, see cache_needs)
         for e in self.schedule:
             if e.writes_cache:
                 continue
@@ -71,9 +71,6 @@ class DecoderModel:
                 raise ValueError("layer %d reads cache slot %d as %d planes with %d kv heads of %d, its writer (layer %d) "
                                  "keeps %d planes with %d of %d" % (e.layer, e.cache, rn.planes, rn.n_kv_heads, rn.head_dim,
                                                                     writers[e.cache], wn.planes, wn.n_kv_heads, wn.head_dim))
-            if wn.window and (not rn.window or rn.window > wn.window):
-                raise ValueError("layer %d reads cache slot %d over %s keys, its writer (layer %d) keeps a window of %d"
-                                 % (e.layer, e.cache, rn.window or "all", writers[e.cache], wn.window))
 
     # ---- parts and weights ---------------------------------------------------------
     def all_parts(self):
@@ -116,11 +113,20 @@ class DecoderModel:
         return CacheNeed() if mixer is None else mixer.cache_need()       # a layer without a mixer keeps nothing
 
     def cache_needs(self) -> List[CacheNeed]:
-        """One need per cache slot, in slot order."""
+        """One need per cache slot, in slot order: what the entry that writes the slot keeps, for as long as any entry that
+        reads it wants (a window group gives pages back once the widest window has passed)."""
         n = self.spec.num_cache_slots()
         needs = [CacheNeed() for _ in range(n)]
         for slot, layer in self._writers.items():
             needs[slot] = self._cache_need_of(layer)
+        for e in self.schedule:
+            need, want = needs[e.cache], self._cache_need_of(e.layer)
+            if e.writes_cache or not (need.paged and want.paged) or not need.window:
+                continue
+            if not want.window:
+                needs[e.cache] = replace(need, window=None, keep_first=0)
+            else:
+                needs[e.cache] = replace(need, window=max(need.window, want.window), keep_first=max(need.keep_first, want.keep_first))
         return needs
 
     def embedding_cache_need(self) -> CacheNeed:
@@ -165,7 +171,7 @@ class DecoderModel:
                     ops.residual_add(x, pending[0], pending[1])
                 pending = None
                 ops.residual_add(x, embedded, 1.0)
-            if hasattr(pending, "settle") and not getattr(block, "accepts_owed_update", False):
+            if hasattr(pending, "settle") and not isinstance(pending, getattr(block, "accepts_owed_update", ())):
                 pending = pending.settle(x, ctx)                      # an update only its own kind of block can fuse
             if isinstance(pending, StreamCopy) and not getattr(block, "accepts_stream_copy", False):
                 pending = None                                        # nothing is owed; this block makes its own input

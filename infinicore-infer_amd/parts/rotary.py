@@ -45,13 +45,27 @@ def rotary_tables(head_dim, theta, max_positions, scaling=None, rot_dim=None, mo
     return (torch.cos(ang) * magnitude).to(torch.float32), (torch.sin(ang) * magnitude).to(torch.float32)
 
 
-def pair_frequencies(rot_dims: int, base: float) -> torch.Tensor:
+def pair_frequencies(rot_dims: int, base: float, scaling=None) -> torch.Tensor:
     """f_i = base^(-2i/rot_dims), i < rot_dims / 2, as float32 [2, rot_dims / 2]: the float64 value rounded, and what the
-    rounding left (the kernel forms the angle from both, so that its error does not grow with the position)."""
+    rounding left (the kernel forms the angle from both, so that its error does not grow with the position).
+
+    ``scaling`` {factor, original, fast, slow}: wavelengths are stretched by ``factor`` where a pair makes fewer than ``slow`` turns
+    over ``original`` positions, kept where it makes more than ``fast``, with a ramp over the pair index between the two."""
     i = torch.arange(rot_dims // 2, dtype=torch.float64)
     f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / rot_dims)
-    hi = f.to(torch.float32)
-    return torch.stack([hi, (f - hi.double()).to(torch.float32)]).contiguous()
+    if scaling:
+        pair_of = lambda turns: rot_dims * math.log(scaling["original"] / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+        lo = max(math.floor(pair_of(scaling["fast"])), 0)
+        hi = min(math.ceil(pair_of(scaling["slow"])), rot_dims - 1)
+        ramp = torch.clamp((i - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+        f = f / float(scaling["factor"]) * ramp + f * (1.0 - ramp)
+    hi32 = f.to(torch.float32)
+    return torch.stack([hi32, (f - hi32.double()).to(torch.float32)]).contiguous()
+
+
+def stretched_magnitude(scaling=None) -> float:
+    """The factor on cos and sin that goes with stretched wavelengths: 0.1 ln(factor) + 1."""
+    return 0.1 * math.log(float(scaling["factor"])) + 1.0 if scaling else 1.0
 
 
 _TABLES = {}

@@ -9,7 +9,9 @@ a rotation.  Options, each a parameter:
   * a norm on queries and keys to unit root mean square, per head (one weight of the key size, shared by the
     heads, or no weight at all) or over the whole projection before it is cut into heads (a weight of the
     projection's size),
+  * values that are the keys as projected, before their norm (no tensor ``v``),
   * a cap on the scaled score, s <- c tanh(s / c),
+  * a distance bias: slope_h (i - j) is taken off the (capped) score, one slope per head,
   * a sink: one more term in the softmax's denominator that has no value, p_j = e^{s_j} / (e^{z} + sum e^{s_j}),
     with z = 0 or z a learned number per head (the tensor ``sink``), neither scaled nor capped,
   * value mixing: the first mixing layer of the model keeps its values of the step's tokens, every later one
@@ -43,13 +45,15 @@ class SpanAttention(Mixer):
                  value_dim: int, softmax_scale: float, window=None, keep_first: int = 0, sink: bool = False,
                  qk_norm=None, qk_norm_eps: float = 1e-6, qkv_bias: bool = False, out_bias: bool = False,
                  gate: bool = False, value_mix=None, value_mix_width=None, value_mix_optional: bool = False,
-                 softcap=None, qk_norm_weight: bool = True, conv_taps: int = 0, rot_dims: int = 0, rot_base=None):
+                 softcap=None, qk_norm_weight: bool = True, conv_taps: int = 0, rot_dims: int = 0, rot_base=None,
+                 values_from_keys: bool = False, distance_slopes=None):
         """``sink``: False, True (the constant term exp(0)) or "learned" (one number per head, the tensor ``sink``).
         ``softcap``: None or the cap c > 0.  ``qk_norm_weight`` False: the per-head norm has no weight tensors.
         ``qk_norm``: None, "head" or "row".  ``value_mix``: None, "keep" (this layer's values are the ones later
         layers mix in) or "mix"; all mixing layers of a model have the same kv heads and value size.
         ``value_mix_optional``: the files may hold the mixing scalar although this layer does not mix.
-        ``conv_taps``: 0 (no convolution) or its taps; ``rot_dims`` / ``rot_base``: the rotation, 0 for none."""
+        ``conv_taps``: 0 (no convolution) or its taps; ``rot_dims`` / ``rot_base``: the rotation, 0 for none.
+        ``values_from_keys``: no value projection.  ``distance_slopes``: None or one number per head."""
         super().__init__(name, runtime)
         if num_heads <= 0 or num_kv_heads <= 0 or num_heads % num_kv_heads:
             raise ValueError("span attention: %d heads are not a multiple of %d kv heads" % (num_heads, num_kv_heads))
@@ -92,6 +96,14 @@ class SpanAttention(Mixer):
             raise ValueError("span attention: a convolution or a rotation goes with no norm or the norm per head, without biases and value mixing")
         self.freq = pair_frequencies(self.rot_dims, rot_base).to(runtime.device) if self.rot_dims else None
         self.conv_w = None
+        self.tied_values = bool(values_from_keys)
+        if self.tied_values and (key_dim != value_dim or self.shaped or self.mix_mode):
+            raise ValueError("span attention: values that are keys have their size and go without a convolution, a rotation and value mixing")
+        self.slopes = None
+        if distance_slopes is not None:
+            if len(distance_slopes) != num_heads:
+                raise ValueError("span attention: %d heads but %d distance slopes" % (num_heads, len(distance_slopes)))
+            self.slopes = torch.tensor([float(a) for a in distance_slopes], dtype=torch.float64).to(torch.float32).to(runtime.device)
         self.nq, self.nk, self.nv = self.nh * self.dk, self.nkvh * self.dk, self.nkvh * self.dv
         self.state_size = max(0, self.taps - 1) * (self.nq + self.nk + self.nv)      # the convolution's last inputs
         self.na = self.nh * self.dv                       # width of the concatenated heads
@@ -111,15 +123,17 @@ class SpanAttention(Mixer):
         specs = {
             n + "q": WeightSpec((self.nq, d), pack=(pack, 0)),
             n + "k": WeightSpec((self.nk, d), pack=(pack, 1)),
-            n + "v": WeightSpec((self.nv, d), pack=(pack, 2)),
             n + "o": WeightSpec((d, self.na)),
         }
+        if not self.tied_values:
+            specs[n + "v"] = WeightSpec((self.nv, d), pack=(pack, 2))
         if self.gate:
             specs[n + "g"] = WeightSpec((self.na, d), pack=(pack, 3))
         if self.qkv_bias:
             specs[n + "q.b"] = WeightSpec((self.nq,), "vector", pack=(bpack, 0), mean=0.0)
             specs[n + "k.b"] = WeightSpec((self.nk,), "vector", pack=(bpack, 1), mean=0.0)
-            specs[n + "v.b"] = WeightSpec((self.nv,), "vector", pack=(bpack, 2), mean=0.0)
+            if not self.tied_values:
+                specs[n + "v.b"] = WeightSpec((self.nv,), "vector", pack=(bpack, 2), mean=0.0)
         if self.out_bias:
             specs[n + "o.b"] = WeightSpec((d,), "vector", mean=0.0)
         for i, c in enumerate((self.nq, self.nk, self.nv) if self.taps else ()):
@@ -137,7 +151,8 @@ class SpanAttention(Mixer):
 
     def load_weights(self, tensors):
         n = self.name
-        names = ["q", "k", "v"] + (["g"] if self.gate else [])
+        qkv = ["q", "k"] + ([] if self.tied_values else ["v"])
+        names = qkv + (["g"] if self.gate else [])
         packed = tensors.get(n + "qkvg.packed")
         if packed is None:
             mats = [tensors[n + s] for s in names]
@@ -149,7 +164,7 @@ class SpanAttention(Mixer):
         if self.qkv_bias:
             b = tensors.get(n + "qkv_bias.packed")
             if b is None:
-                b = torch.cat([tensors[n + s + ".b"].to(torch.float32).reshape(-1) for s in ("q", "k", "v")]).contiguous()
+                b = torch.cat([tensors[n + s + ".b"].to(torch.float32).reshape(-1) for s in qkv]).contiguous()
             self.b_rows = b
         if self.taps:
             self.conv_w = packed_rows(tensors, n + "qkv_conv.packed", [n + s + ".conv" for s in ("q", "k", "v")])
@@ -181,7 +196,7 @@ class SpanAttention(Mixer):
         else:
             self._norm_and_store(rows, q, v_keep, ctx, cache, slots)
         out = ctx.ws.buffer("span_out", (T, self.na), rt.dtype)
-        gate = rows[:, self.nq + self.nk + self.nv:] if self.gate else None
+        gate = rows[:, rows.shape[1] - self.na:] if self.gate else None
         self._attend(q, out, gate, ctx, cache)
         y = ctx.ws.buffer(self.out_buffer, (T, self.hidden_size), rt.dtype)
         linear(out, self.w_o, y, rt.gemm_impl, ws=ctx.ws)
@@ -191,14 +206,15 @@ class SpanAttention(Mixer):
 
     def _norm_and_store(self, rows, q, v_keep, ctx, cache, slots):
         ops.qk_norm_store(rows, self.b_rows, self.q_norm, self.k_norm, self.norm_mode, self.qk_norm_eps, self.mix_mode,
-                          self.mix_lambda, v_keep, q, cache.k, cache.v, slots, self.nh, self.nkvh, self.dk, self.dv, ctx.page_size)
+                          self.mix_lambda, v_keep, q, cache.k, cache.v, slots, self.nh, self.nkvh, self.dk, self.dv, ctx.page_size,
+                          values_from_keys=self.tied_values)
 
     def _attend(self, q, out, gate, ctx, cache):
         """Single-token rows go to the split-key kernel, prompt portions to the matrix-core kernel, where the sizes
         have one (and the runtime does not ask for the general kernel alone); everything else to the general kernel."""
         rt = self.runtime
         args = (self.nh, self.nkvh, self.dk, self.dv, ctx.page_size, self.scale, self.window, self.keep_first,
-                self.sinks if self.sink_learned else self.sink, self.softcap)
+                self.sinks if self.sink_learned else self.sink, self.softcap, self.slopes)
         n_dec, n_tiles = ctx.n_decode_rows, ctx.n_prefill_tiles
         tiled = rt.attention_impl == "auto" and n_dec + n_tiles > 0
         use_dec = tiled and n_dec > 0 and ops.attention_span_decode_supported(rt.dtype, self.dk, self.dv)

@@ -12,7 +12,7 @@ seeded uniform-random token ids.  One JSON line is printed.
   --workload mixed   the 1B shape's workload: 64 requests, prompts of 128..2,048 tokens, portions of 512
   --workload long    the 8B shape's workload: 4 prompts of 16,384 tokens, then decoding
   --direct           decode by calling the step function directly, without the scheduler
-  --workload designs the Fopezen, Mezinex, Daborax, Fizelix and Pekarax decoders beside the MiniCPM decoder at equal layer sizes
+  --workload designs the Fopezen, Mezinex, Daborax, Fizelix, Pekarax and Fokinex decoders beside the MiniCPM decoder at equal layer sizes
                      (a few layers of three real models' sizes): prefill and decode throughput of each, with the fraction
                      of the memory or matrix-core peak it reaches (--only <design>: one of them, for a profiler)
 """
@@ -255,7 +255,21 @@ def _design_configs(z, layers):
     pek_kinds = [("channel_delta", dl), ("gla", gla), ("parallel", par), ("channel_delta", dl)]
     pek = dict(architecture="Pekarax", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-5), postln_alpha=2.0,
                layers=[dict(type=pek_kinds[i % 4][0], mixer=pek_kinds[i % 4][1], mlp=pek_moe) for i in range(layers)])
-    return {"minicpm": mini, "fopezen": fop, "mezinex": mez, "daborax": dab, "fizelix": fiz, "pekarax": pek}
+    # Fokinex at the same width and feed-forward: attention through a latent of the Mezinex row's sizes over the Fopezen row's window
+    # (the third layer reads the first one's rows), and in the second layer attention with the row's heads, kv heads, key size
+    # and window beside the delta rule in as many heads of the row's size, four of them sharing a query and a key
+    fok_lat = dict(latent, mask=dict(size=z["window"]),
+                   rot=dict(latent["rot"], scaling=dict(factor=16.0, original=1024, fast=32.0, slow=1.0)))
+    fok_par = dict(left=dict(heads=z["heads"], kv_heads=z["kv"], dim=z["dim"], vdim=z["dim"], scale=z["dim"] ** -0.5, softcap=50.0,
+                             mask=dict(size=z["window"])),
+                   right=dict(heads=z["heads"], kv_heads=z["heads"] // 4, dim=z["dim"], vdim=z["dim"], conv=4), left_scale=0.7, right_scale=0.7)
+    fok_kinds = [("latent_attention", fok_lat), ("parallel", fok_par), ("latent_attention", fok_lat), ("latent_attention", fok_lat)]
+    fok_layers = []
+    for i in range(layers):
+        kind, m = fok_kinds[i % 4]
+        fok_layers.append(dict(type=kind, mixer=dict(m, kv_from=i - 2) if i % 4 == 2 else m, mlp=dict(kind="dense", ff=z["ff"])))
+    fok = dict(architecture="Fokinex", vocab=z["vocab"], width=z["width"], norm=dict(eps=1e-5), embedding=dict(scale=1.0), layers=fok_layers)
+    return {"minicpm": mini, "fopezen": fop, "mezinex": mez, "daborax": dab, "fizelix": fiz, "pekarax": pek, "fokinex": fok}
 
 
 def _design_numbers(design, z, layers, kinds=None):
@@ -270,6 +284,8 @@ def _design_numbers(design, z, layers, kinds=None):
         return _fizelix_numbers(z, layers)
     if design == "pekarax":
         return _pekarax_numbers(z, layers)
+    if design == "fokinex":
+        return _fokinex_numbers(z, layers)
     if design == "minicpm":
         per_layer = (H + 2 * G) * dk * d + H * dk * d + 3 * d * ff
         kv = lambda n: 2 * layers * G * dk * eb * n
@@ -433,6 +449,36 @@ def _pekarax_numbers(z, layers):
     return weights, kv, flops
 
 
+def _fokinex_numbers(z, layers):
+    """As ``_design_numbers`` for the Fokinex configuration of ``_design_configs``.  A layer that reads another's latent rows reads
+    them again.  The flops of a prompt count attention over keys and values made per head, and what making them costs."""
+    cfg = _design_configs(z, layers)["fokinex"]
+    d, ff, V, eb = z["width"], z["ff"], z["vocab"], _elem_bytes()
+    weights, per_tok_lin, scan, state_bytes = V * d, 0.0, 0.0, 0.0
+    spans = []         # (heads * (key + value size), elements cached per token, window) per attention
+    for l in cfg["layers"]:
+        m = l["mixer"]
+        n = 3 * d * ff
+        if l["type"] == "latent_attention":
+            H, R, E = m["heads"], m["kv_rank"], m["rot_dim"]
+            n += (m["q_rank"] + (0 if "kv_from" in m else R + E) + H * m["vdim"]) * d + H * (m["dim"] + E) * m["q_rank"] + H * (m["dim"] + m["vdim"]) * R
+            spans.append((H * (m["dim"] + E + m["vdim"]), R + E, m["mask"]["size"]))
+        else:
+            a, b = m["left"], m["right"]
+            H, G, dk = a["heads"], a["kv_heads"], a["dim"]
+            n += (H * dk + G * dk + H * dk) * d + d * H * dk
+            spans.append((2 * H * dk, 2 * G * dk, a["mask"]["size"]))
+            H, G, dk, dv = b["heads"], b["kv_heads"], b["dim"], b["vdim"]
+            n += (2 * G * dk + 2 * H * dv + 2 * H) * d + d * H * dv
+            state_bytes += 2 * 4 * (H * dk * dv + (b["conv"] - 1) * (2 * G * dk + H * dv))
+            scan += 8.0 * H * dk * dv
+        weights += n
+        per_tok_lin += 2.0 * n
+    kv = lambda n: sum(c * eb * min(n, w) for _, c, w in spans) + state_bytes
+    flops = lambda T: T * (per_tok_lin + scan) + sum(2.0 * h * sum(min(i + 1, w) for i in range(T)) for h, _, w in spans) + 2.0 * V * d
+    return eb * weights, kv, flops
+
+
 def run_designs(args):
     """Prefill and decode of the two decoders at equal layer sizes.  Decoding calls the step function directly (recorded
     steps), greedy sampling on the device; a row gives tokens/s and what fraction of the memory bandwidth (decoding:
@@ -568,7 +614,7 @@ def main():
     ap.add_argument("--layers", type=int, default=0, help="fewer layers than the shape has (0: all)")
     ap.add_argument("--shape", default=None, choices=sorted(SHAPES), help="2b is the benchmark's configuration (default; 1b for --workload mixed)")
     ap.add_argument("--sizes", default=None, help="--workload designs: comma-separated sizes (default: all of 2b-like, 8b-like, 1b-like)")
-    ap.add_argument("--only", default=None, choices=["fopezen", "minicpm", "mezinex", "daborax", "fizelix", "pekarax"], help="--workload designs: one design only")
+    ap.add_argument("--only", default=None, choices=["fopezen", "minicpm", "mezinex", "daborax", "fizelix", "pekarax", "fokinex"], help="--workload designs: one design only")
     ap.add_argument("--workload", default="decode", choices=["decode", "mixed", "long", "designs"],
                     help="decode: the benchmark (prefill of one prompt, decode steps at fixed batches); "
                          "mixed: 64 requests of 128..2048 prompt tokens through the scheduler, --steps tokens generated each; "

@@ -288,7 +288,7 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
     // 32-column tiles of the result.
     constexpr int D = R + E, NC = D / 16, ND = R / 32, PK = D + 8, PIECES = D / 8;
     constexpr int WAVES = ND >= 4 ? 4 : ND, NDW = ND / WAVES, THREADS = 64 * WAVES;
-    constexpr int NL = (32 * PIECES + THREADS - 1) / THREADS;       // 16-byte pieces of a step a thread loads
+    constexpr int TPR = THREADS / 32, NL = (PIECES + TPR - 1) / TPR; // threads that load a row, 16-byte pieces each of them loads
     constexpr bool QLDS = NC > 20;         // long rows: the queries wait in LDS (in registers they would halve the waves a unit holds)
     __shared__ __attribute__((aligned(16))) uint16_t Ks[32 * PK];
     __shared__ __attribute__((aligned(16))) uint16_t Qs[QLDS ? 32 * PK : 8];
@@ -329,27 +329,25 @@ attn_latent_mfma_kernel(const bf16* __restrict__ qa, int qa_stride, bf16* __rest
     const int vcol = 16 * ((lane >> 4) & 1) + 4 * (lane & 3);
 
     // A step's rows are asked for one step ahead: while this step is computed out of LDS the next one's loads are in flight.
-    uint4 got[NL];
+    // (TPR threads share a row, so a thread looks up one page a step.)
+    const int my_row = threadIdx.x / TPR, my_piece = threadIdx.x % TPR;
+    sp_v4u got[NL];
     auto fetch = [&](int step) {
-        const int kb = 32 * step;
+        const int want = 32 * step + my_row;
+        const int key = (want < lo) ? lo : (want < pos) ? want : pos;
+        const bf16* src = cache + ((long long)bt[key / page_size] * page_size + key % page_size) * D + my_piece * 8;
 #pragma unroll
         for (int k = 0; k < NL; ++k) {
-            const int e = threadIdx.x + THREADS * k;
-            if (e < 32 * PIECES) {
-                const int row = e / PIECES, piece = e % PIECES;
-                const int key = (kb + row < lo) ? lo : (kb + row < pos) ? kb + row : pos;
-                got[k] = *reinterpret_cast<const uint4*>(cache + ((long long)bt[key / page_size] * page_size + key % page_size) * D + piece * 8);
-            }
+            if (PIECES % TPR == 0 || my_piece + TPR * k < PIECES) got[k] = *reinterpret_cast<const sp_v4u*>(src + TPR * 8 * k);
+            else got[k] = sp_v4u{0u, 0u, 0u, 0u};
         }
     };
     if (s_lo < s_hi) fetch(s_lo);
     for (int s = s_lo; s < s_hi; ++s) {
         const int kb = 32 * s;
 #pragma unroll
-        for (int k = 0; k < NL; ++k) {
-            const int e = threadIdx.x + THREADS * k;
-            if (e < 32 * PIECES) *reinterpret_cast<uint4*>(Ks + (e / PIECES) * PK + (e % PIECES) * 8) = got[k];
-        }
+        for (int k = 0; k < NL; ++k)
+            if (PIECES % TPR == 0 || my_piece + TPR * k < PIECES) *reinterpret_cast<sp_v4u*>(Ks + my_row * PK + (my_piece + TPR * k) * 8) = got[k];
         __syncthreads();
         if (s + 1 < s_hi) fetch(s + 1);
         lat_v16f sacc, sacc2;                  // two chains of dependent products instead of one
@@ -601,10 +599,30 @@ latent_gather_kernel(const T* __restrict__ cache, const int* __restrict__ table,
     }
 }
 
+// The rows alone, 16 bytes a thread (rows and cache of whole 16-byte pieces).
+__global__ void __launch_bounds__(256)
+latent_gather_vec_kernel(const uint4* __restrict__ cache, const int* __restrict__ table, int page_size, int pieces, int key0, int first,
+                         int L, int L_pad, uint4* __restrict__ rows) {
+    const long long e = (long long)blockIdx.x * 256 + threadIdx.x;
+    const int j = (int)(e / pieces), c = (int)(e % pieces), key = key0 + j;
+    if (j >= L_pad) return;
+    uint4 v = uint4{0u, 0u, 0u, 0u};
+    if (key >= first && key < L) v = cache[((long long)table[key / page_size] * page_size + key % page_size) * pieces + c];
+    rows[e] = v;
+}
+
 IC_EXPORT int ic_latent_gather(const void* cache, int dtype, const int* table, int page_size, int D, int R, int key0, int first, int L,
                                int L_pad, void* rows, void* rows_t, hipStream_t stream) {
     if (L <= 0) return IC_OK;
     if (page_size <= 0 || D <= 0 || R <= 0 || R > D || key0 < 0 || first < key0 || L <= first || L_pad < L - key0) return IC_ERR_ARG;
+    const int piece = dtype == IC_F32 ? 4 : 8;
+    if (!rows_t && (dtype == IC_F32 || dtype == IC_BF16) && D % piece == 0 && (((uintptr_t)cache | (uintptr_t)rows) & 15) == 0) {
+        const long long blocks = ((long long)L_pad * (D / piece) + 255) / 256;
+        if (blocks > 0x7fffffffLL) return IC_ERR_TOO_LARGE;
+        hipLaunchKernelGGL(latent_gather_vec_kernel, dim3((unsigned)blocks), dim3(256), 0, stream, (const uint4*)cache, table, page_size,
+                           D / piece, key0, first, L, L_pad, (uint4*)rows);
+        return ic_launch_status();
+    }
     dim3 grid((L_pad + 63) / 64, rows_t ? 1 + (R + 63) / 64 : 1), block(256);
     if (dtype == IC_F32)
         hipLaunchKernelGGL(latent_gather_kernel<float>, grid, block, 0, stream, (const float*)cache, table, page_size, D, R, key0, first,

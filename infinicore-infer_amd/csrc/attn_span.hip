@@ -290,7 +290,11 @@ attn_span_decode_kernel(const T* __restrict__ q, int q_stride, const T* __restri
 #pragma unroll
                     for (int i = 0; i < VEC; ++i) d += qv[j][i] * kf[u][i];
                     d = group_sum<LPK>(d);                  // over the lanes that share the key (DPP steps inside a row of 16 lanes)
-                    if (softcap > 0.f) d = cap2 * tanhf(d);
+                    if (softcap > 0.f) {
+                        // 16-bit keys: tanh(z) = 1 - 2 / (1 + e^(2z)), a last place of the cap off; finite for every z
+                        if (sizeof(T) == 2) d = cap2 - 2.f * cap2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(2.f * kLog2e * d));
+                        else d = cap2 * tanhf(d);
+                    }
                     d -= sl[j] * back[u];
                     s[u] = ok[u] ? d : -INFINITY;
                     mx = fmaxf(mx, s[u]);

@@ -31,7 +31,7 @@ __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf
 //   kSpanLatent  one request's keys and values made from its latent rows, in two matrices: row key - key0 of `kcache` holds
 //                every head's unrotated key part (dk - e_rot entries at head * (dk - e_rot)) and, from v_off on, every head's
 //                value; row key - key0 of `krot` the rotated part (e_rot entries) that the heads share.  The tiles are
-//                the portion's own, the last one first: tiles[0] = (.., first token row, tokens, first position).
+//                the portion's own, the last one first; z.portion = (.., first token row, tokens, first position).
 // =============================================================================================
 typedef __bf16 sp_bf16x8 __attribute__((ext_vector_type(8)));
 typedef float sp_v16f __attribute__((ext_vector_type(16)));
@@ -41,6 +41,7 @@ typedef unsigned sp_v4u __attribute__((ext_vector_type(4)));
 
 constexpr int kSpRows = 128;      // query rows per block
 constexpr int kSpKeys = 64;       // keys per step
+constexpr int kSpUnits = 256;     // compute units of the chip
 
 enum { kSpanPaged = 0, kSpanPadded = 1, kSpanLatent = 2 };
 
@@ -80,12 +81,17 @@ attn_span_prefill_kernel(const uint16_t* __restrict__ q, int q_stride, uint16_t*
 
     const int slot = (int)blockIdx.x;
     const int h = slot % nh;
+    // Tiles come longest first.  Where two blocks a unit hold the whole grid, its second half is taken shortest first, so that a
+    // unit's two blocks add up to about the same number of steps everywhere.
+    const int n_tiles = (int)gridDim.x / nh;
+    int place = slot / nh;
+    if ((int)gridDim.x <= 2 * kSpUnits && place >= (n_tiles + 1) / 2) place = n_tiles - 1 - (place - (n_tiles + 1) / 2);
     int4 tile;
     if (MODE == kSpanLatent) {
-        const int i = ((int)gridDim.x - 1 - slot) / nh * kSpRows;
+        const int i = (n_tiles - 1 - place) * kSpRows;
         tile = int4{0, z.portion.y + i, z.portion.z - i < kSpRows ? z.portion.z - i : kSpRows, z.portion.w + i};
     } else {
-        tile = tiles[slot / nh];
+        tile = tiles[place];
     }
     const int req = tile.x, row0 = tile.y, n_rows = tile.z, pos0 = tile.w;
     const int kvh = h / (nh / nkvh);

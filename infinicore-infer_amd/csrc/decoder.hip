@@ -194,7 +194,7 @@ struct IcDecoder {
         const int slices = ic_gemm_splitk_slices(d, K);
         const int st = ic_gemm_splitk(a, w, parts, T, d, K, K, K, slices, stream);
         if (st) return st;
-        return ic_splitk_add_rmsnorm(parts, slices, T, x, alpha, weight, out, d, eps, stream);
+        return ic_splitk_add_rmsnorm(parts, slices, T, x, alpha, weight, out, d, eps, nullptr, 0.f, nullptr, 0.f, stream);
     }
 
     int forward(const IcStepBatch& b, void* workspace, long long workspace_bytes, void* lib_ws, long long lib_ws_bytes,

@@ -221,7 +221,8 @@ __device__ __forceinline__ void sum4(const float* __restrict__ P, size_t slice_s
 // One block a row, the row in registers between the sum of squares and the scaling (d % 4 == 0, d <= 16 * threads).
 template <int VPT>
 __global__ void splitk_add_norm_kernel(const float* __restrict__ P, int S, int M, float* __restrict__ x, float alpha,
-                                       const float* __restrict__ w, uint16_t* __restrict__ out, int d, float eps) {
+                                       const float* __restrict__ w, uint16_t* __restrict__ out, int d, float eps,
+                                       const uint16_t* __restrict__ y0, float s0, const uint16_t* __restrict__ y1, float s1) {
     __shared__ float red[16];
     const int m = blockIdx.x;
     const size_t ss = (size_t)M * d, row = (size_t)m * d;
@@ -236,6 +237,13 @@ __global__ void splitk_add_norm_kernel(const float* __restrict__ P, int S, int M
             const float4 xv = *reinterpret_cast<const float4*>(x + row + c);
             v[i][0] = xv.x + alpha * y[0]; v[i][1] = xv.y + alpha * y[1];
             v[i][2] = xv.z + alpha * y[2]; v[i][3] = xv.w + alpha * y[3];
+            auto also = [&](const uint16_t* yk, float sk) {            // another result of four 16-bit values
+                const uint2 b = *reinterpret_cast<const uint2*>(yk + row + c);
+                v[i][0] += sk * __uint_as_float(b.x << 16); v[i][1] += sk * __uint_as_float(b.x & 0xffff0000u);
+                v[i][2] += sk * __uint_as_float(b.y << 16); v[i][3] += sk * __uint_as_float(b.y & 0xffff0000u);
+            };
+            if (y0) also(y0, s0);
+            if (y1) also(y1, s1);
             *reinterpret_cast<float4*>(x + row + c) = make_float4(v[i][0], v[i][1], v[i][2], v[i][3]);
 #pragma unroll
             for (int e = 0; e < 4; ++e) sq += v[i][e] * v[i][e];
@@ -329,8 +337,9 @@ IC_EXPORT int ic_gemm_splitk(const void* A, const void* W, float* P, int M, int 
 
 // x (float32 [M, d]) += alpha * (the product of slices P [S, M, d], rounded to bfloat16); out (bfloat16 [M, d]) = rmsnorm(x) * w.
 IC_EXPORT int ic_splitk_add_rmsnorm(const float* P, int n_slices, int M, float* x, float alpha, const float* w, void* out, int d,
-                                    float eps, hipStream_t stream) {
+                                    float eps, const void* y0, float s0, const void* y1, float s1, hipStream_t stream) {
     if (M <= 0) return IC_OK;
+    if (((uintptr_t)y0 & 7) || ((uintptr_t)y1 & 7)) return IC_ERR_ARG;
     if (d <= 0 || !x || !w || !out || !splits_ok(P, n_slices, M, d)) return IC_ERR_ARG;
     if (((uintptr_t)x & 15) || ((uintptr_t)w & 15) || ((uintptr_t)out & 7)) return IC_ERR_ARG;
     if (d % 4) return IC_ERR_UNSUPPORTED;
@@ -341,11 +350,12 @@ IC_EXPORT int ic_splitk_add_rmsnorm(const float* P, int n_slices, int M, float* 
     if (vpt > 4) return IC_ERR_UNSUPPORTED;
     dim3 grid(M), block(threads);
     uint16_t* o = (uint16_t*)out;
+    const uint16_t *a = (const uint16_t*)y0, *b = (const uint16_t*)y1;
     switch (vpt) {
-    case 1: hipLaunchKernelGGL(splitk_add_norm_kernel<1>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps); break;
-    case 2: hipLaunchKernelGGL(splitk_add_norm_kernel<2>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps); break;
-    case 3: hipLaunchKernelGGL(splitk_add_norm_kernel<3>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps); break;
-    default: hipLaunchKernelGGL(splitk_add_norm_kernel<4>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps); break;
+    case 1: hipLaunchKernelGGL(splitk_add_norm_kernel<1>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps, a, s0, b, s1); break;
+    case 2: hipLaunchKernelGGL(splitk_add_norm_kernel<2>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps, a, s0, b, s1); break;
+    case 3: hipLaunchKernelGGL(splitk_add_norm_kernel<3>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps, a, s0, b, s1); break;
+    default: hipLaunchKernelGGL(splitk_add_norm_kernel<4>, grid, block, 0, stream, P, n_slices, M, x, alpha, w, o, d, eps, a, s0, b, s1); break;
     }
     return ic_launch_status();
 }

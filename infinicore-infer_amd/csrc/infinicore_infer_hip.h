@@ -137,8 +137,8 @@ int ic_gemm_splitk_supported(int M, int N, int K, int lda, int ldw);
 int ic_gemm_splitk_slices(int N, int K);      // how many slices to use (never an empty one)
 int ic_gemm_splitk_pays(int M, int N, int K);
 int ic_gemm_splitk(const void* A, const void* W, float* P, int M, int N, int K, int lda, int ldw, int n_slices, hipStream_t stream);
-// P [S, M, d]: x += alpha * (the product, rounded to bfloat16); out = rmsnorm(x) * w.
-int ic_splitk_add_rmsnorm(const float* P, int n_slices, int M, float* x, float alpha, const float* w, void* out, int d, float eps, hipStream_t stream);
+// P [S, M, d]: x += alpha * (the product, rounded to bfloat16) + s0 y0 + s1 y1 (bfloat16 [M, d], nullable); out = rmsnorm(x) * w.
+int ic_splitk_add_rmsnorm(const float* P, int n_slices, int M, float* x, float alpha, const float* w, void* out, int d, float eps, const void* y0, float s0, const void* y1, float s1, hipStream_t stream);
 
 // ---- matmul_library.hip ------------------------------------------------------------------------------
 // The library (hipBLASLt) matrix product for many rows: C[M, N] = alpha * A[M, K] W[N, K]^T, bfloat16 operands with a

@@ -182,7 +182,7 @@ _SIGNATURES = {
     "ic_gemm_splitk_slices": [_I, _I],
     "ic_gemm_splitk": [_P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "ic_gemm_splitk_pays": [_I, _I, _I],
-    "ic_splitk_add_rmsnorm": [_P, _I, _I, _P, _F, _P, _P, _I, _F, _P],
+    "ic_splitk_add_rmsnorm": [_P, _I, _I, _P, _F, _P, _P, _I, _F, _P, _F, _P, _F, _P],
     "ic_rule_few_rows": [],
     "ic_rule_sumsq_parts_max": [],
     "ic_rule_own_product": [_I, _I, _I, _I],

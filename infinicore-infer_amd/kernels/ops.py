@@ -665,15 +665,21 @@ def gemm_splitk(a, w, parts, n_slices=None):
     return parts.view(-1)[:S * M * N].view(S, M, N)
 
 
-def splitk_add_rmsnorm(parts, x, alpha: float, weight, out, eps: float):
-    """x += alpha * (the product given as slices parts [S, M, d], rounded to bfloat16); out = rmsnorm(x) * weight."""
+def splitk_add_rmsnorm(parts, x, alpha: float, weight, out, eps: float, also=()):
+    """x += alpha * (the product given as slices parts [S, M, d], rounded to bfloat16) + the sum of s_i y_i over ``also`` (up to
+    two (y, s), bfloat16); out = rmsnorm(x) * weight."""
     _dev(parts, x, weight, out)
     S, M, d = parts.shape
     _need(parts.dtype == torch.float32 and parts.is_contiguous() and x.dtype == torch.float32 and x.is_contiguous()
           and tuple(x.shape) == (M, d) and weight.dtype == torch.float32 and weight.numel() == d and weight.is_contiguous()
           and out.dtype == torch.bfloat16 and out.is_contiguous() and tuple(out.shape) == (M, d), "splitk_add_rmsnorm: layout")
+    _need(len(also) <= 2, "splitk_add_rmsnorm: at most two more results")
+    for y, _ in also:
+        _dev(y)
+        _need(y.dtype == torch.bfloat16 and y.is_contiguous() and tuple(y.shape) == (M, d), "splitk_add_rmsnorm: another result")
+    two = [(y.data_ptr(), float(f)) for y, f in also] + [(None, 0.0)] * (2 - len(also))
     check(get_lib().ic_splitk_add_rmsnorm(parts.data_ptr(), S, M, x.data_ptr(), float(alpha), weight.data_ptr(), out.data_ptr(),
-                                          d, float(eps), _stream()), "splitk_add_rmsnorm")
+                                          d, float(eps), *[v for pair in two for v in pair], _stream()), "splitk_add_rmsnorm")
     return out
 
 

@@ -130,11 +130,13 @@ class ResidualTail:
     """What a block asks of a part's LAST projection (a part with ``fuses_tail``): add the part's
     output y to the float32 residual stream, x += alpha * y, and hand back the input of the norm
     that follows (weight, eps) as ``DeferredRows``.  A part that cannot do it for this step returns
-    its plain output and the block does the add and the norm itself."""
+    its plain output and the block does the add and the norm itself.  ``also``: other results (tensor, factor)
+    that are owed to the stream and belong under the same norm; who cannot add them returns its plain output."""
     x: torch.Tensor
     alpha: float
     weight: torch.Tensor
     eps: float
+    also: Tuple[Tuple[torch.Tensor, float], ...] = ()
 
 
 def packed_rows(tensors, pack: str, names):
@@ -261,6 +263,7 @@ class Mixer(Part):
     accepts_deferred = False     # forward() takes DeferredRows as h
     fuses_tail = False           # forward() takes tail=ResidualTail and may return DeferredRows
     yields_branches = False      # forward() takes branches=True and may return Branches
+    adds_into_stream = False     # forward() takes into=ResidualTail: it may add its result to tail.x (no norm) and return None
     # Where a mixer's state begins in its cache slot's state row, and the workspace buffer of its result: a mixer that joins
     # others sets them for its children.  A mixer that honours both says so with ``relocatable``.
     relocatable = False

@@ -271,9 +271,15 @@ class OwedBranches:
 @register_part("block", "shared_norm_residual")
 class SharedNormResidualBlock(Block):
     """h = norm(x); x += mixer(h) + ff(h): one norm, whose output both sublayers read (the second term only when the layer has a
-    feed-forward).  The stream is float32; both results (and the branches of a mixer that yields them) stay owed, and one row
-    kernel of the next block adds them all and forms its norm."""
+    feed-forward).  The stream is float32.
+
+    For few rows nothing stands between the products: the mixer's last projection (of every branch) adds its result to the
+    stream in its epilogue, the feed-forward's does so too and hands on the next norm's rows (``ResidualTail``), and both
+    sublayers' first products apply the row factors (``DeferredRows``).  Otherwise the results (and the branches of a mixer that
+    yields them) stay owed, and one row kernel adds them all and forms the next block's norm: the sliced down projection's,
+    or this block's own."""
     graph_safe = True
+    fuses_successor = True
     accepts_owed_update = (OwedBranches,)
 
     def __init__(self, name, runtime, mixer=None, mixer_norm=None, feed_forward=None, feed_forward_norm=None):
@@ -283,7 +289,13 @@ class SharedNormResidualBlock(Block):
         if mixer_norm.deferred() is None:
             raise ValueError("block %s: norm part %s is not a weighted RMS norm" % (name, type(mixer_norm).__name__))
 
-    def forward(self, x, pending, ctx, cache):
+    def entry_norm(self):
+        takers = [self.mixer] + ([self.feed_forward] if self.feed_forward is not None else [])
+        return self.mixer_norm if all(getattr(p, "accepts_deferred", False) for p in takers) else None
+
+    def _normed(self, x, pending, ctx):
+        if isinstance(pending, DeferredRows):
+            return pending
         h = ctx.ws.buffer("normed", tuple(x.shape), self.runtime.dtype)
         weight, eps = self.mixer_norm.deferred()
         if isinstance(pending, OwedBranches):
@@ -292,11 +304,25 @@ class SharedNormResidualBlock(Block):
             self.mixer_norm.forward(x, h)
         else:
             self.mixer_norm.forward_add(x, pending[0], pending[1], h)
-        y = self.mixer.forward(h, ctx, cache, branches=True) if self.mixer.yields_branches else self.mixer.forward(h, ctx, cache)
-        owed = y.parts if isinstance(y, Branches) else ((y, 1.0),)
+        return h
+
+    def forward(self, x, pending, ctx, cache, successor=None):
+        h = self._normed(x, pending, ctx)
+        weight, eps = self.mixer_norm.deferred()
+        options = {"branches": True} if self.mixer.yields_branches else {}
+        if self.mixer.adds_into_stream:
+            options["into"] = ResidualTail(x, 1.0, weight, eps)          # (the norm's part of it is not used)
+        y = self.mixer.forward(h, ctx, cache, **options)
+        owed = () if y is None else y.parts if isinstance(y, Branches) else ((y, 1.0),)
         if self.feed_forward is not None:
-            owed += ((self.feed_forward.forward(h, ctx), 1.0),)
-        return OwedBranches(owed)
+            tail = None
+            if successor is not None and successor.deferred() is not None and getattr(self.feed_forward, "fuses_tail", False):
+                tail = ResidualTail(x, 1.0, *successor.deferred(), also=owed)
+            f = self.feed_forward.forward(h, ctx, tail=tail) if tail is not None else self.feed_forward.forward(h, ctx)
+            if isinstance(f, DeferredRows):
+                return f
+            owed += ((f, 1.0),)
+        return OwedBranches(owed) if owed else None
 
 
 @register_part("block", "sandwich_gated")

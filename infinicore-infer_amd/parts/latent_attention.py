@@ -23,7 +23,7 @@ import torch
 from ..kernels import ops
 from ..weights.loader import WeightSpec
 from .base import CacheNeed, Mixer, packed_rows, register_part
-from .linear import _library, linear
+from .linear import _library, linear, linear_into_stream
 from .rotary import pair_frequencies, stretched_magnitude
 
 PORTION_MIN = 32                       # tokens from which a portion makes keys and values per head
@@ -33,6 +33,8 @@ MADE_KEYS_BYTES = 8 << 30              # most memory the keys and values made fo
 @register_part("mixer", "latent_attention")
 class LatentAttention(Mixer):
     graph_safe = True
+    accepts_deferred = True
+    adds_into_stream = True
 
     def __init__(self, name, runtime, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, value_dim: int,
                  q_rank: int, kv_rank: int, softmax_scale: float, rot_base: float, rot_dims=None, norm_eps: float = 1e-6,
@@ -202,7 +204,7 @@ class LatentAttention(Mixer):
         ops.blocked_product(walked.view(n, H, R), self.w_uv, heads_out[rows].view(n, H, self.dv),
                             gate=None if gate is None else gate[rows].view(n, H, self.dv))
 
-    def forward(self, h, ctx, cache):
+    def forward(self, h, ctx, cache, into=None):
         rt, T, H, R, E = self.runtime, h.shape[0], self.H, self.R, self.E
         rows = ctx.ws.buffer("latent_rows", (T, self.w_down.shape[0]), rt.dtype)
         linear(h, self.w_down, rows, rt.gemm_impl, ws=ctx.ws)
@@ -219,6 +221,8 @@ class LatentAttention(Mixer):
         for portion in portions:
             if not (self._makes_keys() and self._portion_by_keys(portion, q, gate, heads_out, ctx, cache)):
                 self._portion_by_products(portion, q, gate, heads_out, ctx, cache)
+        if linear_into_stream(heads_out, self.w_o, into, ctx.ws, "mixer_tail", rt.gemm_impl):
+            return None
         y = ctx.ws.buffer("mixer_out", (T, self.hidden_size), rt.dtype)
         linear(heads_out, self.w_o, y, rt.gemm_impl, ws=ctx.ws)
         return y

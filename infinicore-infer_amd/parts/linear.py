@@ -91,7 +91,7 @@ def linear_tail(x, w, tail, ws, name: str, impl: str = "auto"):
     if tail is None or impl != "auto" or tuple(tail.x.shape) != (M, N) or x.stride(1) != 1 or w.stride(1) != 1:
         return None
     how = ops.rule_tail(x.dtype, x, w)
-    if how == ops.TAIL_PLAIN:
+    if how == ops.TAIL_PLAIN or (tail.also and how != ops.TAIL_SLICES):
         return None
     if how == ops.TAIL_SLICES:
         # 17..64 rows into the residual stream (and 13..16 long ones): the product as slices over K; the kernel that
@@ -99,10 +99,18 @@ def linear_tail(x, w, tail, ws, name: str, impl: str = "auto"):
         slices = ops.gemm_splitk_slices(N, w.shape[1])
         parts = ops.gemm_splitk(x, w, ws.buffer("tail_parts", (slices * M * N,), torch.float32), slices)
         y = ws.buffer(name + "_values", (M, N), torch.bfloat16)
-        ops.splitk_add_rmsnorm(parts, tail.x, tail.alpha, tail.weight, y, tail.eps)
+        ops.splitk_add_rmsnorm(parts, tail.x, tail.alpha, tail.weight, y, tail.eps, also=tail.also)
         return DeferredRows(y, None, N, tail.eps)
     parts = ops.residual_parts(N)
     y = ws.buffer(name + "_values", (M, N), torch.bfloat16)
     sumsq = ws.buffer(name + "_sumsq", (parts, 16), torch.float32)
     ops.gemm_nt(x, w, y, residual=(tail.x, tail.weight, tail.alpha, sumsq))
     return DeferredRows(y, sumsq, N, tail.eps)
+
+
+def linear_into_stream(x, w, tail, ws, name: str, impl: str = "auto") -> bool:
+    """The last projection of a part with the residual add in its epilogue and no norm (another part's result joins the stream
+    before it is normed): True when it was done, for few rows; otherwise the caller computes the plain product."""
+    if tail is None or ops.rule_tail(x.dtype, x, w) != ops.TAIL_SPLIT_NORM:
+        return False
+    return linear_tail(x, w, tail, ws, name, impl) is not None

@@ -24,7 +24,7 @@ import torch
 from ..kernels import ops
 from ..weights.loader import FreeDim, WeightSpec
 from .base import CacheNeed, Mixer, packed_rows, register_part
-from .linear import linear
+from .linear import linear, linear_into_stream
 
 UNIT_EPS = 1e-6            # under the root of the unit length of the delta rule's queries and keys
 MAX_KEY_DIM = 1024         # rows of a head's state that the recurrence keeps in registers
@@ -43,11 +43,14 @@ LIBRARY_ROWS = 256         # from so many tokens on the thin products (K an inne
 class _MatrixMemory(Mixer):
     graph_safe = True
     relocatable = True
+    adds_into_stream = True
 
     def cache_need(self):
         return CacheNeed("state", state_shape=((self.state_size + 3) // 4 * 4,), state_dtype=torch.float32)
 
-    def _result(self, rows, ctx):
+    def _result(self, rows, ctx, into=None):
+        if linear_into_stream(rows, self.w_o, into, ctx.ws, "mixer_tail", self.runtime.gemm_impl):
+            return None
         y = ctx.ws.buffer(self.out_buffer, (rows.shape[0], self.hidden_size), self.runtime.dtype)
         linear(rows, self.w_o, y, self.runtime.gemm_impl, ws=ctx.ws)
         return y
@@ -73,6 +76,8 @@ class _MatrixMemory(Mixer):
 
 @register_part("mixer", "gated_delta")
 class GatedDeltaRule(_MatrixMemory):
+    accepts_deferred = True
+
     def __init__(self, name, runtime, hidden_size: int, heads: int, kv_heads: int, key_dim: int, value_dim: int, conv_taps: int,
                  norm_eps: float, decay: str = "channel"):
         """``decay``: "channel" (low-rank decay and gate projections, a sigmoid gate) or "head" (dense ones, a silu gate)."""
@@ -133,7 +138,7 @@ class GatedDeltaRule(_MatrixMemory):
             ops.blocked_product(g1.unsqueeze(1), self.w_g2.unsqueeze(0), gate.unsqueeze(1))
         return rows[:, c + self.ra + self.rg:], decay, gate
 
-    def forward(self, h, ctx, cache):
+    def forward(self, h, ctx, cache, into=None):
         rt, T, c = self.runtime, h.shape[0], self.channels
         buf = ctx.ws.buffer
         rows = self._project(h, ctx)
@@ -155,11 +160,13 @@ class GatedDeltaRule(_MatrixMemory):
                           compute_units=ctx.cu_count)
         g = buf("memory_gated", (T, self.nv), rt.dtype)
         ops.gated_head_norm(o, gate, self.norm_w, self.heads, self.eps, g, gate="silu" if self.per_head else "sigmoid")
-        return self._result(g, ctx)
+        return self._result(g, ctx, into)
 
 
 @register_part("mixer", "gated_linear_attention")
 class GatedLinearAttention(_MatrixMemory):
+    accepts_deferred = True
+
     def __init__(self, name, runtime, hidden_size: int, heads: int, key_dim: int, value_dim: int, tau: float, norm_eps: float):
         super().__init__(name, runtime)
         _check_sizes("gated linear attention", heads, heads, key_dim, value_dim)
@@ -188,7 +195,7 @@ class GatedLinearAttention(_MatrixMemory):
         self.w_a2 = tensors[n + "a2"].to(self.runtime.dtype).contiguous()
         self.b_a2, self.norm_w, self.w_o = tensors[n + "a2.b"], tensors[n + "norm"], tensors[n + "o"]
 
-    def forward(self, h, ctx, cache):
+    def forward(self, h, ctx, cache, into=None):
         rt, T, nq, nv = self.runtime, h.shape[0], self.nq, self.nv
         buf = ctx.ws.buffer
         rows = self._project(h, ctx)
@@ -199,11 +206,13 @@ class GatedLinearAttention(_MatrixMemory):
                           q_scale=self.dk ** -0.5, compute_units=ctx.cu_count)
         g = buf("memory_gated", (T, nv), rt.dtype)
         ops.gated_head_norm(o, rows[:, 2 * nq + nv:2 * nq + 2 * nv], self.norm_w, self.heads, self.eps, g, gate="silu")
-        return self._result(g, ctx)
+        return self._result(g, ctx, into)
 
 
 @register_part("mixer", "exponential_memory")
 class ExponentialMemory(_MatrixMemory):
+    accepts_deferred = True
+
     def __init__(self, name, runtime, hidden_size: int, heads: int, key_dim: int, value_dim: int, gate_cap: float, norm_eps: float):
         super().__init__(name, runtime)
         _check_sizes("exponential memory", heads, heads, key_dim, value_dim)
@@ -233,7 +242,7 @@ class ExponentialMemory(_MatrixMemory):
         self.b_i, self.b_f = tensors[n + "i.b"], tensors[n + "f.b"]
         self.norm_w, self.w_o = tensors[n + "norm"], tensors[n + "o"]
 
-    def forward(self, h, ctx, cache):
+    def forward(self, h, ctx, cache, into=None):
         rt, T, H, nq, nv = self.runtime, h.shape[0], self.heads, self.nq, self.nv
         buf = ctx.ws.buffer
         rows = self._project(h, ctx)
@@ -248,4 +257,4 @@ class ExponentialMemory(_MatrixMemory):
                           compute_units=ctx.cu_count)
         g = buf("memory_gated", (T, nv), rt.dtype)
         ops.gated_head_norm(o, rows[:, 2 * nq + nv:], self.norm_w, H, self.eps, g, num=num, floor=floor)
-        return self._result(g, ctx)
+        return self._result(g, ctx, into)

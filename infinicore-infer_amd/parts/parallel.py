@@ -2,6 +2,8 @@
 
 At most one of them walks a paged cache; their states lie one after the other in the slot's state row (every mixer is told
 where its own begins), and each writes its result to a buffer of its own."""
+from dataclasses import replace
+
 from .base import Branches, CacheNeed, Mixer, build_part, register_part
 
 
@@ -28,6 +30,8 @@ class ParallelMixers(Mixer):
                     raise ValueError("parallel mixers: %s keeps a state that is no row of numbers" % type(c).__name__)
                 base += (need.state_shape[0] + 3) // 4 * 4           # every state starts on 16 bytes
         self.state_size = base
+        self.accepts_deferred = all(c.accepts_deferred for c in self.children)
+        self.adds_into_stream = any(c.adds_into_stream for c in self.children)
         self._need = self._joined_need()
 
     def _joined_need(self) -> CacheNeed:
@@ -50,10 +54,19 @@ class ParallelMixers(Mixer):
     def cache_need(self):
         return self._need
 
-    def forward(self, h, ctx, cache, branches: bool = False):
-        out = Branches(tuple((c.forward(h, ctx, cache), f) for c, f in zip(self.children, self.factors)))
+    def forward(self, h, ctx, cache, branches: bool = False, into=None):
+        parts = []
+        for c, f in zip(self.children, self.factors):
+            # a child that adds its result to the stream by itself does so with its factor
+            mine = None if into is None or not c.adds_into_stream else replace(into, alpha=into.alpha * f)
+            y = c.forward(h, ctx, cache) if mine is None else c.forward(h, ctx, cache, into=mine)
+            if y is not None:
+                parts.append((y, f))
+        out = Branches(tuple(parts))
         if branches:
             return out
+        if not parts:
+            return None
         y = ctx.ws.buffer("mixer_out", tuple(out.parts[0][0].shape), self.runtime.dtype)
         y.zero_()
         for v, f in out.parts:

@@ -28,7 +28,7 @@ import torch
 from ..kernels import ops
 from ..weights.loader import WeightSpec
 from .base import CacheNeed, Mixer, packed_rows, register_part
-from .linear import linear
+from .linear import linear, linear_into_stream
 from .rotary import pair_frequencies
 
 _NORM_MODES = {None: 0, "none": 0, "head": 1, "row": 2}
@@ -39,6 +39,8 @@ _MIX_MODES = {None: 0, "none": 0, "keep": 1, "mix": 2}
 class SpanAttention(Mixer):
     graph_safe = True
     relocatable = True
+    accepts_deferred = True
+    adds_into_stream = True
     defers_bias = True           # forward(.., defer_bias=True) leaves the output projection's bias to the caller
 
     def __init__(self, name, runtime, hidden_size: int, num_heads: int, num_kv_heads: int, key_dim: int,
@@ -180,7 +182,7 @@ class SpanAttention(Mixer):
         return self.b_o
 
     # ---- forward ------------------------------------------------------------------------------
-    def forward(self, h, ctx, cache, defer_bias: bool = False):
+    def forward(self, h, ctx, cache, defer_bias: bool = False, into=None):
         rt = self.runtime
         T = h.shape[0]
         rows = ctx.ws.buffer("span_rows", (T, self.w_rows.shape[0]), rt.dtype)
@@ -198,6 +200,8 @@ class SpanAttention(Mixer):
         out = ctx.ws.buffer("span_out", (T, self.na), rt.dtype)
         gate = rows[:, rows.shape[1] - self.na:] if self.gate else None
         self._attend(q, out, gate, ctx, cache)
+        if self.b_o is None and linear_into_stream(out, self.w_o, into, ctx.ws, "mixer_tail", rt.gemm_impl):
+            return None
         y = ctx.ws.buffer(self.out_buffer, (T, self.hidden_size), rt.dtype)
         linear(out, self.w_o, y, rt.gemm_impl, ws=ctx.ws)
         if self.b_o is not None and not defer_bias:

@@ -67,7 +67,9 @@ attn_span_prefill_kernel(const uint16_t* __restrict__ q, int q_stride, uint16_t*
     constexpr int PK = DK + 8;            // padded row pitches in LDS (elements)
     constexpr int PV = DV + 8;
     constexpr int KCH = DK / 8, VCH = DV / 8;              // 16-byte chunks of a row
-    constexpr int NLK = kSpKeys * KCH / 256, NLV = kSpKeys * VCH / 256;     // loads per thread and step
+    constexpr int LPR = (KCH % 8 == 0 && VCH % 8 == 0) ? 8 : 4;             // threads that fetch a row
+    constexpr int RP = 256 / LPR, NP = kSpKeys / RP;                        // rows fetched side by side, passes over a step's rows
+    constexpr int NKC = KCH / LPR, NVC = VCH / LPR, NLK = NP * NKC, NLV = NP * NVC;     // loads per row, per thread and step
     static_assert(DK % 32 == 0 && DV % 32 == 0, "a step's rows split evenly over the block");
     // long rows keep one stage in LDS, so that two blocks fit a compute unit
     constexpr bool ONE_STAGE = 2 * kSpKeys * (PK + PV) * 2 > 80 * 1024;
@@ -139,8 +141,12 @@ attn_span_prefill_kernel(const uint16_t* __restrict__ q, int q_stride, uint16_t*
 
     const size_t khead = (size_t)kvh * page_size * dk, vhead = (size_t)kvh * page_size * dv;
     sp_v4u kreg0[NLK], vreg0[NLV], kreg1[NLK], vreg1[NLV];     // two steps' keys and values on their way: a load has two steps' time to arrive
-    int pgk[NLK], pgv[NLV];                            // page ids of the keys this thread fetches next: looked up a step ahead of the
-                                                       // fetch, so a step waits for one trip to memory, not for two in a row
+    // A thread fetches the same rows' pieces of keys and of values, and looks their page ids up a step ahead of the fetch, so a
+    // step waits for one trip to memory, not for two in a row.
+    const int my_key = tid / LPR, piece = tid % LPR;
+    const int k_last = dk / 8 - 1, v_last = dv / 8 - 1;       // (MODE kSpanPaged: never reached beyond)
+    const bool padded = MODE != kSpanPaged && (dk < DK || dv < DV);
+    int page[NP];
     auto key_of = [&](int s, int kk) -> int {
         int kb, klo, khi;
         step_of(s, kb, klo, khi);
@@ -151,49 +157,54 @@ attn_span_prefill_kernel(const uint16_t* __restrict__ q, int q_stride, uint16_t*
     auto lookup = [&](int s) {
         if (MODE == kSpanLatent) return;
 #pragma unroll
-        for (int i = 0; i < NLK; ++i) pgk[i] = bt[key_of(s, (tid + i * 256) / KCH) >> page_shift];
-#pragma unroll
-        for (int i = 0; i < NLV; ++i) pgv[i] = bt[key_of(s, (tid + i * 256) / VCH) >> page_shift];
+        for (int p = 0; p < NP; ++p) page[p] = bt[key_of(s, my_key + RP * p) >> page_shift];
     };
     auto fetch = [&](int s, sp_v4u* kreg, sp_v4u* vreg) {
 #pragma unroll
-        for (int i = 0; i < NLK; ++i) {
-            const int idx = tid + i * 256, kk = idx / KCH, c = idx - kk * KCH;
-            const int key = key_of(s, kk);
+        for (int p = 0; p < NP; ++p) {
+            const int key = key_of(s, my_key + RP * p);
+            const uint16_t *kp, *vp, *rp = nullptr;
             if (MODE == kSpanLatent) {
-                const size_t row = (size_t)(key - z.key0);
-                kreg[i] = sp_v4u{0u, 0u, 0u, 0u};
-                if (c * 8 < d_plain) kreg[i] = *reinterpret_cast<const sp_v4u*>(kcache + row * z.kv_stride + (size_t)kvh * d_plain + c * 8);
-                else if (c * 8 < dk) kreg[i] = *reinterpret_cast<const sp_v4u*>(z.krot + row * z.krot_stride + (c * 8 - d_plain));
-                continue;
+                const uint16_t* row = kcache + (size_t)(key - z.key0) * z.kv_stride;
+                kp = row + kvh * d_plain;
+                vp = row + z.v_off + kvh * dv;
+                rp = z.krot + (size_t)(key - z.key0) * z.krot_stride - d_plain;
+            } else {
+                const size_t rowi = (((size_t)page[p] * nkvh) << page_shift) + (key & page_mask);
+                kp = kcache + khead + rowi * dk;
+                vp = vcache + vhead + rowi * dv;
             }
-            const size_t rowi = (((size_t)pgk[i] * nkvh) << page_shift) + (key & page_mask);
-            if (MODE == kSpanPadded) kreg[i] = sp_v4u{0u, 0u, 0u, 0u};
-            if (MODE == kSpanPaged || c * 8 < dk) kreg[i] = *reinterpret_cast<const sp_v4u*>(kcache + khead + rowi * dk + c * 8);
-        }
 #pragma unroll
-        for (int i = 0; i < NLV; ++i) {
-            const int idx = tid + i * 256, kk = idx / VCH, c = idx - kk * VCH;
-            const int key = key_of(s, kk);
-            if (MODE != kSpanPaged) vreg[i] = sp_v4u{0u, 0u, 0u, 0u};
-            if (MODE == kSpanLatent) {
-                if (c * 8 < dv) vreg[i] = *reinterpret_cast<const sp_v4u*>(kcache + (size_t)(key - z.key0) * z.kv_stride + z.v_off + (size_t)kvh * dv + c * 8);
-                continue;
+            for (int i = 0; i < NKC; ++i) {
+                int c = piece + LPR * i;
+                if (MODE != kSpanPaged) c = c < k_last ? c : k_last;         // pieces beyond the true size: a real one, cleared on the way to LDS
+                const uint16_t* src = (MODE == kSpanLatent && c * 8 >= d_plain) ? rp : kp;
+                kreg[p * NKC + i] = *reinterpret_cast<const sp_v4u*>(src + c * 8);
             }
-            const size_t rowi = (((size_t)pgv[i] * nkvh) << page_shift) + (key & page_mask);
-            if (MODE == kSpanPaged || c * 8 < dv) vreg[i] = *reinterpret_cast<const sp_v4u*>(vcache + vhead + rowi * dv + c * 8);
+#pragma unroll
+            for (int i = 0; i < NVC; ++i) {
+                int c = piece + LPR * i;
+                if (MODE != kSpanPaged) c = c < v_last ? c : v_last;
+                vreg[p * NVC + i] = *reinterpret_cast<const sp_v4u*>(vp + c * 8);
+            }
         }
     };
-    auto stash = [&](const sp_v4u* kreg, const sp_v4u* vreg, uint16_t* Ks, uint16_t* Vs) {
+    auto stash = [&](sp_v4u* kreg, sp_v4u* vreg, uint16_t* Ks, uint16_t* Vs) {
+        if (padded) {
 #pragma unroll
-        for (int i = 0; i < NLK; ++i) {
-            const int idx = tid + i * 256, kk = idx / KCH, c = idx - kk * KCH;
-            *reinterpret_cast<sp_v4u*>(Ks + kk * PK + c * 8) = kreg[i];
+            for (int p = 0; p < NP; ++p) {
+#pragma unroll
+                for (int i = 0; i < NKC; ++i) if (piece + LPR * i > k_last) kreg[p * NKC + i] = sp_v4u{0u, 0u, 0u, 0u};
+#pragma unroll
+                for (int i = 0; i < NVC; ++i) if (piece + LPR * i > v_last) vreg[p * NVC + i] = sp_v4u{0u, 0u, 0u, 0u};
+            }
         }
 #pragma unroll
-        for (int i = 0; i < NLV; ++i) {
-            const int idx = tid + i * 256, kk = idx / VCH, c = idx - kk * VCH;
-            *reinterpret_cast<sp_v4u*>(Vs + kk * PV + c * 8) = vreg[i];
+        for (int p = 0; p < NP; ++p) {
+#pragma unroll
+            for (int i = 0; i < NKC; ++i) *reinterpret_cast<sp_v4u*>(Ks + (my_key + RP * p) * PK + (piece + LPR * i) * 8) = kreg[p * NKC + i];
+#pragma unroll
+            for (int i = 0; i < NVC; ++i) *reinterpret_cast<sp_v4u*>(Vs + (my_key + RP * p) * PV + (piece + LPR * i) * 8) = vreg[p * NVC + i];
         }
     };
 
@@ -252,14 +263,14 @@ attn_span_prefill_kernel(const uint16_t* __restrict__ q, int q_stride, uint16_t*
         const bool all_seen = kb >= klo && kb + kSpKeys - 1 <= khi && kb + kSpKeys - 1 <= wave_first
                               && (window == 0 || wave_last - kb < window || kb + kSpKeys - 1 < keep_first);
         if (!all_seen) {
+            const int up = khi < qpos ? khi : qpos, low = (window > 0 && qpos - window + 1 > klo) ? qpos - window + 1 : klo;
 #pragma unroll
             for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
                 for (int r = 0; r < 16; ++r) {
                     const int key = kb + 32 * tt + 8 * (r >> 2) + 4 * half + (r & 3);
-                    const bool seen = key >= klo && key <= khi && key <= qpos
-                                      && (window == 0 || qpos - key < window || key < keep_first);
-                    if (!seen) sacc[tt][r] = -INFINITY;
+                    const bool seen = (key <= up) & ((key >= low) | ((key >= klo) & (key < keep_first)));
+                    sacc[tt][r] = seen ? sacc[tt][r] : -INFINITY;
                 }
         }
         // ---- running softmax, base 2: p = 2^(s c - m c) ---------------------------------

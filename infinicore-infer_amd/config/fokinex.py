@@ -4,7 +4,8 @@ Keys: ``architecture`` ("Fokinex"), ``vocab``, ``width``, ``norm.eps``, ``embedd
 ``type`` ("latent_attention" or "parallel"), ``mixer`` (the sizes and constants of that mixer) and ``mlp``: null or {kind: "dense",
 ff}.  Mixers: "latent_attention" {heads, dim, rot_dim, vdim, q_rank, kv_rank, scale, mask{size}, rot{base, dims, scaling{factor,
 original, fast, slow}}, kv_from}; "parallel" {left{heads, kv_heads, dim, vdim, scale, softcap, mask{size}}, left_scale, right{heads,
-kv_heads, dim, vdim, conv}, right_scale}.  ``kv_from``, ``mask``, ``rot.scaling``, ``softcap`` and ``embedding`` may be absent.  Tensor
+kv_heads, dim, vdim, conv}, right_scale}.  ``kv_from``, ``mask``, ``rot.scaling``, ``softcap`` and ``embedding`` may be absent, and ``q_rank`` (the
+tensors then decide it).  Tensor
 names: ``embed``, ``final.norm``, ``head`` and per layer i ``l<i>.norm1``, ``l<i>.mix.*`` (``mix.left.*`` and ``mix.right.*``),
 ``l<i>.mlp.gate`` / ``.up`` / ``.down``.
 
@@ -154,14 +155,14 @@ class FokinexConfig:
     def _mixer_spec(self, i: int, l: FokinexLayer) -> PartSpec:
         d, eps, name, where = self.hidden_size, self.norm_eps, "l%d.mix." % i, "layers[%d].mixer." % i
         if l.kind == "latent_attention":
-            s = _sizes(l.mixer, where, "heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank")
+            s = _sizes(l.mixer, where, "heads", "dim", "rot_dim", "vdim", "kv_rank")
             rot = _need(l.mixer, "rot", where)
             scaling = rot.get("scaling")
             if scaling:
                 scaling = {k: float(_need(scaling, k, where + "rot.scaling.")) for k in ("factor", "original", "fast", "slow")}
             return PartSpec("latent_attention", name, {
                 "hidden_size": d, "num_heads": s["heads"], "head_dim": s["dim"], "rot_dim": s["rot_dim"], "value_dim": s["vdim"],
-                "q_rank": s["q_rank"], "kv_rank": s["kv_rank"], "softmax_scale": float(_need(l.mixer, "scale", where)),
+                "q_rank": _sizes(l.mixer, where, "q_rank")["q_rank"] if l.mixer.get("q_rank") is not None else None, "kv_rank": s["kv_rank"], "softmax_scale": float(_need(l.mixer, "scale", where)),
                 "rot_base": float(_need(rot, "base", where + "rot.")), "rot_dims": int(rot.get("dims") or s["rot_dim"]),
                 "rot_scaling": scaling or None, "norm_eps": eps, "gate": False, "sink": True, "window": _window(l.mixer, where),
                 "own_rows": l.kv_from is None})

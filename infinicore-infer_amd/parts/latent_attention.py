@@ -21,7 +21,7 @@ rotated part turn by position * f_i, computed in float32.
 import torch
 
 from ..kernels import ops
-from ..weights.loader import WeightSpec
+from ..weights.loader import FreeDim, WeightSpec
 from .base import CacheNeed, Mixer, packed_rows, register_part
 from .linear import _library, linear, linear_into_stream
 from .rotary import pair_frequencies, stretched_magnitude
@@ -37,11 +37,12 @@ class LatentAttention(Mixer):
     adds_into_stream = True
 
     def __init__(self, name, runtime, hidden_size: int, num_heads: int, head_dim: int, rot_dim: int, value_dim: int,
-                 q_rank: int, kv_rank: int, softmax_scale: float, rot_base: float, rot_dims=None, norm_eps: float = 1e-6,
+                 q_rank, kv_rank: int, softmax_scale: float, rot_base: float, rot_dims=None, norm_eps: float = 1e-6,
                  gate: bool = True, window=None, sink: bool = False, rot_scaling=None, own_rows: bool = True):
+        """``q_rank`` None: the tensors decide the query latent's size."""
         super().__init__(name, runtime)
         rot_dims = rot_dim if rot_dims is None else int(rot_dims)
-        if min(num_heads, head_dim, value_dim, q_rank, kv_rank) <= 0 or rot_dim < 0:
+        if min(num_heads, head_dim, value_dim, 1 if q_rank is None else q_rank, kv_rank) <= 0 or rot_dim < 0:
             raise ValueError("latent attention: sizes must be positive")
         if kv_rank > ops.LATENT_MAX_RANK:
             raise ValueError("latent attention: a latent of %d values is beyond the kernel's %d" % (kv_rank, ops.LATENT_MAX_RANK))
@@ -50,7 +51,7 @@ class LatentAttention(Mixer):
         if window is not None and int(window) <= 0:
             raise ValueError("latent attention: the window must be positive (got %r)" % (window,))
         self.hidden_size, self.H, self.dim, self.E, self.dv = int(hidden_size), int(num_heads), int(head_dim), int(rot_dim), int(value_dim)
-        self.Rq, self.R = int(q_rank), int(kv_rank)
+        self.Rq, self.R = None if q_rank is None else int(q_rank), int(kv_rank)
         self.scale, self.eps, self.gate = float(softmax_scale), float(norm_eps), bool(gate)
         self.window, self.sink, self.own_rows = int(window) if window else 0, bool(sink), bool(own_rows)
         self.rot_dims = rot_dims
@@ -64,10 +65,11 @@ class LatentAttention(Mixer):
     def weight_specs(self):
         n, d, H = self.name, self.hidden_size, self.H
         pack = n + "down.packed"
+        Rq = FreeDim(n + "q.rank", max(1, d // 3)) if self.Rq is None else self.Rq
         specs = {
-            n + "dq": WeightSpec((self.Rq, d), pack=(pack, 0)),
-            n + "dq.norm": WeightSpec((self.Rq,), "vector"),
-            n + "uq": WeightSpec((H * (self.dim + self.E), self.Rq)),
+            n + "dq": WeightSpec((Rq, d), pack=(pack, 0)),
+            n + "dq.norm": WeightSpec((Rq,), "vector"),
+            n + "uq": WeightSpec((H * (self.dim + self.E), Rq)),
             n + "uk": WeightSpec((H * self.dim, self.R), pack=(n + "ukv.packed", 0)),
             n + "uv": WeightSpec((H * self.dv, self.R), pack=(n + "ukv.packed", 1)),
             n + "o": WeightSpec((d, H * self.dv)),
@@ -86,6 +88,7 @@ class LatentAttention(Mixer):
         self.w_down = packed_rows(tensors, n + "down.packed",
                                   [n + x for x, there in (("dq", True), ("dkv", self.own_rows), ("g", self.gate)) if there])
         self.qn_w = tensors[n + "dq.norm"]
+        self.Rq = self.qn_w.shape[0]
         if self.own_rows:
             self.kvn_w = tensors[n + "dkv.norm"]
         if self.sink:

@@ -159,6 +159,13 @@ def test_weights_and_fused_layouts(tmp_path):
     assert torch.allclose(right.rate, torch.exp(W["l1.mix.right.A_log"]))
     assert left.state_base == 0 and right.state_base == 0 and (left.out_buffer, right.out_buffer) == ("mixer_out_0", "mixer_out_1")
     assert set(model.weight_specs()) == set(W)
+    # the query latent's size may stand in the tensors alone
+    open_cfg = json.loads(json.dumps(F1))
+    for i in (0, 2, 3):
+        open_cfg["layers"][i]["mixer"].pop("q_rank")
+    other = _cpu_model(open_cfg)
+    other.load_from_dir(folder)
+    assert [other.layers[i].mixer.Rq for i in (0, 2, 3)] == [40, 24, 40] and torch.equal(other.layers[0].mixer.w_down, m.w_down)
     # an unexpected tensor is named
     from infinicore_infer_amd.weights.loader import WeightError
     from safetensors.torch import save_file
@@ -178,7 +185,7 @@ def test_who_hands_rows_on():
     assert SharedNormResidualBlock("b.", other.runtime, mixer=other, mixer_norm=model.layers[0].mixer_norm).entry_norm() is None
 
 
-@pytest.mark.parametrize("dims,base,scaling", [(32, 10000.0, (8.0, 512, 32.0, 1.0)), (64, 5e5, (40.0, 4096, 32.0, 1.0)), (6, 10.0, (2.0, 4, 3.0, 3.0)),
+@pytest.mark.parametrize("dims,base,scaling", [(48, 10000.0, (10.0, 300, 24.0, 1.0)), (64, 5e5, (40.0, 4096, 32.0, 1.0)), (6, 10.0, (2.0, 4, 3.0, 3.0)),
                                                (16, 100.0, (1.0, 64, 8.0, 1.0)), (8, 1000.0, (4.0, 1, 32.0, 16.0))])
 def test_stretched_wavelengths(dims, base, scaling):
     from infinicore_infer_amd.parts.rotary import pair_frequencies, stretched_magnitude

@@ -62,7 +62,7 @@ F2 = {"architecture": "Fokinex", "vocab": 97, "width": 70, "norm": {"eps": 1e-6}
                  _parallel((2, 1, 14, 1.0, 5.0, 3), (2, 2, 5, 3, 2), (1.0, -0.5))]}
 # F3: the tiled kernels' sizes, windows that are multiples of a page, large head sizes in the recurrence, five taps, a source
 # that keeps everything because one of its readers does.
-ROT3 = (500000.0, (16.0, 32, 4.0, 0.5))
+ROT3 = (300000.0, (16.0, 32, 4.0, 0.5))
 F3 = {"architecture": "Fokinex", "vocab": 300, "width": 128, "norm": {"eps": 1e-5}, "embedding": {"scale": 0.5},
       "layers": [_latent(4, 64, 32, 64, 64, 128, 0.1, 64, ROT3, ff=192),
                  _latent(6, 32, 32, 128, 48, 128, 0.15, None, ROT3, kv_from=0, ff=128),
@@ -590,7 +590,7 @@ def _close(got, want, tol, what):
 
 
 @pytest.mark.parametrize("dims,base,scaling", [(16, 10000.0, (4.0, 64, 8.0, 1.0)), (64, 1e6, (32.0, 4096, 32.0, 1.0)), (6, 77.0, None),
-                                               (32, 5e5, (8.0, 100, 2.0, 2.0)), (8, 100.0, (2.0, 3, 50.0, 0.01)), (2, 10.0, (3.0, 512, 32.0, 1.0))])
+                                               (24, 3e5, (6.0, 100, 2.0, 2.0)), (8, 100.0, (2.0, 3, 50.0, 0.01)), (2, 10.0, (3.0, 512, 32.0, 1.0))])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 def test_rotation_with_stretched_wavelengths(dtype, dims, base, scaling):
     """The cached row (normed latent, rotated part) and the queries' rotated parts, into another tensor and in place, at
@@ -682,7 +682,7 @@ def test_walk_over_a_window_of_latent_rows_with_sinks(R, E, Hn, page, window, dn
 
 
 @pytest.mark.parametrize("dim,E,dv,R,Hn,window,with_gate", [(24, 16, 40, 64, 3, 37, False), (64, 32, 64, 256, 4, 0, True), (128, 64, 128, 512, 2, 129, False),
-                                                            (32, 32, 80, 72, 5, 64, False), (56, 8, 96, 40, 2, 1, True), (80, 48, 128, 96, 2, 200, False),
+                                                            (40, 32, 72, 72, 5, 64, False), (56, 8, 96, 40, 2, 1, True), (80, 48, 128, 96, 2, 200, False),
                                                             (160, 32, 56, 64, 1, 63, False), (8, 8, 8, 8, 6, 5, False)])
 @pytest.mark.parametrize("n,pos0", [(2, 0), (33, 0), (300, 0), (129, 171), (64, 64), (40, 299)])
 def test_portions_over_keys_and_values_made_per_head(dim, E, dv, R, Hn, window, with_gate, n, pos0):
@@ -808,7 +808,7 @@ def test_values_that_are_the_projected_keys(dtype, mode, Hq, G, d):
         assert bias is not None or torch.equal(vc[s // page, :, s % page].cpu(), rows[t, Hq * d:(Hq + G) * d].view(G, d))
 
 
-@pytest.mark.parametrize("Hq,G,dk,dv,window,cap,page", [(4, 2, 96, 96, 33, 4.0, 16), (6, 2, 128, 128, 0, 50.0, 64), (3, 3, 40, 40, 17, 0.0, 16),
+@pytest.mark.parametrize("Hq,G,dk,dv,window,cap,page", [(6, 3, 96, 96, 33, 4.0, 16), (6, 2, 128, 128, 0, 50.0, 64), (3, 3, 40, 40, 17, 0.0, 16),
                                                         (8, 1, 64, 64, 64, 20.0, 16), (5, 5, 80, 48, 1, 3.0, 32), (2, 1, 24, 104, 100, 0.0, 16),
                                                         (2, 2, 10, 14, 20, 8.0, 16)])
 @pytest.mark.parametrize("dname,dtype,tol", DTYPES)
@@ -1091,7 +1091,7 @@ def _drawn_config(seed):
         own = not sources or rng.random() < 0.5
         if own:
             kv_rank, rot_dim = rng.choice([16, 22, 64, 96, 128]), rng.choice([2, 8, 16, 32])
-            rot = (rng.choice([100.0, 10000.0, 5e5]), rng.choice([None, (2.0, 16, 4.0, 0.5), (8.0, 128, 32.0, 1.0), (40.0, 4096, 32.0, 1.0)]))
+            rot = (rng.choice([100.0, 10000.0, 3e5]), rng.choice([None, (2.0, 16, 4.0, 0.5), (8.0, 128, 32.0, 1.0), (40.0, 4096, 32.0, 1.0)]))
             sources.append((i, kv_rank, rot_dim, rot))
         j, kv_rank, rot_dim, rot = sources[-1] if own else rng.choice(sources)
         layers.append(_latent(rng.choice([1, 2, 5, 8]), rng.choice([8, 10, 32, 64]), rot_dim, rng.choice([8, 14, 40, 64, 96]), rng.choice([8, 20, 48]),
